@@ -38,7 +38,8 @@ enum {
 };
 
 /* GGML tensor types accepted, numbered as in GGUF (src/load_gguf.jl:26-42). */
-enum { L2H_TYPE_F32 = 0, L2H_TYPE_Q4_K = 12, L2H_TYPE_Q5_K = 13, L2H_TYPE_Q6_K = 14 };
+enum { L2H_TYPE_F32 = 0, L2H_TYPE_Q4_K = 12, L2H_TYPE_Q5_K = 13, L2H_TYPE_Q6_K = 14,
+       L2H_TYPE_BF16 = 30 /* layered models only (below) */ };
 
 /* Tensor roles: the fields of TransformerWeights / TransformerLayerWeights
  * (src/inference.jl:27-48). */
@@ -182,6 +183,10 @@ int l2h_generate_greedy_timed(l2h_model *m, const int32_t *prompt, int n_prompt,
  * already be in the cache.  Decoding continues with l2h_generate_greedy(&next, 1, pos0+n, ...).
  * Needs head size 32/64/96/128, dim and hidden_dim multiples of 8, w1 and w3 of one type. */
 int l2h_prefill(l2h_model *m, const int32_t *tokens, int n, int pos0, float *last_logits, int32_t *next_token);
+/* The same pass with the logits of chosen positions: want[0..n_want) are indexes into tokens, ascending; logits receives
+ * [n_want][vocab].  n_want may be 0. */
+int l2h_prefill_logits(l2h_model *m, const int32_t *tokens, int n, int pos0, const int32_t *want, int n_want,
+                       float *logits, int32_t *next_token);
 /* The temperature branch of sample() (src/inference.jl:363-367) on the logits the last step left on
  * the device: logits ./= temperature, softmax!, then wsample's walk with the caller's uniform number
  * u in [0, 1) in place of the global RNG: token = first index whose cumulative probability reaches
@@ -243,6 +248,77 @@ int l2h_argmax(l2h_ctx *ctx, const float *x, int64_t n, int32_t *out);
  * L2H_ARGMAX_NOALLOC_MAX_N is L2H_EINVAL. */
 #define L2H_ARGMAX_NOALLOC_MAX_N ((int64_t)1 << 30)
 int l2h_argmax_noalloc(l2h_ctx *ctx, const float *x_dev, int64_t n, int32_t *out_dev);
+
+/* ---- layered models ----------------------------------------------------------------- */
+/* A decoder whose layers are described one by one.  No counterpart in the reference.  A layered model is an
+ * l2h_model like any other: tensors go in through l2h_model_set_tensor (roles below), l2h_model_finalize,
+ * l2h_state_reset, l2h_forward, l2h_generate_greedy(_timed), l2h_prefill(_logits), l2h_sample, l2h_state_read (x
+ * and logits) work on it; decode steps are a recorded launch sequence (launch path 1).  A sequence starts at position 0
+ * and its positions come in order (a call at another position is L2H_EINVAL): recurrent layers carry state.
+ * The calls that concern k-quant weights, the other launch paths, or rows of the Llama KV cache are
+ * L2H_EINVAL.
+ *
+ * With residual stream x and mult = residual_mult, a layer is
+ *   x += mult * mixer(norm1(x));  x += mult * ff(norm2(x));
+ *   with side_dim > 0:  e = the layer's slice of the token's row of the side embedding,
+ *     y = side_proj(gelu_tanh(side_gate x) * e);  x += mult * rmsnorm(y) * side_norm
+ * Mixers:
+ *   ATTENTION      q, k, v projections; rotation of interleaved pairs in the first rot_dims dimensions, frequencies
+ *                  rot_base^(-2i/rot_dims), scaled in three bands of the wavelength when rot_original > 0; qk_norm: q and k
+ *                  over their root mean square per head; softmax(scale q.k) over the last `window` positions; head_gate:
+ *                  times sigmoid(gate row . input) per head; output projection.
+ *   CHANNEL_DELTA  q, k, v through causal convolutions of `taps` and silu; q, k unit vectors (q times dim^-1/2); gated
+ *                  delta rule with beta = sigmoid(beta row . input) per head and a decay per head and key channel,
+ *                  exp(-exp(decay rate) softplus(factor_out factor_in input + decay bias)); per-head rmsnorm, times
+ *                  sigmoid(gate factors); output projection.
+ * Feed-forward: dense act(up) -> down, or the `top` of n_experts experts by sigmoid(router), the score multiplying the
+ * expert's input. */
+enum { L2H_MIX_ATTENTION = 0, L2H_MIX_CHANNEL_DELTA = 1 };
+enum { L2H_FF_NONE = 0, L2H_FF_DENSE = 1, L2H_FF_EXPERTS = 2 };
+enum { L2H_ACT_GELU_ERF = 0, L2H_ACT_RELU2 = 1, L2H_ACT_GELU_TANH = 2 };
+/* Roles shared with Llama models: TOK_EMB, RMS_FINAL, OUTPUT, RMS_ATT (norm1), RMS_FFN (norm2), WQ, WK, WV, WO, W1 (up),
+ * W2 (down).  Matrices are bf16 of any size; vectors bf16 or F32 (convolutions: ne0 = taps, ne1 = channels). */
+enum {
+    L2H_HEAD_GATE = 12,  /* (width, heads)                  */
+    L2H_BETA = 13,       /* (width, heads)                  */
+    L2H_DECAY_RATE = 14, /* (heads): log of the rate        */
+    L2H_DECAY_BIAS = 15, /* (heads * dim)                   */
+    L2H_DECAY_IN = 16,   /* (width, decay_rank)             */
+    L2H_DECAY_OUT = 17,  /* (decay_rank, heads * dim)       */
+    L2H_GATE_IN = 18,    /* (width, gate_rank)              */
+    L2H_GATE_OUT = 19,   /* (gate_rank, heads * vdim)       */
+    L2H_MIX_NORM = 20,   /* (vdim)                          */
+    L2H_CONV_Q = 21, L2H_CONV_K = 22, L2H_CONV_V = 23,
+    L2H_ROUTER = 24,     /* (width, n_experts)              */
+    L2H_EXPERT_UP = 25, L2H_EXPERT_DOWN = 26, /* through l2h_layered_set_expert */
+    L2H_SIDE_EMB = 27,   /* (n_layers * side_dim, vocab)    */
+    L2H_SIDE_GATE = 28,  /* (width, side_dim)               */
+    L2H_SIDE_PROJ = 29,  /* (side_dim, width)               */
+    L2H_SIDE_NORM = 30,  /* (width)                         */
+    L2H_N_LAYERED_ROLES = 31
+};
+typedef struct l2h_layer {
+    int32_t mixer, n_heads, n_kv_heads, dim, vdim;
+    int32_t window, rot_dims, qk_norm, head_gate;   /* attention */
+    int32_t taps, decay_rank, gate_rank;            /* channel delta */
+    int32_t ff, ff_dim, ff_act, n_experts, top;
+    float scale;                                    /* attention */
+    double rot_base, rot_factor, rot_low, rot_high, rot_original;
+} l2h_layer;
+typedef struct l2h_layered_config {
+    int32_t width, vocab_size, n_layers, seq_len, side_dim;
+    int32_t precision; /* prompt pass: 0 bf16 activations, fp32 sums; 1 fp32 throughout.  Decode steps, caches, state and
+                          everything between the products are fp32 either way. */
+    float norm_eps, residual_mult;
+} l2h_layered_config;
+int l2h_layered_create(l2h_ctx *ctx, const l2h_layered_config *cfg, const l2h_layer *layers, l2h_model **out);
+/* one expert's matrix: role L2H_EXPERT_UP (width, ff_dim) or L2H_EXPERT_DOWN (ff_dim, width) */
+int l2h_layered_set_expert(l2h_model *m, int role, int layer, int expert, int type, const void *host, int64_t ne0,
+                           int64_t ne1);
+/* For checks: with on = 1, prompt passes keep the residual stream after every layer; l2h_layered_kept copies that of one
+ * layer for the last chunk of up to 2048 positions, n = positions * width floats. */
+int l2h_layered_keep(l2h_model *m, int on);
+int l2h_layered_kept(l2h_model *m, int layer, float *host, int64_t n);
 
 /* ---- measurement -------------------------------------------------------------------- */
 /* Launches the model's matvec for `role` on every layer in turn, `iters` times over,

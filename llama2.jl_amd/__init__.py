@@ -11,7 +11,9 @@ from .inference import (DeviceModel, LanguageModel, ModelConfig, RunState, Trans
                         TransformerWeights, generate, sample, transformer_)
 from .karpathy import load_karpathy_model, save_karpathy_model  # noqa: F401
 from .kquants import QuantMatrix, dequantize, matmul, quantize_q8_K, quantize_weights  # noqa: F401
-from .tokenizer import BPETokenizer, CharTokenizer, encode  # noqa: F401
+from .layered import LayeredConfig, LayeredDevice, LayeredWeights, LayerSpec  # noqa: F401
+from .registry import ARCHITECTURES, load_model  # noqa: F401
+from .tokenizer import BPETokenizer, CharTokenizer, IdTokenizer, encode  # noqa: F401
 
 __all__ = ["ModelConfig", "CharTokenizer", "LanguageModel", "load_gguf_model", "load_karpathy_model", "encode",
            "sample"]  # the reference's exports minus `train` (src/Llama2.jl:12-14)

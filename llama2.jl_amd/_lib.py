@@ -12,9 +12,11 @@ LIB_PATH = os.environ.get("L2H_LIB") or os.path.join(HERE, "libl2hip.so")
 
 # error codes / enums of include/l2h.h
 OK, EINVAL, ETYPE, ESTATE, EHIP, ENOMEM, ENODEV = 0, -1, -2, -3, -4, -5, -6
-TYPE_F32, TYPE_Q4_K, TYPE_Q5_K, TYPE_Q6_K = 0, 12, 13, 14
+TYPE_F32, TYPE_Q4_K, TYPE_Q5_K, TYPE_Q6_K, TYPE_BF16 = 0, 12, 13, 14, 30
 (TOK_EMB, RMS_FINAL, OUTPUT, RMS_ATT, RMS_FFN, WQ, WK, WV, WO, W1, W2, W3) = range(12)
 N_ROLES = 12
+(HEAD_GATE, BETA, DECAY_RATE, DECAY_BIAS, DECAY_IN, DECAY_OUT, GATE_IN, GATE_OUT, MIX_NORM, CONV_Q, CONV_K, CONV_V, ROUTER,
+ EXPERT_UP, EXPERT_DOWN, SIDE_EMB, SIDE_GATE, SIDE_PROJ, SIDE_NORM) = range(12, 31)  # layered models
 
 
 class L2HError(RuntimeError):
@@ -63,6 +65,11 @@ SIGNATURES = {
     "l2h_generate_greedy": (_I, [_P, _P, _I, _I, _I, _P, _P]),
     "l2h_generate_greedy_timed": (_I, [_P, _P, _I, _I, _I, _P, _PF]),
     "l2h_prefill": (_I, [_P, _P, _I, _I, _P, _PI32]),
+    "l2h_prefill_logits": (_I, [_P, _P, _I, _I, _P, _I, _P, _PI32]),
+    "l2h_layered_create": (_I, [_P, _P, _P, C.POINTER(_P)]),
+    "l2h_layered_set_expert": (_I, [_P, _I, _I, _I, _I, _P, _I64, _I64]),
+    "l2h_layered_keep": (_I, [_P, _I]),
+    "l2h_layered_kept": (_I, [_P, _I, _P, _I64]),
     "l2h_sample": (_I, [_P, C.c_float, C.c_float, _PI32, _P]),
     "l2h_state_read": (_I, [_P, _I, _P, _I64]),
     "l2h_quantize_q8k": (_I, [_P, _P, _I64, _P]),

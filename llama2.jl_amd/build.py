@@ -20,7 +20,8 @@ OBJ = os.path.join(HERE, "build")
 LIB = os.path.join(HERE, "libl2hip.so")
 LIB_TIMELINE = os.path.join(HERE, "libl2hip_tl.so")
 
-SOURCES = ["api.cpp", "synth.cpp", "pf_lt.cpp", "k_misc.hip", "k_matvec.hip", "k_attn.hip", "k_mega.hip", "k_prefill.hip", "k_flow.hip"]
+SOURCES = ["api.cpp", "synth.cpp", "pf_lt.cpp", "k_misc.hip", "k_matvec.hip", "k_attn.hip", "k_mega.hip", "k_prefill.hip", "k_flow.hip",
+           "layered.cpp", "k_rows.hip", "k_delta.hip", "k_window.hip", "k_gemm.hip"]
 
 COMMON = [
     "-O3", "-fPIC", "-std=c++17", "-ffp-contract=off", "-Wall", "-Wno-unused-function",
@@ -57,7 +58,7 @@ def build(force=True, verbose=True, timeline=False):
     if not force and os.path.exists(lib) and all(os.path.getmtime(lib) >= os.path.getmtime(d) for d in deps):
         return lib
     objs = []
-    with concurrent.futures.ThreadPoolExecutor(max_workers=min(8, len(SOURCES))) as ex:
+    with concurrent.futures.ThreadPoolExecutor(max_workers=min(16, len(SOURCES))) as ex:
         for src, rc, out, obj in ex.map(lambda s: _compile(s, extra, objdir), SOURCES):
             text = "\n".join(l for l in out.splitlines() if "packed-fp32-ops" not in l)
             if rc != 0:

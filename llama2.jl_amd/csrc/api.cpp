@@ -12,19 +12,12 @@
 #include <string>
 #include <vector>
 
-#include "l2h_internal.h"
+#include "model.h"
 
 // ------------------------------------------------------------------------------------------
-struct l2h_ctx {
-    int device = 0;
-    hipStream_t stream = nullptr;
-    std::string err;
-    hipDeviceProp_t prop;
-};
-
 static std::string g_create_err;
 
-static int set_err(l2h_ctx *ctx, int code, const char *fmt, ...) {
+int set_err(l2h_ctx *ctx, int code, const char *fmt, ...) {
     char buf[512];
     va_list ap;
     va_start(ap, fmt);
@@ -37,14 +30,6 @@ static int set_err(l2h_ctx *ctx, int code, const char *fmt, ...) {
     return code;
 }
 
-#define HIPCHK(ctx, call)                                                                          \
-    do {                                                                                           \
-        hipError_t e_ = (call);                                                                    \
-        if (e_ != hipSuccess)                                                                      \
-            return set_err((ctx), L2H_EHIP, "%s:%d: %s failed: %s", __FILE__, __LINE__, #call,     \
-                           hipGetErrorString(e_));                                                 \
-    } while (0)
-
 static bool is_kquant(int type) {
     return type == L2H_TYPE_Q4_K || type == L2H_TYPE_Q5_K || type == L2H_TYPE_Q6_K;
 }
@@ -52,8 +37,6 @@ static bool type_ok(int type) { return type == L2H_TYPE_F32 || is_kquant(type); 
 // longest input vector of a k-quant matvec: the activation staging of the kernels holds
 // STAGE_MAX_ROUNDS (4) q8_K blocks per wavefront, 16 wavefronts
 #define L2H_MAX_KQ_INPUT 16384
-
-static int64_t align256(int64_t v) { return (v + 255) & ~(int64_t)255; }
 
 // Lays out the field streams of a tensor inside one allocation (see DevTensor).
 static int dev_tensor_alloc(l2h_ctx *ctx, int type, int64_t ne0, int64_t ne1, DevTensor *t) {
@@ -199,77 +182,8 @@ extern "C" int l2h_device_info(l2h_ctx *ctx, char *name, int name_cap, int32_t *
 // ------------------------------------------------------------------------------------------
 // model
 // ------------------------------------------------------------------------------------------
-struct l2h_model;
 static l2h_model *g_bound_model = nullptr;  // whose phase arguments the persistent kernel's constant memory holds
 static l2h_model *g_flow_bound = nullptr;   // whose arguments the streaming kernel's constant memory holds
-
-struct l2h_model {
-    l2h_ctx *ctx = nullptr;
-    l2h_config c{};
-    int hs = 0, kv_dim = 0;
-    float theta_scale = 0.0f;
-    DevTensor glob[3];
-    std::vector<DevTensor> layer;  // [n_layers][L2H_N_ROLES]
-    bool finalized = false;
-    // RunState (reference src/inference.jl:72-100) in device memory
-    float *x = nullptr, *xb = nullptr, *xb2 = nullptr, *hb = nullptr, *hb2 = nullptr, *q = nullptr, *k = nullptr,
-          *v = nullptr, *att = nullptr, *logits = nullptr;
-    double *qd = nullptr, *pd = nullptr, *part = nullptr;
-    float *rope_cs = nullptr;  // cos/sin of the current position's RoPE angles, [hs/2][2]
-    float *kc = nullptr, *vc = nullptr;  // [n_layers] x per-layer cache
-    int64_t cache_layer_elems = 0;
-    DecodeCtl *ctl = nullptr;
-    int32_t *prompt_dev = nullptr, *out_tokens = nullptr;
-    int64_t *argmax_partial = nullptr;
-    int max_out = 0;
-    hipGraph_t graph = nullptr;
-    hipGraphExec_t exec = nullptr;
-    // persistent decode kernel
-    int kv16 = 0;          // 1: the KV cache holds fp16 elements (l2h_model_set_kv_type)
-    bool kv_uncached = false;       // the KV cache lives in uncached memory (see l2h_model_finalize)
-    int flow_steps_per_launch = 1;  // steps of the token loop per launch of the streaming kernel
-    int path_request = 0;  // 0 auto, 1 one kernel per phase, 2 persistent kernel, 3 streaming kernel (2, 3: required)
-    bool mega = false;
-    PhaseArgs mega_ph[5];  // q/k/v, wo, w1+w3, w2 of layer 0 and the classifier, planned for the persistent grid
-    GridBar *bar = nullptr;
-    unsigned long long bar_gen = 0;
-    int mega_grid = 0;
-    size_t mega_lds = 0;
-    int mega_types[5] = {0, 0, 0, 0, 0};
-#ifdef L2H_TIMELINE
-    long long *timeline = nullptr, *timeline2 = nullptr;
-#endif
-    float *sample_p = nullptr;  // probabilities of the last l2h_sample call
-    int32_t *sample_out = nullptr;
-    // streaming decode kernel
-    bool flow = false;
-    FlowArgs flow_args{};
-    int flow_grid = 0, flow_cls_type = 0;
-    std::string flow_why;  // why the streaming kernel was not chosen (empty if it was, or if it was not asked for)
-    unsigned int flow_gen = 1;  // epoch of the next launch's input; 0 is what cleared memory holds
-    // batched prompt pass: buffers for pf_cap positions, allocated at the first l2h_prefill
-    int pf_cap = 0;
-    float *pf_x = nullptr, *pf_raw = nullptr, *pf_cs = nullptr;
-    uint16_t *pf_xn = nullptr, *pf_q = nullptr, *pf_att = nullptr, *pf_hb = nullptr;
-    int32_t *pf_tok = nullptr;
-    unsigned char *pf_kvt = nullptr;  // one layer's K / V^T as bf16 tiles of 32 keys (k_pf_kv_tiles)
-    int pf_kvt_tiles = 0;             // tiles per KV head
-    // bf16 copy of the layer matrices for the prompt pass: per layer q|k|v rows, wo, w1/w3 rows in turn, w2
-    int pf_copy_mode = 1;          // 0 never, 1 when it fits
-    bool pf_copy_tried = false;
-    uint16_t *pf_wbf = nullptr;
-    // the plain products of the prompt pass (q | k | v, wo, w2) through hipBLASLt: asked for (default) / opened / the
-    // layout the copy's three matrices have now (plain rows for the library, tiles for the own kernels)
-    int pf_library_mode = 1;
-    PfLt *pf_lt = nullptr;
-    bool pf_lt_tried = false, pf_plain = false;
-    std::string pf_lt_why, pf_lt_err;
-    int64_t pf_wbf_layer = 0, pf_off_wo = 0, pf_off_w13 = 0, pf_off_w2 = 0;  // elements
-    std::vector<void *> allocs;
-    std::vector<void *> uc_allocs;  // blocks of the uncached pool (uncached_alloc), handed back with the model
-
-    DevTensor &L(int layer_idx, int role) { return layer[(size_t)layer_idx * L2H_N_ROLES + role]; }
-};
 
 static int q8_alloc(l2h_ctx *ctx, int64_t n, Q8Dev *q, std::vector<void *> *track) {
     void *p = nullptr;
@@ -337,6 +251,7 @@ extern "C" void l2h_model_destroy(l2h_model *m) {
     model_free_state(m);
     for (auto &t : m->glob) dev_tensor_free(&t);
     for (auto &t : m->layer) dev_tensor_free(&t);
+    if (m->lay) layered_free(m);
     delete m;
 }
 
@@ -350,6 +265,7 @@ extern "C" int l2h_model_set_tensor(l2h_model *m, int role, int layer, int type,
                                     int64_t ne1) {
     if (!m || !host) return set_err(m ? m->ctx : nullptr, L2H_EINVAL, "l2h_model_set_tensor: NULL argument");
     l2h_ctx *ctx = m->ctx;
+    if (m->lay) return layered_set_tensor(m, role, layer, 0, type, host, ne0, ne1);
     if (m->finalized) return set_err(ctx, L2H_ESTATE, "model already finalized");
     if (role < 0 || role >= L2H_N_ROLES) return set_err(ctx, L2H_EINVAL, "role %d out of range", role);
     if (!type_ok(type)) return set_err(ctx, L2H_ETYPE, "tensor type %d not implemented", type);
@@ -391,8 +307,23 @@ extern "C" int l2h_model_set_tensor(l2h_model *m, int role, int layer, int type,
     return rc;
 }
 
+extern "C" int l2h_layered_set_expert(l2h_model *m, int role, int layer, int expert, int type, const void *host, int64_t ne0,
+                                      int64_t ne1) {
+    if (!m || !host) return set_err(m ? m->ctx : nullptr, L2H_EINVAL, "l2h_layered_set_expert: NULL argument");
+    if (!m->lay || (role != L2H_EXPERT_UP && role != L2H_EXPERT_DOWN))
+        return set_err(m->ctx, L2H_EINVAL, "l2h_layered_set_expert takes an expert matrix of a layered model");
+    return layered_set_tensor(m, role, layer, expert, type, host, ne0, ne1);
+}
+
+// calls that concern only the Llama models' weights, cache or launch paths
+#define LLAMA_ONLY(m)                                                                                        \
+    do {                                                                                                     \
+        if ((m)->lay) return set_err((m)->ctx, L2H_EINVAL, "%s: not available for a layered model", __func__); \
+    } while (0)
+
 extern "C" int l2h_model_set_wait_limit(l2h_model *m, unsigned int spins) {
     if (!m) return L2H_EINVAL;
+    LLAMA_ONLY(m);
     if (!m->flow) return set_err(m->ctx, L2H_ESTATE, "the wait limit applies to launch path 3 after finalize");
     m->flow_args.spin_limit = spins;
     if (g_flow_bound == m) g_flow_bound = nullptr;  // the kernel's copy of the arguments is refreshed at the next launch
@@ -417,6 +348,7 @@ extern "C" int l2h_model_prefill_library(l2h_model *m) { return (m && m->pf_wbf 
 
 extern "C" int l2h_model_set_kv_type(l2h_model *m, int kv_type) {
     if (!m) return L2H_EINVAL;
+    LLAMA_ONLY(m);
     if (m->finalized) return set_err(m->ctx, L2H_ESTATE, "model already finalized");
     if (kv_type != L2H_KV_F32 && kv_type != L2H_KV_F16) return set_err(m->ctx, L2H_EINVAL, "kv_type must be L2H_KV_F32 or L2H_KV_F16");
     m->kv16 = kv_type == L2H_KV_F16;
@@ -426,6 +358,7 @@ extern "C" int l2h_model_set_kv_type(l2h_model *m, int kv_type) {
 extern "C" int l2h_model_set_path(l2h_model *m, int path) {
     if (!m) return L2H_EINVAL;
     if (m->finalized) return set_err(m->ctx, L2H_ESTATE, "model already finalized");
+    if (m->lay && path > 1) return set_err(m->ctx, L2H_EINVAL, "a layered model decodes on launch path 1");
     if (path < 0 || path > 3) return set_err(m->ctx, L2H_EINVAL, "path must be 0, 1, 2 or 3");
     m->path_request = path;
     return L2H_OK;
@@ -441,6 +374,7 @@ extern "C" int l2h_model_path(l2h_model *m) { return (m && m->finalized) ? (m->f
 
 extern "C" int l2h_model_get_tensor(l2h_model *m, int role, int layer, void *host, int64_t host_bytes) {
     if (!m || !host) return set_err(m ? m->ctx : nullptr, L2H_EINVAL, "l2h_model_get_tensor: NULL argument");
+    LLAMA_ONLY(m);
     if (role < 0 || role >= L2H_N_ROLES || (role >= 3 && (layer < 0 || layer >= m->c.n_layers)))
         return set_err(m->ctx, L2H_EINVAL, "role/layer out of range");
     DevTensor &t = role < 3 ? m->glob[role] : m->L(layer, role);
@@ -490,17 +424,6 @@ static void uncached_release(void *p) {
     std::lock_guard<std::mutex> lock(g_uc_mu);
     for (UncachedBlock &b : g_uc_blocks)
         if (b.p == p) b.used = false;
-}
-
-template <class T>
-static int dalloc(l2h_model *m, T **p, int64_t n, bool zero) {
-    void *v = nullptr;
-    const size_t bytes = (size_t)std::max<int64_t>(n, 1) * sizeof(T);
-    HIPCHK(m->ctx, hipMalloc(&v, bytes));
-    m->allocs.push_back(v);
-    if (zero) HIPCHK(m->ctx, hipMemset(v, 0, bytes));
-    *p = (T *)v;
-    return L2H_OK;
 }
 
 // the caches of layer l (fp32 or fp16 elements: addressed in bytes)
@@ -949,6 +872,10 @@ static hipError_t enqueue_token(l2h_model *m) {
         e = (call);                    \
         if (e != hipSuccess) return e; \
     } while (0)
+    if (m->lay) {
+        CK(layered_enqueue_token(m));
+        return k_argmax(s, m->logits, c.vocab_size, m->argmax_partial, m->ctl, m->out_tokens, m->max_out);
+    }
     // token embedding (:236) and this position's RoPE table
     CK(k_embed(s, m->glob[L2H_TOK_EMB], m->ctl, m->prompt_dev, m->x, m->rope_cs, m->hs, m->theta_scale));
     for (int l = 0; l < c.n_layers; l++) {
@@ -990,11 +917,35 @@ static int record_token(l2h_model *m) {
     return L2H_OK;
 }
 
+// what the token loop itself needs
+static int loop_buffers(l2h_model *m) {
+    int rc;
+#define DA(p, n, z)                       \
+    if ((rc = dalloc(m, &(p), (n), (z)))) \
+        return rc;
+    DA(m->ctl, 1, true);
+    DA(m->prompt_dev, m->c.seq_len, true);
+    m->max_out = m->c.seq_len;
+    DA(m->out_tokens, m->max_out, true);
+    DA(m->argmax_partial, std::max(L2H_ARGMAX_BLOCKS, m->ctx->prop.multiProcessorCount), true);
+#undef DA
+    return L2H_OK;
+}
+
 extern "C" int l2h_model_finalize(l2h_model *m) {
     if (!m) return L2H_EINVAL;
     l2h_ctx *ctx = m->ctx;
     if (m->finalized) return set_err(ctx, L2H_ESTATE, "model already finalized");
     const l2h_config &c = m->c;
+    if (m->lay) {
+        HIPCHK(ctx, hipSetDevice(ctx->device));
+        int rc;
+        if ((rc = layered_finalize(m)) || (rc = loop_buffers(m))) return rc;
+        HIPCHK(ctx, hipDeviceSynchronize());
+        if ((rc = record_token(m))) return rc;
+        m->finalized = true;
+        return L2H_OK;
+    }
     for (int r = 0; r < 3; r++)
         if (!m->glob[r].base) return set_err(ctx, L2H_ESTATE, "missing tensor %s", role_name(r));
     for (int l = 0; l < c.n_layers; l++)
@@ -1051,12 +1002,8 @@ extern "C" int l2h_model_finalize(l2h_model *m) {
             DA(m->vc, n, true);
         }
     }
-    DA(m->ctl, 1, true);
-    DA(m->prompt_dev, c.seq_len, true);
-    m->max_out = c.seq_len;
-    DA(m->out_tokens, m->max_out, true);
-    DA(m->argmax_partial, std::max(L2H_ARGMAX_BLOCKS, ctx->prop.multiProcessorCount), true);
 #undef DA
+    if ((rc = loop_buffers(m))) return rc;
     HIPCHK(ctx, hipDeviceSynchronize());
     if ((rc = mega_setup(m))) return rc;
     if ((rc = flow_setup(m))) return rc;
@@ -1127,6 +1074,7 @@ static int mega_check(l2h_model *m) {
 extern "C" int l2h_state_reset(l2h_model *m) {
     if (!m) return L2H_EINVAL;
     if (!m->finalized) return set_err(m->ctx, L2H_ESTATE, "model not finalized");
+    if (m->lay) return layered_reset(m);
     const size_t bytes = (size_t)m->cache_layer_elems * m->c.n_layers * (m->kv16 ? 2 : 4);
     HIPCHK(m->ctx, hipMemsetAsync(m->kc, 0, bytes, m->ctx->stream));
     HIPCHK(m->ctx, hipMemsetAsync(m->vc, 0, bytes, m->ctx->stream));
@@ -1136,6 +1084,7 @@ extern "C" int l2h_state_reset(l2h_model *m) {
 
 static int kv_xfer(l2h_model *m, int layer, int pos0, int n, float *k, float *v, bool to_cache) {
     if (!m) return L2H_EINVAL;
+    LLAMA_ONLY(m);
     l2h_ctx *ctx = m->ctx;
     if (!m->finalized) return set_err(ctx, L2H_ESTATE, "model not finalized");
     if (layer < 0 || layer >= m->c.n_layers || pos0 < 0 || n < 0 || pos0 + n > m->c.seq_len || !k || !v)
@@ -1185,6 +1134,8 @@ static int generate_impl(l2h_model *m, const int32_t *prompt, int n_prompt, int 
     for (int i = 0; i < n_prompt; i++)
         if (prompt[i] < 0 || prompt[i] >= m->c.vocab_size)
             return set_err(ctx, L2H_EINVAL, "prompt[%d] = %d outside vocabulary", i, prompt[i]);
+    int rc;
+    if (m->lay && (rc = layered_check_pos(m, pos0))) return rc;
     HIPCHK(ctx, hipSetDevice(ctx->device));
     DecodeCtl h{};
     h.token = prompt[0];
@@ -1196,7 +1147,7 @@ static int generate_impl(l2h_model *m, const int32_t *prompt, int n_prompt, int 
     HIPCHK(ctx, hipMemcpyAsync(m->prompt_dev, prompt, (size_t)n_prompt * 4, hipMemcpyHostToDevice, ctx->stream));
     HIPCHK(ctx, hipMemcpyAsync(m->ctl, &h, sizeof h, hipMemcpyHostToDevice, ctx->stream));
     HIPCHK(ctx, hipStreamSynchronize(ctx->stream));
-    int rc;
+    if (m->lay && total > 0) layered_advance(m, pos0 + total);
     if (decode_ms) {
         hipEvent_t e0 = nullptr, e1 = nullptr;
         HIPCHK(ctx, hipEventCreate(&e0));
@@ -1374,8 +1325,9 @@ static hipError_t prefill_chunk(l2h_model *m, int M, int pos0) {
     return hipSuccess;
 }
 
-extern "C" int l2h_prefill(l2h_model *m, const int32_t *tokens, int n, int pos0, float *last_logits,
-                           int32_t *next_token) {
+// want[0..n_want): positions (indexes into tokens) whose logits go to want_logits
+static int prefill_impl(l2h_model *m, const int32_t *tokens, int n, int pos0, const int32_t *want, int n_want, float *want_logits,
+                        float *last_logits, int32_t *next_token) {
     if (!m) return L2H_EINVAL;
     l2h_ctx *ctx = m->ctx;
     if (!m->finalized) return set_err(ctx, L2H_ESTATE, "model not finalized");
@@ -1385,21 +1337,42 @@ extern "C" int l2h_prefill(l2h_model *m, const int32_t *tokens, int n, int pos0,
     for (int i = 0; i < n; i++)
         if (tokens[i] < 0 || tokens[i] >= m->c.vocab_size)
             return set_err(ctx, L2H_EINVAL, "tokens[%d] = %d outside vocabulary", i, tokens[i]);
+    for (int i = 0; i < n_want; i++)
+        if (want[i] < 0 || want[i] >= n || (i && want[i] <= want[i - 1]))
+            return set_err(ctx, L2H_EINVAL, "want[%d] = %d: indexes into the tokens, in ascending order", i, want[i]);
     if (m->kv16) return set_err(ctx, L2H_ESTATE, "the batched prompt pass writes an fp32 cache only (this model's is fp16)");
-    if (!k_pf_attention_supported(m->hs))
+    if (!m->lay && !k_pf_attention_supported(m->hs))
         return set_err(ctx, L2H_EINVAL, "batched prompt pass needs a head size of 32, 64, 96 or 128 (have %d)", m->hs);
-    if (m->c.dim % 8 != 0 || m->c.hidden_dim % 8 != 0)
+    if (!m->lay && (m->c.dim % 8 != 0 || m->c.hidden_dim % 8 != 0))
         return set_err(ctx, L2H_EINVAL, "batched prompt pass needs dim and hidden_dim to be multiples of 8");
-    for (int l = 0; l < m->c.n_layers; l++)
+    for (int l = 0; l < m->c.n_layers && !m->lay; l++)
         if (m->L(l, L2H_W1).type != m->L(l, L2H_W3).type)
             return set_err(ctx, L2H_EINVAL, "batched prompt pass needs w1 and w3 of one type (layer %d)", l);
     HIPCHK(ctx, hipSetDevice(ctx->device));
     int rc;
-    if ((rc = prefill_buffers(m, std::min(n, L2H_PREFILL_CHUNK)))) return rc;
-    if (m->pf_copy_mode && (rc = prefill_weights(m))) return rc;
-    int M = 0;
+    if (m->lay) {
+        if ((rc = layered_check_pos(m, pos0)) || (rc = layered_prefill_buffers(m, std::min(n, L2H_PREFILL_CHUNK), n_want))) return rc;
+    } else {
+        if ((rc = prefill_buffers(m, std::min(n, L2H_PREFILL_CHUNK)))) return rc;
+        if (m->pf_copy_mode && (rc = prefill_weights(m))) return rc;
+    }
+    int M = 0, w0 = 0;
+    std::vector<int32_t> rows;
     for (int c0 = 0; c0 < n; c0 += M) {
-        M = std::min(m->pf_cap, n - c0);
+        M = std::min(m->lay ? layered_capacity(m) : m->pf_cap, n - c0);
+        // the wanted positions of this chunk
+        rows.clear();
+        while (w0 + (int)rows.size() < n_want && want[w0 + rows.size()] < c0 + M) rows.push_back(want[w0 + rows.size()] - c0);
+        float *wl = want_logits ? want_logits + (int64_t)w0 * m->c.vocab_size : nullptr;
+        w0 += (int)rows.size();
+        if (m->lay) {
+            HIPCHK(ctx, hipMemcpyAsync(layered_token_buffer(m), tokens + c0, (size_t)M * 4, hipMemcpyHostToDevice, ctx->stream));
+            const hipError_t e = layered_prefill_chunk(m, M, pos0 + c0);
+            if (e != hipSuccess) return set_err(ctx, L2H_EHIP, "prompt pass launch failed: %s", hipGetErrorString(e));
+            layered_advance(m, pos0 + c0 + M);
+            if (!rows.empty() && (rc = layered_prefill_logits(m, rows.data(), (int)rows.size(), wl))) return rc;
+            continue;
+        }
         if (m->pf_wbf && m->pf_copy_mode && m->pf_plain) {
             // The library must have an algorithm for this chunk's three products before anything is computed with it
             // (it may be installed without the kernels for this device): where it has none, the own kernels take over
@@ -1424,16 +1397,27 @@ extern "C" int l2h_prefill(l2h_model *m, const int32_t *tokens, int n, int pos0,
         if (e != hipSuccess)
             return set_err(ctx, L2H_EHIP, "prompt pass launch failed: %s%s%s", hipGetErrorString(e),
                            m->pf_lt_err.empty() ? "" : "; ", m->pf_lt_err.c_str());
+        for (size_t i = 0; i < rows.size(); i++) {
+            HIPCHK(ctx, hipMemcpyAsync(m->x, m->pf_x + (int64_t)rows[i] * m->c.dim, (size_t)m->c.dim * 4, hipMemcpyDeviceToDevice, ctx->stream));
+            const hipError_t el = launch_output(m);
+            if (el != hipSuccess) return set_err(ctx, L2H_EHIP, "classifier launch failed: %s", hipGetErrorString(el));
+            HIPCHK(ctx, hipMemcpyAsync(wl + (int64_t)i * m->c.vocab_size, m->logits, (size_t)m->c.vocab_size * 4, hipMemcpyDeviceToHost, ctx->stream));
+        }
+    }
+    if (!last_logits && !next_token) {
+        HIPCHK(ctx, hipStreamSynchronize(ctx->stream));
+        return L2H_OK;
     }
     // last position: its hidden state becomes the decode state; classifier and argmax as in a decode step
-    HIPCHK(ctx, hipMemcpyAsync(m->x, m->pf_x + (int64_t)(M - 1) * m->c.dim, (size_t)m->c.dim * 4,
-                               hipMemcpyDeviceToDevice, ctx->stream));
+    if (!m->lay)
+        HIPCHK(ctx, hipMemcpyAsync(m->x, m->pf_x + (int64_t)(M - 1) * m->c.dim, (size_t)m->c.dim * 4,
+                                   hipMemcpyDeviceToDevice, ctx->stream));
     DecodeCtl h{};
     h.token = tokens[n - 1];
     h.pos = pos0 + n - 1;
     h.n_prompt = 1;
     HIPCHK(ctx, hipMemcpyAsync(m->ctl, &h, sizeof h, hipMemcpyHostToDevice, ctx->stream));
-    hipError_t e = launch_output(m);
+    hipError_t e = m->lay ? layered_output(m) : launch_output(m);
     if (e == hipSuccess)
         e = k_argmax(ctx->stream, m->logits, m->c.vocab_size, m->argmax_partial, m->ctl, m->out_tokens, m->max_out);
     if (e != hipSuccess) return set_err(ctx, L2H_EHIP, "classifier launch failed: %s", hipGetErrorString(e));
@@ -1444,6 +1428,16 @@ extern "C" int l2h_prefill(l2h_model *m, const int32_t *tokens, int n, int pos0,
                                    ctx->stream));
     HIPCHK(ctx, hipStreamSynchronize(ctx->stream));
     return L2H_OK;
+}
+
+extern "C" int l2h_prefill(l2h_model *m, const int32_t *tokens, int n, int pos0, float *last_logits, int32_t *next_token) {
+    return prefill_impl(m, tokens, n, pos0, nullptr, 0, nullptr, last_logits, next_token);
+}
+
+extern "C" int l2h_prefill_logits(l2h_model *m, const int32_t *tokens, int n, int pos0, const int32_t *want, int n_want,
+                                  float *logits, int32_t *next_token) {
+    if (m && (n_want < 0 || (n_want > 0 && (!want || !logits)))) return set_err(m->ctx, L2H_EINVAL, "l2h_prefill_logits: NULL argument");
+    return prefill_impl(m, tokens, n, pos0, want, n_want, logits, nullptr, next_token);
 }
 
 extern "C" int l2h_generate_greedy(l2h_model *m, const int32_t *prompt, int n_prompt, int pos0, int n_new,
@@ -1487,6 +1481,7 @@ extern "C" int l2h_sample(l2h_model *m, float temperature, float u, int32_t *tok
 extern "C" int l2h_state_read(l2h_model *m, int which, float *host, int64_t n) {
     if (!m || !host) return L2H_EINVAL;
     if (!m->finalized) return set_err(m->ctx, L2H_ESTATE, "model not finalized");
+    if (m->lay && which != 0 && which != 6) return set_err(m->ctx, L2H_EINVAL, "a layered model has the buffers x (0) and logits (6)");
     const float *src = nullptr;
     int64_t len = 0;
     switch (which) {
@@ -1653,6 +1648,7 @@ extern "C" int l2h_matmul(l2h_ctx *ctx, int type, const void *A, int64_t ne0, in
 // matmul!(y, A, x) with A one of the model's resident matrices (uploaded through l2h_model_set_tensor)
 extern "C" int l2h_model_matmul(l2h_model *m, int role, int layer, const float *x, float *y) {
     if (!m || !x || !y) return set_err(m ? m->ctx : nullptr, L2H_EINVAL, "l2h_model_matmul: NULL argument");
+    LLAMA_ONLY(m);
     l2h_ctx *ctx = m->ctx;
     if (!m->finalized) return set_err(ctx, L2H_ESTATE, "model not finalized");
     const bool glob = role == L2H_TOK_EMB || role == L2H_OUTPUT;
@@ -1840,6 +1836,7 @@ extern "C" int l2h_argmax_noalloc(l2h_ctx *ctx, const float *x_dev, int64_t n, i
 // ------------------------------------------------------------------------------------------
 extern "C" int l2h_profile_matvec(l2h_model *m, int role, int iters, float *avg_us, int64_t *bytes) {
     if (!m || !avg_us) return L2H_EINVAL;
+    LLAMA_ONLY(m);
     l2h_ctx *ctx = m->ctx;
     if (!m->finalized) return set_err(ctx, L2H_ESTATE, "model not finalized");
     if (iters < 1) return set_err(ctx, L2H_EINVAL, "iters must be >= 1");

@@ -84,6 +84,7 @@ __device__ __forceinline__ void kq_scale_min(const uint4 hdr, int s, int &sc, in
 // expressions (src/kquants.jl:93,97 q4_K; :213,217 q5_K; :340-343 q6_K).
 __device__ __forceinline__ float dequant_elem(const DevTensor &t, int64_t row, int64_t e) {
     if (t.type == L2H_TYPE_F32) return t.f32[row * t.ne0 + e];
+    if (t.type == L2H_TYPE_BF16) return __uint_as_float((uint32_t)((const uint16_t *)t.qs)[row * t.ne0 + e] << 16);
     const int64_t blk = row * t.nb + (e >> 8);
     const int r = (int)(e & 255);
     if (t.type == L2H_TYPE_Q4_K || t.type == L2H_TYPE_Q5_K) {

@@ -1,0 +1,417 @@
+// Gated delta rule with one decay per head and key channel.  Per head, with state S [D][V] (fp32), unit vectors q and k,
+// decay g [D], step size beta:
+//   S <- diag(g) S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q = (decayed S)^T q + (k . q) u
+// so both products of a token are taken of the decayed state, before its own write.
+// The value columns of S are independent of one another: workgroups split them.
+#include "layered_dev.h"
+
+// ---------------------------------------------------------------------------------------------------------------
+// one token: workgroup (split, head), 32 value columns x 8 groups of key channels
+// ---------------------------------------------------------------------------------------------------------------
+__device__ __forceinline__ float delta_conv(const DeltaShape &d, const float *conv, const float *ring, float cur, int ch, int pos) {
+    const float *w = conv + (int64_t)ch * d.taps;
+    const int C = d.channels();
+    float v = w[d.taps - 1] * cur;
+    for (int j = 1; j < d.taps && j <= pos; j++) v = fmaf(w[d.taps - 1 - j], ring[(int64_t)((pos - j) % d.taps) * C + ch], v);
+    return l_silu(v);
+}
+
+// dot of a bf16 row (zero-padded to ld) with a vector in LDS of ld floats, by 8 lanes; every one of them gets the sum
+__device__ __forceinline__ float delta_dot8(const uint16_t *w, const float *x, int ld, int l8) {
+    float acc = 0.0f;
+    for (int k = 8 * l8; k < ld; k += 64) {
+        const uint4 p = *(const uint4 *)(w + k);
+        const float4 a = *(const float4 *)(x + k), b = *(const float4 *)(x + k + 4);
+        acc = fmaf(l_bf16_lo(p.x), a.x, acc);
+        acc = fmaf(l_bf16_hi(p.x), a.y, acc);
+        acc = fmaf(l_bf16_lo(p.y), a.z, acc);
+        acc = fmaf(l_bf16_hi(p.y), a.w, acc);
+        acc = fmaf(l_bf16_lo(p.z), b.x, acc);
+        acc = fmaf(l_bf16_hi(p.z), b.y, acc);
+        acc = fmaf(l_bf16_lo(p.w), b.z, acc);
+        acc = fmaf(l_bf16_hi(p.w), b.w, acc);
+    }
+#pragma unroll
+    for (int m = 4; m >= 1; m >>= 1) acc += __shfl_xor(acc, m, WAVE);
+    return acc;
+}
+
+// NR: rows of S per thread (D <= 8 NR)
+template <int NR>
+__global__ __launch_bounds__(256) void delta_step_kernel(DeltaShape d, DeltaWeights w, const float *in, float *ring, float *state,
+                                                         const DecodeCtl *ctl, float *o, float *ssq, float *gate, int n_split) {
+    extern __shared__ __align__(16) float s_mem[];
+    float *s_q = s_mem, *s_k = s_q + 8 * NR, *s_g = s_k + 8 * NR, *s_fa = s_g + 8 * NR, *s_fg = s_fa + w.lda2;
+    __shared__ float s_v[L_DELTA_COLS], s_red[2][8][L_DELTA_COLS], s_kq;
+    const int t = threadIdx.x, lane = t & 63, wave = t >> 6;
+    const int sp = blockIdx.x, h = blockIdx.y, kvh = h / (d.H / d.G), pos = ctl->pos;
+    const int D = d.D, V = d.V, c0 = sp * L_DELTA_COLS, GD = d.G * D;
+    const int col = t & 31, rg = t >> 5, c = c0 + col;
+    const bool live = c < V;
+    float *S = state + (int64_t)h * D * V;
+    float s[NR];
+#pragma unroll
+    for (int i = 0; i < NR; i++) {
+        const int r = rg + 8 * i;
+        s[i] = (live && r < D && pos > 0) ? S[(int64_t)r * V + c] : 0.0f;
+    }
+    // short convolutions; the token's own projections go into the ring (its slot is not read by this token)
+    const int C = d.channels();
+    float *slot = ring + (int64_t)(pos % d.taps) * C;
+    for (int i = t; i < 2 * D + L_DELTA_COLS; i += 256) {
+        int ch;
+        float *dst;
+        bool own;
+        if (i < 2 * D) {
+            const bool isk = i >= D;
+            const int e = isk ? i - D : i;
+            ch = (isk ? GD : 0) + kvh * D + e;
+            dst = (isk ? s_k : s_q) + e;
+            own = sp == 0 && h % (d.H / d.G) == 0;
+        } else {
+            const int e = i - 2 * D;
+            if (c0 + e >= V) {
+                s_v[e] = 0.0f;
+                continue;
+            }
+            ch = 2 * GD + h * V + c0 + e;
+            dst = s_v + e;
+            own = true;
+        }
+        const float cur = in[ch];
+        *dst = delta_conv(d, w.conv, ring, cur, ch, pos);
+        if (own) slot[ch] = cur;
+    }
+    for (int i = t; i < w.lda2; i += 256) s_fa[i] = i < d.ra ? in[d.off_a() + i] : 0.0f;
+    for (int i = t; i < w.ldg2; i += 256) s_fg[i] = i < d.rg ? in[d.off_g() + i] : 0.0f;
+    __syncthreads();
+    // unit vectors (one wavefront each), then k . q
+    if (wave < 2) {
+        float *x = wave ? s_k : s_q;
+        float ss = 0.0f;
+        for (int e = lane; e < D; e += 64) ss = fmaf(x[e], x[e], ss);
+        float r = 1.0f / sqrtf(l_wave_sum(ss) + 1e-6f);
+        if (wave == 0) r *= 1.0f / sqrtf((float)D);
+        for (int e = lane; e < D; e += 64) x[e] *= r;
+    }
+    // decays of all key channels, gates of this workgroup's columns
+    const int l8 = t & 7, r8 = t >> 3;
+    for (int r = r8; r < D; r += 32) {
+        const float z = delta_dot8(w.a2 + ((int64_t)h * D + r) * w.lda2, s_fa, w.lda2, l8) + w.bias[h * D + r];
+        if (l8 == 0) s_g[r] = expf(-w.rate[h] * l_softplus(z));
+    }
+    if (c0 + r8 < V) {
+        const float z = delta_dot8(w.g2 + ((int64_t)h * V + c0 + r8) * w.ldg2, s_fg, w.ldg2, l8);
+        if (l8 == 0) gate[h * V + c0 + r8] = l_sigmoid(z);
+    }
+    __syncthreads();
+    if (wave == 0) {
+        float kq = 0.0f;
+        for (int e = lane; e < D; e += 64) kq = fmaf(s_k[e], s_q[e], kq);
+        kq = l_wave_sum(kq);
+        if (lane == 0) s_kq = kq;
+    }
+    float dk = 0.0f, dq = 0.0f;
+#pragma unroll
+    for (int i = 0; i < NR; i++) {
+        const int r = rg + 8 * i;
+        if (r < D) {
+            s[i] *= s_g[r];
+            dk = fmaf(s[i], s_k[r], dk);
+            dq = fmaf(s[i], s_q[r], dq);
+        }
+    }
+    s_red[0][rg][col] = dk;
+    s_red[1][rg][col] = dq;
+    __syncthreads();
+    dk = dq = 0.0f;
+#pragma unroll
+    for (int i = 0; i < 8; i++) {
+        dk += s_red[0][i][col];
+        dq += s_red[1][i][col];
+    }
+    const float beta = l_sigmoid(in[d.off_b() + h]);
+    const float u = beta * (s_v[col] - dk), ov = fmaf(s_kq, u, dq);
+#pragma unroll
+    for (int i = 0; i < NR; i++) {
+        const int r = rg + 8 * i;
+        if (live && r < D) S[(int64_t)r * V + c] = fmaf(s_k[r], u, s[i]);
+    }
+    if (rg == 0) {  // (the low half of wavefront 0)
+        float ss = live ? ov * ov : 0.0f;
+#pragma unroll
+        for (int m = 16; m >= 1; m >>= 1) ss += __shfl_xor(ss, m, WAVE);
+        if (live) o[h * V + c] = ov;
+        if (col == 0) ssq[h * n_split + sp] = ss;
+    }
+}
+
+hipError_t k_delta_step(hipStream_t s, const DeltaShape &d, const DeltaWeights &w, const float *in, float *ring, float *state,
+                        const DecodeCtl *ctl, float *o, float *ssq, float *gate) {
+    const int ns = delta_splits(d.V), nr = d.D <= 64 ? 8 : d.D <= 128 ? 16 : 32;
+    if (d.D > 256) return hipErrorInvalidValue;
+    const size_t lds = (size_t)(3 * 8 * nr + w.lda2 + w.ldg2) * sizeof(float);
+    if (lds > 60 * 1024) return hipErrorInvalidValue;
+    const dim3 grid((unsigned)ns, (unsigned)d.H);
+#define GO(N) hipLaunchKernelGGL((delta_step_kernel<N>), grid, dim3(256), lds, s, d, w, in, ring, state, ctl, o, ssq, gate, ns)
+    if (nr == 8)
+        GO(8);
+    else if (nr == 16)
+        GO(16);
+    else
+        GO(32);
+#undef GO
+    return hipGetLastError();
+}
+
+// ---------------------------------------------------------------------------------------------------------------
+// many tokens: convolutions and unit vectors.  A wavefront takes one unit (a key head's q and k, or a value head, or the
+// rest of the row) over PREP_T consecutive tokens.
+// ---------------------------------------------------------------------------------------------------------------
+#define PREP_T 8
+
+__device__ __forceinline__ float delta_raw_at(const float *raw, int64_t ldr, const float *ring, int C, int taps, int ch, int m, int pos0) {
+    if (m >= 0) return raw[(int64_t)m * ldr + ch];
+    const int p = pos0 + m;
+    return p >= 0 ? ring[(int64_t)(p % taps) * C + ch] : 0.0f;
+}
+
+template <int PREC>
+__global__ __launch_bounds__(256) void delta_prepare_kernel(DeltaShape d, const float *conv, const float *raw, int64_t ldr,
+                                                            const float *ring, int M, int pos0, float *qkv, float *kq, float *beta,
+                                                            void *fa, int64_t lfa, void *fg, int64_t lfg) {
+    const int lane = threadIdx.x & 63;
+    const int unit = blockIdx.x * 4 + (threadIdx.x >> 6), n_units = d.G + d.H + 1;
+    const int m0 = blockIdx.y * PREP_T, m1 = min(m0 + PREP_T, M);
+    if (unit >= n_units) return;
+    const int C = d.channels(), GD = d.G * d.D, taps = d.taps;
+    if (unit == d.G + d.H) {  // beta and the low-rank factors
+        for (int m = m0; m < m1; m++) {
+            const float *r = raw + (int64_t)m * ldr;
+            for (int h = lane; h < d.H; h += 64) beta[(int64_t)m * d.H + h] = l_sigmoid(r[d.off_b() + h]);
+            for (int i = lane; i < lfa; i += 64) l_store_act<PREC>(fa, (int64_t)m * lfa + i, i < d.ra ? r[d.off_a() + i] : 0.0f);
+            for (int i = lane; i < lfg; i += 64) l_store_act<PREC>(fg, (int64_t)m * lfg + i, i < d.rg ? r[d.off_g() + i] : 0.0f);
+        }
+        return;
+    }
+    if (unit >= d.G) {  // a value head
+        const int ch0 = 2 * GD + (unit - d.G) * d.V;
+        for (int e = lane; e < d.V; e += 64) {
+            const float *w = conv + (int64_t)(ch0 + e) * taps;
+            for (int m = m0; m < m1; m++) {
+                float v = 0.0f;
+                for (int j = 0; j < taps; j++)
+                    v = fmaf(w[taps - 1 - j], delta_raw_at(raw, ldr, ring, C, taps, ch0 + e, m - j, pos0), v);
+                qkv[(int64_t)m * C + ch0 + e] = l_silu(v);
+            }
+        }
+        return;
+    }
+    // a key head's q and k: D <= 256 elements, four per lane
+    const float qs = 1.0f / sqrtf((float)d.D);
+    for (int m = m0; m < m1; m++) {
+        float q[4], k[4], qq = 0.0f, kk = 0.0f, qk = 0.0f;
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+            const int e = lane + 64 * i;
+            q[i] = k[i] = 0.0f;
+            if (e >= d.D) continue;
+            const int cq = unit * d.D + e, ck = GD + cq;
+            for (int j = 0; j < taps; j++) {
+                q[i] = fmaf(conv[(int64_t)cq * taps + taps - 1 - j], delta_raw_at(raw, ldr, ring, C, taps, cq, m - j, pos0), q[i]);
+                k[i] = fmaf(conv[(int64_t)ck * taps + taps - 1 - j], delta_raw_at(raw, ldr, ring, C, taps, ck, m - j, pos0), k[i]);
+            }
+            q[i] = l_silu(q[i]);
+            k[i] = l_silu(k[i]);
+            qq = fmaf(q[i], q[i], qq);
+            kk = fmaf(k[i], k[i], kk);
+        }
+        const float rq = qs / sqrtf(l_wave_sum(qq) + 1e-6f), rk = 1.0f / sqrtf(l_wave_sum(kk) + 1e-6f);
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+            const int e = lane + 64 * i;
+            if (e >= d.D) continue;
+            q[i] *= rq;
+            k[i] *= rk;
+            qk = fmaf(q[i], k[i], qk);
+            qkv[(int64_t)m * C + unit * d.D + e] = q[i];
+            qkv[(int64_t)m * C + GD + unit * d.D + e] = k[i];
+        }
+        qk = l_wave_sum(qk);
+        if (lane == 0) kq[(int64_t)m * d.G + unit] = qk;
+    }
+}
+
+hipError_t k_delta_prepare(hipStream_t s, const DeltaShape &d, const float *conv, const float *raw, int64_t ldr, const float *ring,
+                           int M, int pos0, float *qkv, float *kq, float *beta, void *fa, int64_t lfa, void *fg, int64_t lfg,
+                           int prec) {
+    if (d.D > 256 || M < 1) return hipErrorInvalidValue;
+    const dim3 grid((unsigned)((d.G + d.H + 1 + 3) / 4), (unsigned)((M + PREP_T - 1) / PREP_T));
+    if (prec)
+        hipLaunchKernelGGL((delta_prepare_kernel<1>), grid, dim3(256), 0, s, d, conv, raw, ldr, ring, M, pos0, qkv, kq, beta, fa, lfa, fg, lfg);
+    else
+        hipLaunchKernelGGL((delta_prepare_kernel<0>), grid, dim3(256), 0, s, d, conv, raw, ldr, ring, M, pos0, qkv, kq, beta, fa, lfa, fg, lfg);
+    return hipGetLastError();
+}
+
+// the ring takes the last `taps` tokens' projected channels
+__global__ __launch_bounds__(256) void delta_ring_kernel(const float *raw, int64_t ldr, float *ring, int C, int taps, int M, int pos0) {
+    const int ch = blockIdx.x * 256 + threadIdx.x, m = M - 1 - (int)blockIdx.y;
+    if (ch >= C || m < 0) return;
+    ring[(int64_t)((pos0 + m) % taps) * C + ch] = raw[(int64_t)m * ldr + ch];
+}
+hipError_t k_delta_ring(hipStream_t s, const DeltaShape &d, const float *raw, int64_t ldr, float *ring, int M, int pos0) {
+    const int C = d.channels();
+    hipLaunchKernelGGL(delta_ring_kernel, dim3((unsigned)((C + 255) / 256), (unsigned)std::min(M, d.taps)), dim3(256), 0, s, raw, ldr,
+                       ring, C, d.taps, M, pos0);
+    return hipGetLastError();
+}
+
+// ---------------------------------------------------------------------------------------------------------------
+// the recurrence, token by token: workgroup (16 value columns, head); a wavefront holds 4 columns, 16 lanes per column,
+// E = 4 NE key channels per lane (4 consecutive ones of every 64)
+// ---------------------------------------------------------------------------------------------------------------
+#define SCAN_T 16  // tokens staged in LDS at a time
+
+// sum over the 16 lanes of a row, in every lane
+__device__ __forceinline__ float row16_sum(float v) {
+    v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x128, 0xF, 0xF, true));  // row_ror:8
+    v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x124, 0xF, 0xF, true));
+    v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x122, 0xF, 0xF, true));
+    v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x121, 0xF, 0xF, true));
+    return v;
+}
+
+template <int NE>
+__global__ __launch_bounds__(256) void delta_scan_kernel(DeltaShape d, const float *qkv, const float *kq, const float *beta,
+                                                         const float *lg, float *state, int M, int pos0, float *o) {
+    constexpr int DP = 64 * NE;
+    __shared__ __align__(16) float s_q[SCAN_T][DP], s_k[SCAN_T][DP], s_g[SCAN_T][DP];
+    __shared__ float s_v[SCAN_T][16], s_o[SCAN_T][16], s_b[SCAN_T], s_kq[SCAN_T];
+    const int t = threadIdx.x, lane = t & 63, wave = t >> 6;
+    const int h = blockIdx.y, kvh = h / (d.H / d.G), c0 = blockIdx.x * 16;
+    const int D = d.D, V = d.V, C = d.channels(), GD = d.G * D;
+    const int wc = 4 * wave + (lane >> 4), dl = lane & 15, c = c0 + wc;
+    const bool live = c < V;
+    float *S = state + (int64_t)h * D * V;
+    float s[NE][4];
+#pragma unroll
+    for (int i = 0; i < NE; i++)
+#pragma unroll
+        for (int j = 0; j < 4; j++) {
+            const int r = 64 * i + 4 * dl + j;
+            s[i][j] = (live && r < D && pos0 > 0) ? S[(int64_t)r * V + c] : 0.0f;
+        }
+    for (int m0 = 0; m0 < M; m0 += SCAN_T) {
+        const int n = min(SCAN_T, M - m0);
+        __syncthreads();
+        for (int i = t; i < SCAN_T * DP; i += 256) {
+            const int tt = i / DP, e = i - tt * DP;
+            float q = 0.0f, k = 0.0f, g = 1.0f;
+            if (tt < n && e < D) {
+                const float *row = qkv + (int64_t)(m0 + tt) * C + kvh * D + e;
+                q = row[0];
+                k = row[GD];
+                g = expf(lg[(int64_t)(m0 + tt) * d.H * D + h * D + e]);
+            }
+            s_q[tt][e] = q;
+            s_k[tt][e] = k;
+            s_g[tt][e] = g;
+        }
+        {
+            const int tt = t >> 4, e = t & 15;
+            s_v[tt][e] = (tt < n && c0 + e < V) ? qkv[(int64_t)(m0 + tt) * C + 2 * GD + h * V + c0 + e] : 0.0f;
+            if (e == 0) {
+                s_b[tt] = tt < n ? beta[(int64_t)(m0 + tt) * d.H + h] : 0.0f;
+                s_kq[tt] = tt < n ? kq[(int64_t)(m0 + tt) * d.G + kvh] : 0.0f;
+            }
+        }
+        __syncthreads();
+        for (int tt = 0; tt < n; tt++) {
+            float4 k[NE], q[NE];
+            float dk = 0.0f, dq = 0.0f;
+#pragma unroll
+            for (int i = 0; i < NE; i++) {
+                const float4 g = *(const float4 *)&s_g[tt][64 * i + 4 * dl];
+                k[i] = *(const float4 *)&s_k[tt][64 * i + 4 * dl];
+                q[i] = *(const float4 *)&s_q[tt][64 * i + 4 * dl];
+                s[i][0] *= g.x;
+                s[i][1] *= g.y;
+                s[i][2] *= g.z;
+                s[i][3] *= g.w;
+                dk = fmaf(s[i][0], k[i].x, dk);
+                dq = fmaf(s[i][0], q[i].x, dq);
+                dk = fmaf(s[i][1], k[i].y, dk);
+                dq = fmaf(s[i][1], q[i].y, dq);
+                dk = fmaf(s[i][2], k[i].z, dk);
+                dq = fmaf(s[i][2], q[i].z, dq);
+                dk = fmaf(s[i][3], k[i].w, dk);
+                dq = fmaf(s[i][3], q[i].w, dq);
+            }
+            dk = row16_sum(dk);
+            dq = row16_sum(dq);
+            const float u = s_b[tt] * (s_v[tt][wc] - dk);
+#pragma unroll
+            for (int i = 0; i < NE; i++) {
+                s[i][0] = fmaf(k[i].x, u, s[i][0]);
+                s[i][1] = fmaf(k[i].y, u, s[i][1]);
+                s[i][2] = fmaf(k[i].z, u, s[i][2]);
+                s[i][3] = fmaf(k[i].w, u, s[i][3]);
+            }
+            if (dl == 0) s_o[tt][wc] = fmaf(s_kq[tt], u, dq);
+        }
+        __syncthreads();
+        {
+            const int tt = t >> 4, e = t & 15;
+            if (tt < n && c0 + e < V) o[(int64_t)(m0 + tt) * d.H * V + h * V + c0 + e] = s_o[tt][e];
+        }
+    }
+#pragma unroll
+    for (int i = 0; i < NE; i++)
+#pragma unroll
+        for (int j = 0; j < 4; j++) {
+            const int r = 64 * i + 4 * dl + j;
+            if (live && r < D) S[(int64_t)r * V + c] = s[i][j];
+        }
+}
+
+hipError_t k_delta_scan(hipStream_t s, const DeltaShape &d, const float *qkv, const float *kq, const float *beta, const float *lg,
+                        float *state, int M, int pos0, float *o) {
+    if (d.D > 256 || M < 1) return hipErrorInvalidValue;
+    const dim3 grid((unsigned)((d.V + 15) / 16), (unsigned)d.H);
+#define GO(N) hipLaunchKernelGGL((delta_scan_kernel<N>), grid, dim3(256), 0, s, d, qkv, kq, beta, lg, state, M, pos0, o)
+    switch ((d.D + 63) / 64) {
+    case 1: GO(1); break;
+    case 2: GO(2); break;
+    case 3: GO(3); break;
+    default: GO(4); break;
+    }
+#undef GO
+    return hipGetLastError();
+}
+
+// one wavefront per (token, head)
+template <int PREC>
+__global__ __launch_bounds__(256) void head_norm_rows_kernel(const float *o, const float *gate, const float *normw, int M, int H, int V,
+                                                             float eps, void *outa, int64_t lda) {
+    const int lane = threadIdx.x & 63;
+    const int64_t unit = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (unit >= (int64_t)M * H) return;
+    const int m = (int)(unit / H), h = (int)(unit - (int64_t)m * H);
+    const float *x = o + (int64_t)m * H * V + h * V, *g = gate + (int64_t)m * H * V + h * V;
+    float ss = 0.0f;
+    for (int j = lane; j < V; j += 64) ss = fmaf(x[j], x[j], ss);
+    const float r = 1.0f / sqrtf(l_wave_sum(ss) / (float)V + eps);
+    for (int j = lane; j < V; j += 64) l_store_act<PREC>(outa, m * lda + h * V + j, x[j] * r * normw[j] * g[j]);
+    if (h == H - 1)
+        for (int64_t j = (int64_t)H * V + lane; j < lda; j += 64) l_store_act<PREC>(outa, m * lda + j, 0.0f);
+}
+hipError_t k_head_norm_rows(hipStream_t s, const float *o, const float *gate, const float *normw, int M, int H, int V, float eps,
+                            void *outa, int64_t lda, int prec) {
+    const dim3 grid((unsigned)(((int64_t)M * H + 3) / 4));
+    if (prec)
+        hipLaunchKernelGGL((head_norm_rows_kernel<1>), grid, dim3(256), 0, s, o, gate, normw, M, H, V, eps, outa, lda);
+    else
+        hipLaunchKernelGGL((head_norm_rows_kernel<0>), grid, dim3(256), 0, s, o, gate, normw, M, H, V, eps, outa, lda);
+    return hipGetLastError();
+}

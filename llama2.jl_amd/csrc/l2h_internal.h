@@ -17,6 +17,7 @@
 // (structure-of-arrays over the GGUF super-blocks) so that a wavefront reads every stream
 // with 16-byte lane loads over contiguous memory:
 //   F32   f32 [ne1][ne0]
+//   BF16  qs = bf16 [ne1][ne0] (layered models' embedding table)
 //   Q4_K  hdr  16 B/block  = {f16 d, f16 dmin, u8 scales[12]}  (the block's first 16 bytes)
 //         qs  128 B/block
 //   Q5_K  hdr  16 B/block, qh 32 B/block, qs 128 B/block

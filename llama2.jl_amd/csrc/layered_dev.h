@@ -1,0 +1,86 @@
+// Device helpers of the layered models' kernels.
+#pragma once
+
+#include "dev_common.h"
+#include "layered.h"
+
+typedef __bf16 l_bf16x2 __attribute__((ext_vector_type(2)));
+
+__device__ __forceinline__ uint32_t l_pack_bf16(float a, float b) {
+    l_bf16x2 v;
+    v.x = (__bf16)a;
+    v.y = (__bf16)b;
+    return __builtin_bit_cast(uint32_t, v);
+}
+__device__ __forceinline__ float l_bf16_lo(uint32_t w) { return __uint_as_float(w << 16); }
+__device__ __forceinline__ float l_bf16_hi(uint32_t w) { return __uint_as_float(w & 0xFFFF0000u); }
+__device__ __forceinline__ float l_bf16(uint16_t w) { return __uint_as_float((uint32_t)w << 16); }
+
+__device__ __forceinline__ float l_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
+__device__ __forceinline__ float l_silu(float z) { return z / (1.0f + expf(-z)); }
+__device__ __forceinline__ float l_softplus(float z) { return z > 20.0f ? z : log1pf(expf(z)); }
+__device__ __forceinline__ float l_act(int act, float z) {
+    if (act == LACT_RELU2) {
+        const float r = fmaxf(z, 0.0f);
+        return r * r;
+    }
+    if (act == LACT_GELU_TANH) return 0.5f * z * (1.0f + tanhf(0.797884560802865356f * fmaf(0.044715f * z * z, z, z)));
+    return 0.5f * z * (1.0f + erff(z * 0.707106781186547524f));
+}
+
+__device__ __forceinline__ float l_wave_sum(float v) {
+#pragma unroll
+    for (int m = 32; m >= 1; m >>= 1) v += __shfl_xor(v, m, WAVE);
+    return v;
+}
+// sum over the workgroup; `red` holds one float per wavefront; every thread gets the total
+__device__ __forceinline__ float l_block_sum(float v, float *red) {
+    const int nw = (blockDim.x + 63) >> 6;
+    v = l_wave_sum(v);
+    __syncthreads();
+    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+    __syncthreads();
+    float t = 0.0f;
+    for (int w = 0; w < nw; w++) t += red[w];
+    return t;
+}
+
+// activations: bf16 or fp32 elements behind one pointer
+template <int PREC>
+__device__ __forceinline__ void l_store_act(void *p, int64_t i, float v) {
+    if (PREC)
+        ((float *)p)[i] = v;
+    else
+        ((__bf16 *)p)[i] = (__bf16)v;
+}
+
+// the token of the current decode step (as embed_kernel picks it)
+__device__ __forceinline__ int l_step_token(const DecodeCtl *ctl, const int32_t *prompt) {
+    return ctl->step < ctl->n_prompt ? prompt[ctl->step] : ctl->last_argmax;
+}
+
+// Rotation of the pairs (2 i, 2 i + 1), i < rot / 2, of one head at `pos` and division by the head's root mean square, by
+// one wavefront.  src and dst hold D elements.
+__device__ __forceinline__ void l_rotate_norm(const float *src, float *dst, int D, int rot, const float *freq, int pos, int norm,
+                                              float eps, int lane) {
+    float ss = 0.0f;
+    for (int p = lane; 2 * p < D; p += 64) {
+        float a = src[2 * p], b = 2 * p + 1 < D ? src[2 * p + 1] : 0.0f;
+        if (2 * p < rot) {
+            const float ang = (float)pos * freq[p];
+            const float c = cosf(ang), s = sinf(ang), u = a, v = b;
+            a = u * c - v * s;
+            b = v * c + u * s;
+        }
+        ss = fmaf(a, a, ss);
+        ss = fmaf(b, b, ss);
+        dst[2 * p] = a;
+        if (2 * p + 1 < D) dst[2 * p + 1] = b;
+    }
+    if (!norm) return;
+    const float r = 1.0f / sqrtf(l_wave_sum(ss) / (float)D + eps);
+    for (int p = lane; 2 * p < D; p += 64) {
+        dst[2 * p] *= r;
+        if (2 * p + 1 < D) dst[2 * p + 1] *= r;
+    }
+}

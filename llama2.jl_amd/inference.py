@@ -67,21 +67,11 @@ class DeviceModel:
     def __init__(self, config, weights, ctx=None, path=0, kv_fp16=False):
         self.ctx = ctx or _lib.default_context()
         self.config = config
-        cfg = _lib.Config(config.dim, config.hidden_dim, config.n_layers, config.n_heads, config.n_kv_heads,
-                          config.vocab_size, config.seq_len, float(config.rope_freq_base),
-                          1 if config.rope_is_neox else 0)
         self.handle = C.c_void_p()
         self._shapes = {}
-        self.ctx.check(_lib.lib().l2h_model_create(self.ctx.handle, C.byref(cfg), C.byref(self.handle)))
+        self._create()
         try:
-            self._set(_lib.TOK_EMB, 0, weights.token_embedding_table)
-            self._set(_lib.RMS_FINAL, 0, weights.rms_final_weight)
-            self._set(_lib.OUTPUT, 0, weights.output_weight)
-            if len(weights.layers) != config.n_layers:
-                raise ValueError("config.n_layers = %d but %d layers given" % (config.n_layers, len(weights.layers)))
-            for l, lw in enumerate(weights.layers):
-                for name, role in _LAYER_ROLES:
-                    self._set(role, l, getattr(lw, name))
+            self._upload(weights)
             if kv_fp16:
                 self.ctx.check(_lib.lib().l2h_model_set_kv_type(self.handle, 1))
             self.ctx.check(_lib.lib().l2h_model_set_path(self.handle, path))
@@ -92,6 +82,22 @@ class DeviceModel:
         except Exception:
             self.close()
             raise
+
+    def _create(self):
+        c = self.config
+        cfg = _lib.Config(c.dim, c.hidden_dim, c.n_layers, c.n_heads, c.n_kv_heads, c.vocab_size, c.seq_len,
+                          float(c.rope_freq_base), 1 if c.rope_is_neox else 0)
+        self.ctx.check(_lib.lib().l2h_model_create(self.ctx.handle, C.byref(cfg), C.byref(self.handle)))
+
+    def _upload(self, weights):
+        self._set(_lib.TOK_EMB, 0, weights.token_embedding_table)
+        self._set(_lib.RMS_FINAL, 0, weights.rms_final_weight)
+        self._set(_lib.OUTPUT, 0, weights.output_weight)
+        if len(weights.layers) != self.config.n_layers:
+            raise ValueError("config.n_layers = %d but %d layers given" % (self.config.n_layers, len(weights.layers)))
+        for l, lw in enumerate(weights.layers):
+            for name, role in _LAYER_ROLES:
+                self._set(role, l, getattr(lw, name))
 
     def _set(self, role, layer, A):
         if isinstance(A, np.ndarray) and A.ndim == 1:
@@ -176,6 +182,17 @@ class DeviceModel:
                                               C.byref(nxt)))
         return logits, nxt.value
 
+    def prefill_logits(self, tokens, want, pos0=0, want_next=False):
+        """The same pass; returns the logits [len(want)][vocab] of the positions tokens[want] (l2h_prefill_logits), with
+        want_next also the argmax of the last position."""
+        tokens = np.ascontiguousarray(tokens, dtype=np.int32)
+        want = np.ascontiguousarray(want, dtype=np.int32)
+        logits = np.empty((want.size, self.config.vocab_size), np.float32)
+        nxt = C.c_int32()
+        self.ctx.check(_lib.lib().l2h_prefill_logits(self.handle, _lib.ptr(tokens), tokens.size, int(pos0), _lib.ptr(want), want.size,
+                                                     _lib.ptr(logits), C.byref(nxt) if want_next else None))
+        return (logits, nxt.value) if want_next else logits
+
     def sample_token(self, temperature, u, want_probs=False):
         """Temperature sampling from the logits of the last step (src/inference.jl:363-367) with the
         uniform number u in [0, 1) standing in for wsample's draw."""
@@ -217,6 +234,12 @@ class DeviceModel:
         return us.value, b.value
 
 
+def device_class(config):
+    """The resident form of a model with this configuration: DeviceModel, or LayeredDevice for a LayeredConfig."""
+    from .layered import LayeredConfig, LayeredDevice
+    return LayeredDevice if isinstance(config, LayeredConfig) else DeviceModel
+
+
 class LanguageModel:  # src/inference.jl:50-54
     def __init__(self, config, tokenizer, weights):
         self.config, self.tokenizer, self.weights = config, tokenizer, weights
@@ -226,7 +249,7 @@ class LanguageModel:  # src/inference.jl:50-54
         """Upload once; later calls reuse the resident copy (a closed one is replaced).  path: see
         l2h_model_set_path; kv_fp16: an fp16 KV cache (l2h_model_set_kv_type).  Both take effect when the copy is made."""
         if self._device is None or not self._device.handle:
-            self._device = DeviceModel(self.config, self.weights, ctx, path, kv_fp16)
+            self._device = device_class(self.config)(self.config, self.weights, ctx, path, kv_fp16)
         return self._device
 
     def __str__(self):  # src/inference.jl:56-60

@@ -23,6 +23,8 @@ class BPETokenizer(Tokenizer):
 
 def encode(text, tokenizer, pad_input=True):
     """encode(text, tokenizer) (src/tokenizer.jl:11-57 for BPE, :82-84 for characters)."""
+    if isinstance(tokenizer, IdTokenizer):
+        return tokenizer.encode(text)
     if isinstance(tokenizer, CharTokenizer):
         return [tokenizer.token_to_id[ch] for ch in text]
     data = text.encode("utf-8") if isinstance(text, str) else bytes(text)
@@ -55,6 +57,25 @@ class CharTokenizer(Tokenizer):
         self.token_to_id = {t: i for i, t in enumerate(self.id_to_token)}
         self.bos_token_id = len(self.id_to_token) - 2
         self.eos_token_id = len(self.id_to_token) - 1
+
+    def decode(self, ids):
+        return "".join(self.id_to_token[i] for i in ids)
+
+
+class IdTokenizer(Tokenizer):
+    """For models that come without a vocabulary: a text is token ids with blanks between them.  There are no special
+    tokens, so sample() takes such a model with bos_token=False."""
+    bos_token_id = eos_token_id = -1
+
+    def __init__(self, vocab_size):
+        self.id_to_token = ["%d " % i for i in range(vocab_size)]
+
+    def encode(self, text):
+        ids = [int(w) for w in text.split()]
+        for i in ids:
+            if not 0 <= i < len(self.id_to_token):
+                raise ValueError("token id %d outside the vocabulary of %d" % (i, len(self.id_to_token)))
+        return ids
 
     def decode(self, ids):
         return "".join(self.id_to_token[i] for i in ids)

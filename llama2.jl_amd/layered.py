@@ -138,6 +138,12 @@ class LayeredDevice(DeviceModel):
         self.ctx.check(_lib.lib().l2h_layered_kept(self.handle, layer, _lib.ptr(out), out.size))
         return out
 
+    def kv_read(self, layer, pos0, n):
+        raise ValueError("the rows of a layered model's cache are not exchanged with the host")
+
+    def kv_write(self, layer, pos0, k, v):
+        raise ValueError("the rows of a layered model's cache are not exchanged with the host")
+
     def state(self, name):
         n = {"x": self.config.width, "logits": self.config.vocab_size}[name]
         out = np.empty(n, np.float32)

@@ -2,8 +2,7 @@
 position by position, no shared code with the product path.  Test infrastructure only.
 
 A model is (config, tensors): config is the dictionary of config.json, tensors maps names to numpy arrays of shape
-[out, in].  `Sequence` holds what a sequence carries from token to token; `Sequence.step` runs one token.  `forward`
-runs a whole sequence at once in a second form (attention over the full score matrix).
+[out, in].  `Sequence` holds what a sequence carries from token to token; `Sequence.step` runs one token.
 
 `twist` plants one mistake by name, so that a test can show that it would notice it (see TWISTS)."""
 import math
@@ -15,7 +14,7 @@ TWISTS = {
     "window-1": "one key too few in the sliding window",
     "no_gate": "attention output gate left out",
     "no_qk_norm": "query/key norm left out",
-    "norm_before_rot": "half-split instead of interleaved rotation pairs",
+    "half_split": "half-split instead of interleaved rotation pairs",
     "no_rot_scaling": "frequency scaling left out",
     "no_conv_state": "short convolution sees zeros before the last token",
     "decay_first_channel": "one decay per head instead of one per key channel",
@@ -145,7 +144,7 @@ class Sequence:
         v = (t[p + "v"] @ h).reshape(G, V)
         if m.get("rot"):
             f = rot_frequencies(m["rot"], self.twist != "no_rot_scaling")
-            half = self.twist == "norm_before_rot"
+            half = self.twist == "half_split"
             q, k = rotate(q, self.pos, f, half), rotate(k, self.pos, f, half)
         if self.twist != "no_qk_norm":
             q, k = rms(q, eps), rms(k, eps)

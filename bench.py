@@ -63,6 +63,9 @@ WORKLOADS = {
                                       seq_len=512, rope_freq_base=500000.0, rope_is_neox=False), 32),
 }
 
+# layered models beside a Llama model of equal size (llama2.jl_amd/bench_layered.py)
+LAYERED_WORKLOADS = ["vudelix-2k", "vudelix-4k"]
+
 
 def log(*a):
     print(*a, file=sys.stderr, flush=True)
@@ -85,7 +88,7 @@ def main():
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=128)
     ap.add_argument("--warmup", type=int, default=8)
-    ap.add_argument("--workload", default="8b-q4ks", choices=sorted(WORKLOADS))
+    ap.add_argument("--workload", default="8b-q4ks", choices=sorted(WORKLOADS) + LAYERED_WORKLOADS)
     ap.add_argument("--repeats", type=int, default=3, help="timed regions; the median is reported")
     ap.add_argument("--path", type=int, default=0, help="0 auto, 1 kernel per phase, 2 persistent kernel, 3 streaming kernel")
     ap.add_argument("--cpu-seconds", type=float, default=15.0, help="budget of the CPU baseline leg (0 = skip)")
@@ -98,6 +101,9 @@ def main():
         sys.exit(2)
 
     pkg = entry.load_package()
+    if args.workload in LAYERED_WORKLOADS:
+        from llama2_jl_amd import bench_layered
+        return bench_layered.run(pkg, args, log)
     from llama2_jl_amd import _lib, synth
     plan_name, kw, n_prompt = WORKLOADS[args.workload]
     cfg = pkg.ModelConfig(**kw)

@@ -8,29 +8,39 @@
 // ---------------------------------------------------------------------------------------------------------------
 // one token: workgroup (split, head), 32 value columns x 8 groups of key channels
 // ---------------------------------------------------------------------------------------------------------------
-__device__ __forceinline__ float delta_conv(const DeltaShape &d, const float *conv, const float *ring, float cur, int ch, int pos) {
-    const float *w = conv + (int64_t)ch * d.taps;
-    const int C = d.channels();
-    float v = w[d.taps - 1] * cur;
-    for (int j = 1; j < d.taps && j <= pos; j++) v = fmaf(w[d.taps - 1 - j], ring[(int64_t)((pos - j) % d.taps) * C + ch], v);
+#define CONV_AHEAD 4  // taps whose inputs are fetched together
+
+// the channel's convolution at `pos`: cur is its projection, ring slot `now` = pos % taps will hold it
+__device__ __forceinline__ float delta_conv(const float *conv, const float *ring, int C, int taps, float cur, int ch, int pos, int now) {
+    float w[CONV_AHEAD], x[CONV_AHEAD];
+#pragma unroll
+    for (int j = 0; j < CONV_AHEAD; j++) {
+        const bool use = j < taps && j <= pos;
+        const int slot = now - j < 0 ? now - j + taps : now - j;
+        w[j] = use ? conv[(int64_t)(taps - 1 - j) * C + ch] : 0.0f;
+        x[j] = j == 0 ? cur : use ? ring[(int64_t)slot * C + ch] : 0.0f;
+    }
+    float v = 0.0f;
+#pragma unroll
+    for (int j = 0; j < CONV_AHEAD; j++) v = fmaf(w[j], x[j], v);
+    for (int j = CONV_AHEAD; j < taps && j <= pos; j++)
+        v = fmaf(conv[(int64_t)(taps - 1 - j) * C + ch], ring[(int64_t)((pos - j) % taps) * C + ch], v);
     return l_silu(v);
 }
 
-// dot of a bf16 row (zero-padded to ld) with a vector in LDS of ld floats, by 8 lanes; every one of them gets the sum
-__device__ __forceinline__ float delta_dot8(const uint16_t *w, const float *x, int ld, int l8) {
-    float acc = 0.0f;
-    for (int k = 8 * l8; k < ld; k += 64) {
-        const uint4 p = *(const uint4 *)(w + k);
-        const float4 a = *(const float4 *)(x + k), b = *(const float4 *)(x + k + 4);
-        acc = fmaf(l_bf16_lo(p.x), a.x, acc);
-        acc = fmaf(l_bf16_hi(p.x), a.y, acc);
-        acc = fmaf(l_bf16_lo(p.y), a.z, acc);
-        acc = fmaf(l_bf16_hi(p.y), a.w, acc);
-        acc = fmaf(l_bf16_lo(p.z), b.x, acc);
-        acc = fmaf(l_bf16_hi(p.z), b.y, acc);
-        acc = fmaf(l_bf16_lo(p.w), b.z, acc);
-        acc = fmaf(l_bf16_hi(p.w), b.w, acc);
-    }
+// 8 lanes take a bf16 row (zero-padded to ld) against a vector in LDS; every one of them gets the sum
+__device__ __forceinline__ float delta_fma8(uint4 p, const float *x, float acc) {
+    const float4 a = *(const float4 *)x, b = *(const float4 *)(x + 4);
+    acc = fmaf(l_bf16_lo(p.x), a.x, acc);
+    acc = fmaf(l_bf16_hi(p.x), a.y, acc);
+    acc = fmaf(l_bf16_lo(p.y), a.z, acc);
+    acc = fmaf(l_bf16_hi(p.y), a.w, acc);
+    acc = fmaf(l_bf16_lo(p.z), b.x, acc);
+    acc = fmaf(l_bf16_hi(p.z), b.y, acc);
+    acc = fmaf(l_bf16_lo(p.w), b.z, acc);
+    return fmaf(l_bf16_hi(p.w), b.w, acc);
+}
+__device__ __forceinline__ float delta_sum8(float acc) {
 #pragma unroll
     for (int m = 4; m >= 1; m >>= 1) acc += __shfl_xor(acc, m, WAVE);
     return acc;
@@ -55,32 +65,45 @@ __global__ __launch_bounds__(256) void delta_step_kernel(DeltaShape d, DeltaWeig
         const int r = rg + 8 * i;
         s[i] = (live && r < D && pos > 0) ? S[(int64_t)r * V + c] : 0.0f;
     }
-    // short convolutions; the token's own projections go into the ring (its slot is not read by this token)
-    const int C = d.channels();
-    float *slot = ring + (int64_t)(pos % d.taps) * C;
-    for (int i = t; i < 2 * D + L_DELTA_COLS; i += 256) {
-        int ch;
-        float *dst;
-        bool own;
-        if (i < 2 * D) {
-            const bool isk = i >= D;
-            const int e = isk ? i - D : i;
-            ch = (isk ? GD : 0) + kvh * D + e;
-            dst = (isk ? s_k : s_q) + e;
-            own = sp == 0 && h % (d.H / d.G) == 0;
-        } else {
-            const int e = i - 2 * D;
-            if (c0 + e >= V) {
-                s_v[e] = 0.0f;
-                continue;
-            }
-            ch = 2 * GD + h * V + c0 + e;
-            dst = s_v + e;
-            own = true;
+    // the first 128 inputs of the low-rank factors' rows are fetched ahead
+    const int l8 = t & 7, r8 = t >> 3;
+    uint4 fa[NR / 4][2], fg[2];
+#pragma unroll
+    for (int i = 0; i < NR / 4; i++)
+#pragma unroll
+        for (int e = 0; e < 2; e++) {
+            const int r = r8 + 32 * i, kk = 8 * l8 + 64 * e;
+            fa[i][e] = make_uint4(0, 0, 0, 0);
+            if (r < D && kk < w.lda2) fa[i][e] = *(const uint4 *)(w.a2 + ((int64_t)h * D + r) * w.lda2 + kk);
         }
-        const float cur = in[ch];
-        *dst = delta_conv(d, w.conv, ring, cur, ch, pos);
-        if (own) slot[ch] = cur;
+#pragma unroll
+    for (int e = 0; e < 2; e++) {
+        const int kk = 8 * l8 + 64 * e;
+        fg[e] = make_uint4(0, 0, 0, 0);
+        if (c0 + r8 < V && kk < w.ldg2) fg[e] = *(const uint4 *)(w.g2 + ((int64_t)h * V + c0 + r8) * w.ldg2 + kk);
+    }
+    // short convolutions; the token's own projections go into the ring (its slot is not read by this token)
+    const int C = d.channels(), now = pos % d.taps;
+    float *slot = ring + (int64_t)now * C;
+#pragma unroll
+    for (int ii = 0; ii < (16 * NR + L_DELTA_COLS + 255) / 256; ii++) {
+        const int i = t + 256 * ii;
+        if (i >= 2 * D + L_DELTA_COLS) break;
+        const bool isv = i >= 2 * D, isk = !isv && i >= D;
+        const int e = isv ? i - 2 * D : isk ? i - D : i;
+        if (isv && c0 + e >= V) {
+            s_v[e] = 0.0f;
+            continue;
+        }
+        const int ch = isv ? 2 * GD + h * V + c0 + e : (isk ? GD : 0) + kvh * D + e;
+        const float cur = in[ch], y = delta_conv(w.conv, ring, C, d.taps, cur, ch, pos, now);
+        if (isv)
+            s_v[e] = y;
+        else if (isk)
+            s_k[e] = y;
+        else
+            s_q[e] = y;
+        if (isv || (sp == 0 && h % (d.H / d.G) == 0)) slot[ch] = cur;
     }
     for (int i = t; i < w.lda2; i += 256) s_fa[i] = i < d.ra ? in[d.off_a() + i] : 0.0f;
     for (int i = t; i < w.ldg2; i += 256) s_fg[i] = i < d.rg ? in[d.off_g() + i] : 0.0f;
@@ -95,13 +118,27 @@ __global__ __launch_bounds__(256) void delta_step_kernel(DeltaShape d, DeltaWeig
         for (int e = lane; e < D; e += 64) x[e] *= r;
     }
     // decays of all key channels, gates of this workgroup's columns
-    const int l8 = t & 7, r8 = t >> 3;
-    for (int r = r8; r < D; r += 32) {
-        const float z = delta_dot8(w.a2 + ((int64_t)h * D + r) * w.lda2, s_fa, w.lda2, l8) + w.bias[h * D + r];
+#pragma unroll
+    for (int i = 0; i < NR / 4; i++) {
+        const int r = r8 + 32 * i;
+        if (r >= D) break;
+        const uint16_t *row = w.a2 + ((int64_t)h * D + r) * w.lda2;
+        float z = 0.0f;
+#pragma unroll
+        for (int e = 0; e < 2; e++)
+            if (8 * l8 + 64 * e < w.lda2) z = delta_fma8(fa[i][e], s_fa + 8 * l8 + 64 * e, z);
+        for (int kk = 8 * l8 + 128; kk < w.lda2; kk += 64) z = delta_fma8(*(const uint4 *)(row + kk), s_fa + kk, z);
+        z = delta_sum8(z) + w.bias[h * D + r];
         if (l8 == 0) s_g[r] = expf(-w.rate[h] * l_softplus(z));
     }
     if (c0 + r8 < V) {
-        const float z = delta_dot8(w.g2 + ((int64_t)h * V + c0 + r8) * w.ldg2, s_fg, w.ldg2, l8);
+        const uint16_t *row = w.g2 + ((int64_t)h * V + c0 + r8) * w.ldg2;
+        float z = 0.0f;
+#pragma unroll
+        for (int e = 0; e < 2; e++)
+            if (8 * l8 + 64 * e < w.ldg2) z = delta_fma8(fg[e], s_fg + 8 * l8 + 64 * e, z);
+        for (int kk = 8 * l8 + 128; kk < w.ldg2; kk += 64) z = delta_fma8(*(const uint4 *)(row + kk), s_fg + kk, z);
+        z = delta_sum8(z);
         if (l8 == 0) gate[h * V + c0 + r8] = l_sigmoid(z);
     }
     __syncthreads();
@@ -197,11 +234,10 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(DeltaShape d, const 
     if (unit >= d.G) {  // a value head
         const int ch0 = 2 * GD + (unit - d.G) * d.V;
         for (int e = lane; e < d.V; e += 64) {
-            const float *w = conv + (int64_t)(ch0 + e) * taps;
             for (int m = m0; m < m1; m++) {
                 float v = 0.0f;
                 for (int j = 0; j < taps; j++)
-                    v = fmaf(w[taps - 1 - j], delta_raw_at(raw, ldr, ring, C, taps, ch0 + e, m - j, pos0), v);
+                    v = fmaf(conv[(int64_t)(taps - 1 - j) * C + ch0 + e], delta_raw_at(raw, ldr, ring, C, taps, ch0 + e, m - j, pos0), v);
                 qkv[(int64_t)m * C + ch0 + e] = l_silu(v);
             }
         }
@@ -218,8 +254,8 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(DeltaShape d, const 
             if (e >= d.D) continue;
             const int cq = unit * d.D + e, ck = GD + cq;
             for (int j = 0; j < taps; j++) {
-                q[i] = fmaf(conv[(int64_t)cq * taps + taps - 1 - j], delta_raw_at(raw, ldr, ring, C, taps, cq, m - j, pos0), q[i]);
-                k[i] = fmaf(conv[(int64_t)ck * taps + taps - 1 - j], delta_raw_at(raw, ldr, ring, C, taps, ck, m - j, pos0), k[i]);
+                q[i] = fmaf(conv[(int64_t)(taps - 1 - j) * C + cq], delta_raw_at(raw, ldr, ring, C, taps, cq, m - j, pos0), q[i]);
+                k[i] = fmaf(conv[(int64_t)(taps - 1 - j) * C + ck], delta_raw_at(raw, ldr, ring, C, taps, ck, m - j, pos0), k[i]);
             }
             q[i] = l_silu(q[i]);
             k[i] = l_silu(k[i]);

@@ -3,19 +3,23 @@
 // linear in the position: kc[G][Dp / 4][seq_len][4], vc[G][seq_len][V].
 #include "layered_dev.h"
 
-#define WIN_MAX_HEADS 8  // query heads of a key/value head handled in one pass
+#define WIN_MAX_HEADS 8  // query heads of a key/value head handled in one pass of the one-token kernel
 
 // ---------------------------------------------------------------------------------------------------------------
-// one token: workgroup (split of the window, key/value head); a thread scores one key, then threads split the value columns
+// one token: workgroup (split of the window, key/value head).  Scores: a lane holds one key of the split, the four wavefronts
+// a quarter of the key elements each.  Values: groups of threads take every so-many-th key, a thread one column.
 // ---------------------------------------------------------------------------------------------------------------
+// NH query heads of a key/value head at a time (a missing one has a zero query)
+template <int NH>
 __global__ __launch_bounds__(256) void window_step_kernel(WindowShape w, const float *freq, const float *in, float *kc, float *vc,
                                                           const DecodeCtl *ctl, float *part, float *out, int n_split) {
     extern __shared__ __align__(16) float s_mem[];
+    constexpr int KA = 8, VA = 32;  // key quads and value rows a thread fetches ahead
     const int t = threadIdx.x, lane = t & 63, wave = t >> 6;
     const int g = blockIdx.y, sp = blockIdx.x, pos = ctl->pos;
     const int gq = w.H / w.G, D = w.D, Dp = w.Dp(), V = w.V, D4 = Dp / 4;
-    float *s_k = s_mem, *s_q = s_k + Dp, *s_p = s_q + WIN_MAX_HEADS * Dp, *s_acc = s_p + WIN_MAX_HEADS * L_WIN_SPLIT;
-    __shared__ float s_red[4][WIN_MAX_HEADS], s_l[WIN_MAX_HEADS], s_m[WIN_MAX_HEADS];
+    float *s_k = s_mem, *s_q = s_k + Dp, *s_acc = s_q + NH * Dp;
+    __shared__ float s_part[4][NH][L_WIN_SPLIT], s_p[NH][L_WIN_SPLIT], s_l[NH], s_m[NH];
     const int lo = max(0, pos - w.window + 1);
     const int k0 = lo + sp * L_WIN_SPLIT, n = min(L_WIN_SPLIT, pos + 1 - k0);  // this workgroup's keys
     if (n <= 0) {
@@ -27,7 +31,23 @@ __global__ __launch_bounds__(256) void window_step_kernel(WindowShape w, const f
         return;
     }
     const int64_t krow = (int64_t)g * D4 * w.seq_len;
-    const bool has_new = k0 + n - 1 == pos;
+    const bool has_new = k0 + n - 1 == pos;  // the token's own key and value come from its projections, not from the cache
+    const int nc = has_new ? n - 1 : n;      // keys of the split that the cache holds
+    const int kl = max(0, min(lane, nc - 1));  // (lanes beyond the cached keys repeat the last one)
+    const int i0 = D4 * wave / 4, i1 = D4 * (wave + 1) / 4;
+    const float *kp = kc + (krow + k0 + kl) * 4;
+    const int tv = min(256, V), np = 256 / tv, pg = t / tv, c = t - pg * tv;  // V <= 256
+    const bool mine = pg < np;
+    const float *vp = vc + ((int64_t)g * w.seq_len + k0) * V + c;
+    float4 kr[KA];
+    float vr[VA];
+#pragma unroll
+    for (int u = 0; u < KA; u++) kr[u] = *(const float4 *)(kp + (int64_t)min(i0 + u, D4 - 1) * w.seq_len * 4);
+#pragma unroll
+    for (int u = 0; u < VA; u++) {
+        const int i = pg + u * np;
+        vr[u] = (mine && i < nc) ? vp[(int64_t)i * V] : 0.0f;
+    }
     const float *v_new = in + w.off_v() + g * V;
     if (has_new) {
         if (wave == 3) {
@@ -36,98 +56,94 @@ __global__ __launch_bounds__(256) void window_step_kernel(WindowShape w, const f
         }
         for (int i = t; i < V; i += 256) vc[((int64_t)g * w.seq_len + pos) * V + i] = v_new[i];
     }
-    for (int h0 = 0; h0 < gq; h0 += WIN_MAX_HEADS) {
-        const int nh = min(WIN_MAX_HEADS, gq - h0);
+    for (int h0 = 0; h0 < gq; h0 += NH) {
+        const int nh = min(NH, gq - h0);
         __syncthreads();
-        for (int j = wave; j < nh; j += 4) {
-            for (int i = D + lane; i < Dp; i += 64) s_q[j * Dp + i] = 0.0f;
-            l_rotate_norm(in + (g * gq + h0 + j) * D, s_q + j * Dp, D, w.rot, freq, pos, w.qk_norm, w.eps, lane);
+        for (int j = wave; j < NH; j += 4) {
+            for (int i = (j < nh ? D : 0) + lane; i < Dp; i += 64) s_q[j * Dp + i] = 0.0f;
+            if (j < nh) l_rotate_norm(in + (g * gq + h0 + j) * D, s_q + j * Dp, D, w.rot, freq, pos, w.qk_norm, w.eps, lane);
         }
         __syncthreads();
         if (has_new && h0 == 0)
             for (int i = t; i < Dp; i += 256) kc[(krow + (int64_t)(i >> 2) * w.seq_len + pos) * 4 + (i & 3)] = s_k[i];
-        // scores of key k0 + t
-        float sc[WIN_MAX_HEADS];
+        float sc[NH];
 #pragma unroll
-        for (int j = 0; j < WIN_MAX_HEADS; j++) sc[j] = 0.0f;
-        const int key = k0 + t;
-        if (t < n) {
-            for (int i = 0; i < D4; i++) {
-                const float4 kv = key == pos ? *(const float4 *)(s_k + 4 * i)
-                                             : *(const float4 *)(kc + (krow + (int64_t)i * w.seq_len + key) * 4);
+        for (int j = 0; j < NH; j++) sc[j] = 0.0f;
+        auto score = [&](float4 kv, int i) {
 #pragma unroll
-                for (int j = 0; j < WIN_MAX_HEADS; j++)
-                    if (j < nh) {
-                        const float4 qv = *(const float4 *)(s_q + j * Dp + 4 * i);
-                        sc[j] = fmaf(qv.x, kv.x, sc[j]);
-                        sc[j] = fmaf(qv.y, kv.y, sc[j]);
-                        sc[j] = fmaf(qv.z, kv.z, sc[j]);
-                        sc[j] = fmaf(qv.w, kv.w, sc[j]);
-                    }
+            for (int j = 0; j < NH; j++) {
+                const float4 qv = *(const float4 *)(s_q + j * Dp + 4 * i);
+                sc[j] = fmaf(qv.x, kv.x, sc[j]);
+                sc[j] = fmaf(qv.y, kv.y, sc[j]);
+                sc[j] = fmaf(qv.z, kv.z, sc[j]);
+                sc[j] = fmaf(qv.w, kv.w, sc[j]);
+            }
+        };
+#pragma unroll
+        for (int u = 0; u < KA; u++)
+            if (i0 + u < i1) score(kr[u], i0 + u);
+        for (int i = i0 + KA; i < i1; i++) score(*(const float4 *)(kp + (int64_t)i * w.seq_len * 4), i);
+#pragma unroll
+        for (int j = 0; j < NH; j++) s_part[wave][j][lane] = sc[j];
+        __syncthreads();
+        for (int j = wave; j < nh; j += 4) {  // a wavefront per head: the whole scores, their softmax over the split
+            float v = s_part[0][j][lane] + s_part[1][j][lane] + s_part[2][j][lane] + s_part[3][j][lane];
+            if (has_new) {
+                float own = 0.0f;
+                for (int i = lane; i < D; i += 64) own = fmaf(s_q[j * Dp + i], s_k[i], own);
+                own = l_wave_sum(own);
+                if (lane == nc) v = own;
+            }
+            v = lane < n ? v * w.scale : -INFINITY;
+            const float mx = wave_max_f32(v);
+            const float p = lane < n ? expf(v - mx) : 0.0f;
+            s_p[j][lane] = p;
+            const float l = l_wave_sum(p);
+            if (lane == 0) {
+                s_m[j] = mx;
+                s_l[j] = l;
+            }
+        }
+        for (int j = nh + wave; j < NH; j += 4) s_p[j][lane] = 0.0f;
+        __syncthreads();
+        float acc[NH];
+#pragma unroll
+        for (int j = 0; j < NH; j++) acc[j] = 0.0f;
+        if (mine) {
+#pragma unroll
+            for (int u = 0; u < VA; u++) {
+                const int i = min(pg + u * np, L_WIN_SPLIT - 1);  // (a value past the cached keys was fetched as 0)
+#pragma unroll
+                for (int j = 0; j < NH; j++) acc[j] = fmaf(s_p[j][i], vr[u], acc[j]);
+            }
+            for (int i = pg + VA * np; i < nc; i += np) {
+                const float v = vp[(int64_t)i * V];
+#pragma unroll
+                for (int j = 0; j < NH; j++) acc[j] = fmaf(s_p[j][i], v, acc[j]);
+            }
+            if (has_new && pg == 0) {
+                const float v = v_new[c];
+#pragma unroll
+                for (int j = 0; j < NH; j++) acc[j] = fmaf(s_p[j][nc], v, acc[j]);
             }
         }
 #pragma unroll
-        for (int j = 0; j < WIN_MAX_HEADS; j++)
-            if (j < nh) {
-                sc[j] = t < n ? sc[j] * w.scale : -INFINITY;
-                const float mx = wave_max_f32(sc[j]);
-                if (lane == 0) s_red[wave][j] = mx;
-            }
+        for (int j = 0; j < NH; j++) s_acc[j * 256 + t] = acc[j];
         __syncthreads();
-#pragma unroll
-        for (int j = 0; j < WIN_MAX_HEADS; j++)
-            if (j < nh) {
-                const float mx = fmaxf(fmaxf(s_red[0][j], s_red[1][j]), fmaxf(s_red[2][j], s_red[3][j]));
-                const float p = t < n ? expf(sc[j] - mx) : 0.0f;
-                s_p[j * L_WIN_SPLIT + t] = p;
-                sc[j] = l_wave_sum(p);
-                if (t == 0) s_m[j] = mx;
-            }
-        __syncthreads();
-        if (lane == 0)
-#pragma unroll
-            for (int j = 0; j < WIN_MAX_HEADS; j++)
-                if (j < nh) s_red[wave][j] = sc[j];
-        __syncthreads();
-        if (t < nh) s_l[t] = s_red[0][t] + s_red[1][t] + s_red[2][t] + s_red[3][t];
-        // values: np groups of threads take every np-th key, a thread V / threads-of-a-group columns
-        const int tv = min(256, V), np = 256 / tv, pg = t / tv, cc = t - pg * tv;
-        for (int cb = 0; cb < V; cb += tv) {
-            const int c = cb + cc;
-            float acc[WIN_MAX_HEADS];
-#pragma unroll
-            for (int j = 0; j < WIN_MAX_HEADS; j++) acc[j] = 0.0f;
-            if (pg < np && c < V) {
-                const float *vp = vc + ((int64_t)g * w.seq_len + k0) * V + c;
-#pragma unroll 4
-                for (int i = pg; i < n; i += np) {
-                    const float v = k0 + i == pos ? v_new[c] : vp[(int64_t)i * V];
-#pragma unroll
-                    for (int j = 0; j < WIN_MAX_HEADS; j++)
-                        if (j < nh) acc[j] = fmaf(s_p[j * L_WIN_SPLIT + i], v, acc[j]);
-                }
-            }
-            __syncthreads();
-#pragma unroll
-            for (int j = 0; j < WIN_MAX_HEADS; j++)
-                if (j < nh) s_acc[j * 256 + t] = acc[j];
-            __syncthreads();
-            for (int idx = t; idx < nh * tv; idx += 256) {
-                const int j = idx / tv, e = idx - j * tv, c2 = cb + e, h = g * gq + h0 + j;
-                if (c2 >= V) continue;
-                float v = 0.0f;
-                for (int p = 0; p < np; p++) v += s_acc[j * 256 + p * tv + e];
-                if (n_split == 1) {
-                    v /= s_l[j];
-                    if (w.gated) v *= l_sigmoid(in[w.off_g() + h]);
-                    out[h * V + c2] = v;
-                } else {
-                    float *p = part + ((int64_t)h * n_split + sp) * (V + 2);
-                    p[2 + c2] = v;
-                    if (c2 == 0) {
-                        p[0] = s_m[j];
-                        p[1] = s_l[j];
-                    }
+        for (int idx = t; idx < nh * V; idx += 256) {
+            const int j = idx / V, e = idx - j * V, h = g * gq + h0 + j;
+            float v = 0.0f;
+            for (int p = 0; p < np; p++) v += s_acc[j * 256 + p * tv + e];
+            if (n_split == 1) {
+                v /= s_l[j];
+                if (w.gated) v *= l_sigmoid(in[w.off_g() + h]);
+                out[h * V + e] = v;
+            } else {
+                float *p = part + ((int64_t)h * n_split + sp) * (V + 2);
+                p[2 + e] = v;
+                if (e == 0) {
+                    p[0] = s_m[j];
+                    p[1] = s_l[j];
                 }
             }
         }
@@ -136,30 +152,57 @@ __global__ __launch_bounds__(256) void window_step_kernel(WindowShape w, const f
 
 // one workgroup per head: the splits' partial results joined
 __global__ __launch_bounds__(256) void window_join_kernel(WindowShape w, const float *in, const float *part, float *out, int n_split) {
-    const int h = blockIdx.x, V = w.V;
-    const float *p = part + (int64_t)h * n_split * (V + 2);
+    extern __shared__ __align__(16) float s_mem[];
+    float *s_f = s_mem, *s_acc = s_f + n_split;
+    __shared__ float s_red[4];
+    const int h = blockIdx.x, V = w.V, t = threadIdx.x, st = V + 2;
+    const float *p = part + (int64_t)h * n_split * st;
     float m = -INFINITY;
-    for (int i = 0; i < n_split; i++) m = fmaxf(m, p[(int64_t)i * (V + 2)]);
+    for (int i = t; i < n_split; i += 256) m = fmaxf(m, p[(int64_t)i * st]);
+    m = block_max_f32(m, s_red);
     float l = 0.0f;
-    for (int i = 0; i < n_split; i++) l = fmaf(expf(p[(int64_t)i * (V + 2)] - m), p[(int64_t)i * (V + 2) + 1], l);
-    const float g = w.gated ? l_sigmoid(in[w.off_g() + h]) : 1.0f;
-    for (int c = threadIdx.x; c < V; c += 256) {
-        float v = 0.0f;
-        for (int i = 0; i < n_split; i++) {
-            const float *q = p + (int64_t)i * (V + 2);
-            if (q[0] != -INFINITY) v = fmaf(expf(q[0] - m), q[2 + c], v);
-        }
-        out[h * V + c] = v / l * g;
+    for (int i = t; i < n_split; i += 256) {
+        const float f = expf(p[(int64_t)i * st] - m);  // (0 for a split without keys)
+        s_f[i] = f;
+        l = fmaf(f, p[(int64_t)i * st + 1], l);
+    }
+    l = l_block_sum(l, s_red);
+    const float g = (w.gated ? l_sigmoid(in[w.off_g() + h]) : 1.0f) / l;
+    __syncthreads();
+    const int np = 256 / V, pg = t / V, c = t - pg * V;  // V <= 256
+    float v = 0.0f;
+    if (pg < np)
+#pragma unroll 4
+        for (int i = pg; i < n_split; i += np)
+            if (s_f[i] != 0.0f) v = fmaf(s_f[i], p[(int64_t)i * st + 2 + c], v);
+    s_acc[t] = v;
+    __syncthreads();
+    if (t < V) {
+        v = 0.0f;
+        for (int i = 0; i < np; i++) v += s_acc[i * V + t];
+        out[h * V + t] = v * g;
     }
 }
 
 hipError_t k_window_step(hipStream_t s, const WindowShape &w, const float *freq, const float *in, float *kc, float *vc,
                          const DecodeCtl *ctl, float *part, float *out) {
     const int ns = window_splits(w);
-    const size_t lds = (size_t)(w.Dp() * (1 + WIN_MAX_HEADS) + WIN_MAX_HEADS * (L_WIN_SPLIT + 256)) * sizeof(float);
-    if (lds > 60 * 1024) return hipErrorInvalidValue;
-    hipLaunchKernelGGL(window_step_kernel, dim3((unsigned)ns, (unsigned)w.G), dim3(256), lds, s, w, freq, in, kc, vc, ctl, part, out, ns);
-    if (ns > 1) hipLaunchKernelGGL(window_join_kernel, dim3((unsigned)w.H), dim3(256), 0, s, w, in, part, out, ns);
+    const size_t lds = (size_t)(w.Dp() * (1 + WIN_MAX_HEADS) + WIN_MAX_HEADS * 256) * sizeof(float);
+    const size_t lds_join = (size_t)(ns + 256) * sizeof(float);
+    if (lds > 48 * 1024 || lds_join > 60 * 1024 || w.V > 256) return hipErrorInvalidValue;
+#define GO(N) \
+    hipLaunchKernelGGL((window_step_kernel<N>), dim3((unsigned)ns, (unsigned)w.G), dim3(256), lds, s, w, freq, in, kc, vc, ctl, part, out, ns)
+    const int gq = w.H / w.G;
+    if (gq == 1)
+        GO(1);
+    else if (gq == 2)
+        GO(2);
+    else if (gq <= 4)
+        GO(4);
+    else
+        GO(8);
+#undef GO
+    if (ns > 1) hipLaunchKernelGGL(window_join_kernel, dim3((unsigned)w.H), dim3(256), lds_join, s, w, in, part, out, ns);
     return hipGetLastError();
 }
 

@@ -100,7 +100,7 @@ extern "C" int l2h_layered_create(l2h_ctx *ctx, const l2h_layered_config *cfg, c
             return set_err(ctx, L2H_EINVAL, "layer %d: head sizes %d, %d (1 to 256 are built)", i, d.dim, d.vdim);
         if ((int64_t)d.n_heads * d.vdim > 32768) return set_err(ctx, L2H_EINVAL, "layer %d: heads x value size above 32768", i);
         if (d.mixer == L2H_MIX_ATTENTION) {
-            if (d.window < 1) return set_err(ctx, L2H_EINVAL, "layer %d: window %d", i, d.window);
+            if (d.window < 1 || std::min(d.window, c.seq_len) > 900000) return set_err(ctx, L2H_EINVAL, "layer %d: window %d", i, d.window);
             if (d.rot_dims < 0 || d.rot_dims > d.dim || d.rot_dims % 2) return set_err(ctx, L2H_EINVAL, "layer %d: %d rotated of %d dimensions", i, d.rot_dims, d.dim);
             if (d.rot_dims && !(d.rot_base > 0.0)) return set_err(ctx, L2H_EINVAL, "layer %d: rotation base must be positive", i);
             if (d.rot_original > 0.0 && (!(d.rot_factor > 0.0) || !(d.rot_low > 0.0) || !(d.rot_high > d.rot_low)))
@@ -231,6 +231,7 @@ struct LSlot {
     uint16_t *flat = nullptr;  // bf16, unpadded
     int64_t e0 = 0, e1 = 0;
     bool exp = false;
+    int64_t across = 0;  // a vector of e1 rows stored column by column, this many floats apart
 };
 
 static int layered_slot(l2h_model *m, int role, int layer, int expert, LSlot *s) {
@@ -328,9 +329,12 @@ static int layered_slot(l2h_model *m, int role, int layer, int expert, LSlot *s)
             return L2H_OK;
         case L2H_DECAY_BIAS: vec(L.bias, H * D); return L2H_OK;
         case L2H_MIX_NORM: vec(L.mixnorm, V); return L2H_OK;
-        case L2H_CONV_Q: vec(L.conv, d.taps, G * D); return L2H_OK;
-        case L2H_CONV_K: vec(L.conv + (int64_t)G * D * d.taps, d.taps, G * D); return L2H_OK;
-        case L2H_CONV_V: vec(L.conv + (int64_t)2 * G * D * d.taps, d.taps, H * V); return L2H_OK;
+        case L2H_CONV_Q:
+        case L2H_CONV_K:
+        case L2H_CONV_V:
+            vec(L.conv + (role - L2H_CONV_Q) * G * D, d.taps, role == L2H_CONV_V ? H * V : G * D);
+            t.across = ds.channels();
+            return L2H_OK;
         }
     return set_err(m->ctx, L2H_EINVAL, "layer %d has no tensor \"%s\"", layer, layered_role_name(role));
 }
@@ -355,7 +359,15 @@ int layered_set_tensor(l2h_model *m, int role, int layer, int expert, int type, 
             v[i] = type == L2H_TYPE_F32 ? ((const float *)host)[i] : bf16_value(((const uint16_t *)host)[i]);
             if (s.exp) v[i] = (float)exp((double)v[i]);
         }
-        HIPCHK(ctx, hipMemcpy(s.vec, v.data(), v.size() * 4, hipMemcpyHostToDevice));
+        if (s.across) {  // [channel][tap] -> [tap][channel]
+            std::vector<float> w((size_t)ne1);
+            for (int64_t k = 0; k < ne0; k++) {
+                for (int64_t i = 0; i < ne1; i++) w[(size_t)i] = v[(size_t)(i * ne0 + k)];
+                HIPCHK(ctx, hipMemcpy(s.vec + k * s.across, w.data(), w.size() * 4, hipMemcpyHostToDevice));
+            }
+        } else {
+            HIPCHK(ctx, hipMemcpy(s.vec, v.data(), v.size() * 4, hipMemcpyHostToDevice));
+        }
     } else if (s.flat) {
         HIPCHK(ctx, hipMemcpy(s.flat, host, (size_t)(ne0 * ne1) * 2, hipMemcpyHostToDevice));
     } else {

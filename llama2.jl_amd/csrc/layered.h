@@ -121,7 +121,7 @@ struct DeltaShape {
 #define L_DELTA_COLS 32  // value columns per workgroup of the one-token kernel
 static inline int delta_splits(int V) { return (V + L_DELTA_COLS - 1) / L_DELTA_COLS; }
 struct DeltaWeights {
-    const float *conv;  // [channels][taps]
+    const float *conv;  // [taps][channels], the current token's tap last
     const float *rate, *bias;  // [H], [H D]
     const uint16_t *a2, *g2;
     int lda2, ldg2;
@@ -154,7 +154,7 @@ struct WindowShape {
     __host__ __device__ int off_g() const { return H * D + G * D + G * V; }
     __host__ __device__ int n_in() const { return H * D + G * D + G * V + (gated ? H : 0); }
 };
-#define L_WIN_SPLIT 256  // keys per workgroup of the one-token kernel
+#define L_WIN_SPLIT 64  // keys per workgroup of the one-token kernel (a lane each)
 static inline int window_splits(const WindowShape &w) { return (std::min(w.window, w.seq_len) + L_WIN_SPLIT - 1) / L_WIN_SPLIT; }
 hipError_t k_window_step(hipStream_t s, const WindowShape &w, const float *freq, const float *in, float *kc, float *vc,
                          const DecodeCtl *ctl, float *part, float *out);

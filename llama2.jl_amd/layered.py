@@ -240,3 +240,32 @@ def vudelix_names(config):
 def vudelix_weights(config, tensor):
     """tensor(name) -> array; LayeredWeights with every tensor of the model"""
     return LayeredWeights({key: tensor(name) for name, key in vudelix_names(config).items()})
+
+
+def vudelix_shapes(config):
+    """tensor name -> shape"""
+    W, out = config.width, {}
+    for name in vudelix_names(config):
+        parts = name.split(".")
+        if name in ("embed", "head"):
+            out[name] = (config.vocab_size, W)
+        elif name == "side.embed":
+            out[name] = (config.vocab_size, config.side_dim * config.n_layers)
+        elif parts[-1] in ("norm1", "norm2") or name == "final.norm" or parts[1:] == ["side", "norm"]:
+            out[name] = (W,)
+        elif parts[1] == "side":
+            out[name] = (config.side_dim, W) if parts[2] == "gate" else (W, config.side_dim)
+        elif parts[1] == "mlp":
+            s = config.layers[int(parts[0][1:])]
+            out[name] = (s.n_experts, W) if parts[-1] == "router" else (s.ff_dim, W) if parts[-1] == "up" else (W, s.ff_dim)
+        else:
+            s = config.layers[int(parts[0][1:])]
+            H, G, D, V = s.n_heads, s.n_kv_heads, s.dim, s.vdim
+            qk = G if s.mixer == CHANNEL_DELTA else H
+            vh = H if s.mixer == CHANNEL_DELTA else G
+            n = ".".join(parts[2:])
+            out[name] = {"q": (qk * D, W), "k": (G * D, W), "v": (vh * V, W), "g": (H, W), "o": (W, H * V), "b": (H, W),
+                         "A_log": (H,), "dt_bias": (H * D,), "norm": (V,), "a1": (s.decay_rank, W), "a2": (H * D, s.decay_rank),
+                         "g1": (s.gate_rank, W), "g2": (H * V, s.gate_rank), "q.conv": (qk * D, s.taps), "k.conv": (G * D, s.taps),
+                         "v.conv": (vh * V, s.taps)}[n]
+    return out

@@ -124,3 +124,41 @@ def weight_bytes_per_token(model):
 
 def seeded_prompt(seed, n, vocab_size):
     return np.random.default_rng(seed).integers(0, vocab_size, size=n).astype(np.int32)
+
+
+def layered_model(config, seed=20240607):
+    """A LanguageModel for a LayeredConfig with random bf16 weights: N(0, 1 / inputs) matrices, norms 1, slow decays.  The
+    values of large matrices come from one pool, entered at a different place for every tensor: they are for timing."""
+    from . import layered
+    from .tokenizer import IdTokenizer
+    pool = normal(seed, 0, (1 << 24,), 1.0)
+    rng = np.random.default_rng(seed)
+
+    def bits(a):
+        u = np.ascontiguousarray(a, np.float32).view(np.uint32)
+        return ((u + 0x7FFF + ((u >> 16) & 1)) >> 16).astype(np.uint16)
+
+    scaled = {}
+
+    def matrix(ne1, ne0):
+        if ne0 not in scaled:
+            scaled[ne0] = bits(pool / np.float32(np.sqrt(ne0)))
+        p, n = scaled[ne0], ne1 * ne0
+        if n <= p.size:
+            at = int(rng.integers(0, p.size - n + 1))
+            return p[at:at + n].reshape(ne1, ne0)
+        return np.resize(np.roll(p, -int(rng.integers(0, p.size))), (ne1, ne0))
+
+    shapes = layered.vudelix_shapes(config)
+
+    def tensor(name):
+        last, shape = name.split(".")[-1], shapes[name]
+        if last in ("norm", "norm1", "norm2"):
+            return np.ones(shape, np.float32)
+        if last == "A_log":
+            return np.full(shape, -3.0, np.float32)
+        if last == "dt_bias":
+            return np.full(shape, -2.0, np.float32)
+        return matrix(*shape)
+
+    return LanguageModel(config, IdTokenizer(config.vocab_size), layered.vudelix_weights(config, tensor))

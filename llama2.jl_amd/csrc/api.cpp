@@ -1228,15 +1228,19 @@ static int prefill_expand(l2h_model *m, bool plain) {
     return L2H_OK;
 }
 
-static int prefill_weights(l2h_model *m) {
-    // the library for the plain products: opened once; L2H_PF_LIBRARY=0 keeps every product in this library's kernels
+// the library for the plain products: opened once; L2H_PF_LIBRARY=0 keeps every product in this library's kernels
+static bool prefill_library(l2h_model *m) {
     const char *env = getenv("L2H_PF_LIBRARY");
     const bool want = m->pf_library_mode != 0 && !(env && atoi(env) == 0);
     if (want && !m->pf_lt_tried) {
         m->pf_lt_tried = true;
         m->pf_lt = pf_lt_open(&m->pf_lt_why);
     }
-    const bool plain = want && m->pf_lt != nullptr;
+    return want && m->pf_lt != nullptr;
+}
+
+static int prefill_weights(l2h_model *m) {
+    const bool plain = prefill_library(m);
     if (m->pf_copy_tried) {
         if (m->pf_wbf && plain != m->pf_plain) return prefill_expand(m, plain);
         return L2H_OK;
@@ -1352,6 +1356,7 @@ static int prefill_impl(l2h_model *m, const int32_t *tokens, int n, int pos0, co
     int rc;
     if (m->lay) {
         if ((rc = layered_check_pos(m, pos0)) || (rc = layered_prefill_buffers(m, std::min(n, L2H_PREFILL_CHUNK), n_want))) return rc;
+        if (layered_wants_library(m, n)) (void)prefill_library(m);
     } else {
         if ((rc = prefill_buffers(m, std::min(n, L2H_PREFILL_CHUNK)))) return rc;
         if (m->pf_copy_mode && (rc = prefill_weights(m))) return rc;

@@ -68,6 +68,10 @@ __global__ __launch_bounds__(256) void delta_step_kernel(DeltaShape d, DeltaWeig
     // the first 128 inputs of the low-rank factors' rows are fetched ahead
     const int l8 = t & 7, r8 = t >> 3;
     uint4 fa[NR / 4][2], fg[2];
+    float bias[NR / 4];
+    const float rate = w.rate[h], beta = l_sigmoid(in[d.off_b() + h]);
+#pragma unroll
+    for (int i = 0; i < NR / 4; i++) bias[i] = r8 + 32 * i < D ? w.bias[h * D + r8 + 32 * i] : 0.0f;
 #pragma unroll
     for (int i = 0; i < NR / 4; i++)
 #pragma unroll
@@ -128,8 +132,8 @@ __global__ __launch_bounds__(256) void delta_step_kernel(DeltaShape d, DeltaWeig
         for (int e = 0; e < 2; e++)
             if (8 * l8 + 64 * e < w.lda2) z = delta_fma8(fa[i][e], s_fa + 8 * l8 + 64 * e, z);
         for (int kk = 8 * l8 + 128; kk < w.lda2; kk += 64) z = delta_fma8(*(const uint4 *)(row + kk), s_fa + kk, z);
-        z = delta_sum8(z) + w.bias[h * D + r];
-        if (l8 == 0) s_g[r] = expf(-w.rate[h] * l_softplus(z));
+        z = delta_sum8(z) + bias[i];
+        if (l8 == 0) s_g[r] = expf(-rate * l_softplus(z));
     }
     if (c0 + r8 < V) {
         const uint16_t *row = w.g2 + ((int64_t)h * V + c0 + r8) * w.ldg2;
@@ -167,7 +171,6 @@ __global__ __launch_bounds__(256) void delta_step_kernel(DeltaShape d, DeltaWeig
         dk += s_red[0][i][col];
         dq += s_red[1][i][col];
     }
-    const float beta = l_sigmoid(in[d.off_b() + h]);
     const float u = beta * (s_v[col] - dk), ov = fmaf(s_kq, u, dq);
 #pragma unroll
     for (int i = 0; i < NR; i++) {

@@ -1,7 +1,7 @@
 // Many tokens through a bf16 matrix, C[m][n] = sum_k X[m][k] W[n][k], on the matrix cores: bf16 activations
 // (v_mfma_f32_32x32x16_bf16) or fp32 ones (v_mfma_f32_32x32x2_f32: fp32 operands and sums), with fused epilogues and a grouped
 // form for mixtures of experts; and the row-wise kernels around the products.
-#include "layered_dev.h"
+#include "layered_gemm.h"
 
 typedef __bf16 l_bf16x8 __attribute__((ext_vector_type(8)));
 typedef float l_f32x16 __attribute__((ext_vector_type(16)));
@@ -9,48 +9,6 @@ typedef float l_f32x16 __attribute__((ext_vector_type(16)));
 // Placement of the 16-byte chunks of a 128-byte tile row: 16 consecutive rows' chunks of one index fall into different slots
 // of the 256-byte bank row.
 __device__ __forceinline__ int gemm_swz(int r) { return (r >> 1) & 7; }
-
-// Results of a wavefront: lane holds position mi = 32 j + lane % 32 of its block and, in register 4 rq + e of tile i, weight row
-// 32 i + 8 rq + 4 (lane / 32) + e.
-template <int PREC, int EPI>
-__device__ __forceinline__ void gemm_store4(const GemmArgs &a, int64_t m, int64_t L, float v0, float v1, float v2, float v3) {
-    float v[4] = {v0, v1, v2, v3};
-    if (EPI == GE_STORE || EPI == GE_RESID || EPI == GE_DECAY || EPI == GE_SIGMOID) {
-        if (L >= a.n_rows) return;
-        float *o = a.outf + m * a.ldo + L;
-#pragma unroll
-        for (int e = 0; e < 4; e++) {
-            if (L + e >= a.n_rows) break;
-            if (EPI == GE_RESID)
-                o[e] = fmaf(a.mult, v[e], o[e]);
-            else if (EPI == GE_DECAY)
-                o[e] = -a.rate[(L + e) / a.hd] * l_softplus(v[e] + a.bias[L + e]);
-            else if (EPI == GE_SIGMOID)
-                o[e] = l_sigmoid(v[e]);
-            else
-                o[e] = v[e];
-        }
-    } else {
-        if (L >= a.lda) return;  // (lda a multiple of 64: whole groups of four)
-#pragma unroll
-        for (int e = 0; e < 4; e++) {
-            if (L + e >= a.n_rows) {
-                v[e] = 0.0f;
-                continue;
-            }
-            if (EPI == GE_UP)
-                v[e] = l_act(a.act, a.row_scale[m] * v[e]);
-            else if (EPI == GE_EMBED)
-                v[e] = l_act(a.act, v[e]) * l_bf16(a.emb[(int64_t)a.tokens[m] * a.emb_ld + L + e]);
-            else
-                v[e] = l_act(a.act, v[e]);
-        }
-        if (PREC)
-            *(float4 *)((float *)a.outa + m * a.lda + L) = make_float4(v[0], v[1], v[2], v[3]);
-        else
-            *(uint2 *)((uint16_t *)a.outa + m * a.lda + L) = make_uint2(l_pack_bf16(v[0], v[1]), l_pack_bf16(v[2], v[3]));
-    }
-}
 
 template <int PREC, int EPI, int TN, int TM, bool GROUPED>
 __global__ __launch_bounds__(256) void gemm_kernel(GemmArgs a) {
@@ -368,5 +326,23 @@ __global__ __launch_bounds__(256) void gather_add_kernel(float *x, const float *
 }
 hipError_t k_gather_add(hipStream_t s, float *x, const float *y, const int32_t *slot_of, int M, int top, int K, float mult) {
     hipLaunchKernelGGL(gather_add_kernel, dim3((unsigned)((K + 255) / 256), (unsigned)M), dim3(256), 0, s, x, y, slot_of, top, K, mult);
+    return hipGetLastError();
+}
+
+template <int PREC>
+__global__ __launch_bounds__(256) void embed_rows_kernel(const float *v, int N, int act, const uint16_t *emb, int64_t emb_ld,
+                                                         const int32_t *tokens, void *outa, int64_t lda) {
+    const int64_t m = blockIdx.y;
+    const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+    if (i >= lda) return;
+    l_store_act<PREC>(outa, m * lda + i, i < N ? l_act(act, v[m * N + i]) * l_bf16(emb[(int64_t)tokens[m] * emb_ld + i]) : 0.0f);
+}
+hipError_t k_embed_rows(hipStream_t s, const float *v, int M, int N, int act, const uint16_t *emb, int64_t emb_ld,
+                        const int32_t *tokens, void *outa, int64_t lda, int prec) {
+    const dim3 grid((unsigned)((lda + 255) / 256), (unsigned)M);
+    if (prec)
+        hipLaunchKernelGGL((embed_rows_kernel<1>), grid, dim3(256), 0, s, v, N, act, emb, emb_ld, tokens, outa, lda);
+    else
+        hipLaunchKernelGGL((embed_rows_kernel<0>), grid, dim3(256), 0, s, v, N, act, emb, emb_ld, tokens, outa, lda);
     return hipGetLastError();
 }

@@ -6,18 +6,8 @@
 // The reference has no batched path; the result is defined as what its per-token loop would leave
 // in the KV cache and the last position's logits, to bf16 accuracy.
 #include "matvec_dev.h"
+#include "pf_tile.h"
 
-typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
-typedef __bf16 bf16x2 __attribute__((ext_vector_type(2)));
-typedef float f32x16 __attribute__((ext_vector_type(16)));
-
-__device__ __forceinline__ uint32_t pack_bf16(float a, float b) {
-    bf16x2 v;
-    v.x = (__bf16)a;
-    v.y = (__bf16)b;
-    return __builtin_bit_cast(uint32_t, v);
-}
-__device__ __forceinline__ bf16x8 as_bf16x8(uint4 v) { return __builtin_bit_cast(bf16x8, v); }
 
 // ------------------------------------------------------------------------------------------
 // small per-position kernels
@@ -297,12 +287,6 @@ __device__ __forceinline__ void pf_convert(const PfRaw &r, const PfRowPtr &p, in
     for (int c = 0; c < 4; c++) out[c] = make_uint4(pk[4 * c], pk[4 * c + 1], pk[4 * c + 2], pk[4 * c + 3]);
 }
 
-// Placement of the 16-byte chunks of a 128-byte tile row in LDS.  The LDS has 64 banks of 4 bytes and serves
-// 16-byte accesses 16 lanes at a time; lanes read one chunk index of 16 consecutive rows, which the
-// exclusive-or with (r >> 1) % 8 sends to the 16 different 16-byte slots of the 256-byte bank row (the row's
-// parity picks the half).  With r % 8 instead, rows r and r + 8 collide: half the LDS cycles were conflicts.
-__host__ __device__ __forceinline__ int pf_swz(int r) { return (r >> 1) & 7; }
-
 // the stream pointers of logical weight row L
 template <int TYPE>
 __device__ __forceinline__ void pf_row_ptr(const PfGemmArgs &a, int64_t L, PfRow &lr, PfRowPtr &rp) {
@@ -491,162 +475,20 @@ __global__ __launch_bounds__(256) void pf_gemm_kernel(PfGemmArgs a) {
     pf_epilogue<EPI, JT>(a, acc, n0, m0, wn, wm, lane);
 }
 
-#define PF_AS1 __attribute__((address_space(1)))
-#define PF_AS3 __attribute__((address_space(3)))
 
-// The same product from weights expanded beforehand (pf_expand_kernel): no arithmetic on the operands.
-// The tile is 256 weight rows x 64 JT positions (JT = 4: 256 positions, 64 KB fetched per 64 inputs, half
-// the bytes per product of a 128 x 128 tile; JT = 2: 128 positions, for matrices with too few rows to give
-// every CU a 256 x 256 tile), worked on by 8 wavefronts, 4 row groups x 2 position groups, each 64 rows x
-// 32 JT positions.  Both operand tiles of a K step travel from global memory
-// straight into LDS (16 bytes per lane and load, a wavefront's load filling 1 KB in lane order): the weight
-// tile is a linear copy of its 32 KB image, the position tile gets the c ^ pf_swz(r) placement by the choice
-// of the address each lane reads.  Two LDS stages: the loads of step kt + 1 are in flight during the products
-// of step kt, one barrier per step.  Workgroups are dealt to the 8 XCDs in turn, so workgroup w takes tile
-// (w % 8) * per + w / 8: each XCD works through a contiguous run of tiles, positions fastest, and the
-// workgroups that share a weight tile share an L2.
-typedef uint32_t pf_u32x4 __attribute__((ext_vector_type(4)));
+// The same product from weights expanded beforehand (pf_expand_kernel), tile by tile (pf_tile.h).  Workgroups are dealt to
+// the 8 XCDs in turn, so workgroup w takes tile (w % 8) * per + w / 8: each XCD works through a contiguous run of tiles,
+// positions fastest, and the workgroups that share a weight tile share an L2.
 
 // the tile (row group nt, position block mt) of one workgroup; s_all: two stages of LDS
 template <int EPI, int JT>
 __device__ __forceinline__ void pf_gemm_bf16_tile(const PfGemmArgs &a, unsigned nt, unsigned mt, uint4 *s_all) {
-    constexpr int MT = 64 * JT;                   // positions per workgroup
-    constexpr int STAGE = 32768 + MT * 128;       // bytes: weight tile, then position tile
-    const int t = threadIdx.x, lane = t & 63, wave = __builtin_amdgcn_readfirstlane(t >> 6), wn = wave & 3, wm = wave >> 2;
     const int64_t n0 = (int64_t)nt * 256;
-    const int m0 = (int)mt * MT;
-    const int64_t K = a.K, nk = K >> 6;
-
-    // weights: this wavefront copies bytes [4096 wave, +4096) of every tile, 1 KB per load
-    const unsigned char *gw = (const unsigned char *)(a.wbf + (int64_t)nt * nk * 16384) + wave * 4096 + lane * 16;
-    // positions: load i of this wavefront fills chunks 64 (JT wave + i) + lane: row 8 (JT wave + i) + lane / 8,
-    // placed chunk lane % 8 = the data chunk (lane % 8) ^ pf_swz(row)
-    const unsigned char *gx[JT];
-#pragma unroll
-    for (int i = 0; i < JT; i++) {
-        const int r = 8 * (JT * wave + i) + (lane >> 3);
-        int m = m0 + r;
-        m = m < a.M ? m : a.M - 1;  // rows past the end repeat the last one; their results are not stored
-        gx[i] = (const unsigned char *)(a.act + (int64_t)m * K + 8 * ((lane & 7) ^ pf_swz(r)));
-    }
-    // LDS byte offsets of this lane's operands inside a stage: slice kk holds chunk 2 kk + lane / 32 of its rows
-    unsigned aw[2][4], ax[JT][4];
-#pragma unroll
-    for (int kk = 0; kk < 4; kk++) {
-        const int c = 2 * kk + (lane >> 5);
-#pragma unroll
-        for (int i = 0; i < 2; i++) {
-            const int ra = 64 * wn + 32 * i + (lane & 31);
-            aw[i][kk] = 16u * (unsigned)(ra * 8 + (c ^ pf_swz(ra)));
-        }
-#pragma unroll
-        for (int j = 0; j < JT; j++) {
-            const int rb = 32 * JT * wm + 32 * j + (lane & 31);
-            ax[j][kk] = 32768u + 16u * (unsigned)(rb * 8 + (c ^ pf_swz(rb)));
-        }
-    }
-    const unsigned lds0 = (unsigned)(size_t)s_all;
-
-    f32x16 acc[2][JT];
-#pragma unroll
-    for (int i = 0; i < 2; i++)
-#pragma unroll
-        for (int j = 0; j < JT; j++)
-#pragma unroll
-            for (int r = 0; r < 16; r++) acc[i][j][r] = 0.0f;
-
-    auto issue = [&](int stage) {
-        unsigned char *lw = (unsigned char *)s_all + stage * STAGE + wave * 4096;
-        unsigned char *lx = (unsigned char *)s_all + stage * STAGE + 32768 + wave * (1024 * JT);
-        __builtin_amdgcn_global_load_lds((const PF_AS1 void *)gw, (PF_AS3 void *)lw, 16, 0, 0);
-        __builtin_amdgcn_global_load_lds((const PF_AS1 void *)gw, (PF_AS3 void *)lw, 16, 1024, 0);
-        __builtin_amdgcn_global_load_lds((const PF_AS1 void *)gw, (PF_AS3 void *)lw, 16, 2048, 0);
-        __builtin_amdgcn_global_load_lds((const PF_AS1 void *)gw, (PF_AS3 void *)lw, 16, 3072, 0);
-#pragma unroll
-        for (int i = 0; i < JT; i++) {
-            __builtin_amdgcn_global_load_lds((const PF_AS1 void *)gx[i], (PF_AS3 void *)(lx + 1024 * i), 16, 0, 0);
-            gx[i] += 128;
-        }
-        gw += 32768;
-    };
-
-    // The operands of a 16-wide slice (2 weight groups, JT position groups) are read from LDS one slice ahead
-    // of the products that use them, into two register sets used in turn, so that a wavefront's LDS latency
-    // lies under its own products.  Reads and waits are asm: the compiler then does not make them wait for the
-    // copies in flight into the other stage.  Between a PF_READ and the PF_WAIT that retires it the registers
-    // of the set hold nothing yet: the set only appears as an operand of those two statements and of the
-    // products after the wait (LDS reads complete in order, so lgkmcnt(2 + JT) retires all but the newest set;
-    // the build's asm check walks the generated code for any other touch of such a register).
-    pf_u32x4 F0[2 + JT], F1[2 + JT];
-#define PF_READ(F, KK)                                                                                            \
-    do {                                                                                                          \
-        if constexpr (JT == 2)                                                                                    \
-            asm volatile("ds_read_b128 %0, %4\n\tds_read_b128 %1, %5\n\tds_read_b128 %2, %6\n\tds_read_b128 %3, %7"  \
-                         : "=&v"(F[0]), "=&v"(F[1]), "=&v"(F[2]), "=&v"(F[3])                                     \
-                         : "v"(sb + aw[0][KK]), "v"(sb + aw[1][KK]), "v"(sb + ax[0][KK]), "v"(sb + ax[1][KK])     \
-                         : "memory");                                                                             \
-        else                                                                                                      \
-            asm volatile("ds_read_b128 %0, %6\n\tds_read_b128 %1, %7\n\tds_read_b128 %2, %8\n\tds_read_b128 %3, %9"  \
-                         "\n\tds_read_b128 %4, %10\n\tds_read_b128 %5, %11"                                       \
-                         : "=&v"(F[0]), "=&v"(F[1]), "=&v"(F[2]), "=&v"(F[3]), "=&v"(F[4]), "=&v"(F[5])           \
-                         : "v"(sb + aw[0][KK]), "v"(sb + aw[1][KK]), "v"(sb + ax[0][KK]), "v"(sb + ax[1][KK]),    \
-                           "v"(sb + ax[JT - 2][KK]), "v"(sb + ax[JT - 1][KK])                                     \
-                         : "memory");                                                                             \
-    } while (0)
-    // LAST: nothing newer is in flight
-#define PF_WAIT(F, LAST)                                                                                          \
-    do {                                                                                                          \
-        if constexpr (JT == 2) {                                                                                  \
-            if (LAST)                                                                                             \
-                asm volatile("s_waitcnt lgkmcnt(0)" : "+v"(F[0]), "+v"(F[1]), "+v"(F[2]), "+v"(F[3])::"memory");  \
-            else                                                                                                  \
-                asm volatile("s_waitcnt lgkmcnt(4)" : "+v"(F[0]), "+v"(F[1]), "+v"(F[2]), "+v"(F[3])::"memory");  \
-        } else {                                                                                                  \
-            if (LAST)                                                                                             \
-                asm volatile("s_waitcnt lgkmcnt(0)"                                                               \
-                             : "+v"(F[0]), "+v"(F[1]), "+v"(F[2]), "+v"(F[3]), "+v"(F[JT]), "+v"(F[JT + 1])::"memory"); \
-            else                                                                                                  \
-                asm volatile("s_waitcnt lgkmcnt(6)"                                                               \
-                             : "+v"(F[0]), "+v"(F[1]), "+v"(F[2]), "+v"(F[3]), "+v"(F[JT]), "+v"(F[JT + 1])::"memory"); \
-        }                                                                                                         \
-    } while (0)
-#define PF_PRODUCTS(F)                                                                                            \
-    do {                                                                                                          \
-        const bf16x8 W0 = __builtin_bit_cast(bf16x8, F[0]), W1 = __builtin_bit_cast(bf16x8, F[1]);                \
-        _Pragma("unroll") for (int j = 0; j < JT; j++) {                                                          \
-            const bf16x8 P = __builtin_bit_cast(bf16x8, F[2 + j]);                                                \
-            acc[0][j] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(W0, P, acc[0][j], 0, 0, 0);                       \
-            acc[1][j] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(W1, P, acc[1][j], 0, 0, 0);                       \
-        }                                                                                                         \
-    } while (0)
-
-    issue(0);
-    for (int64_t kt = 0; kt < nk; kt++) {
-        const int stage = (int)(kt & 1);
-        // this wavefront's loads of the stage have landed; the barrier says the same of the others' and that
-        // everyone is done reading the other stage (its last PF_WAIT retired every read), which the next loads
-        // then overwrite
-        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-        __builtin_amdgcn_s_barrier();
-        if (kt + 1 < nk) issue(stage ^ 1);
-        const unsigned sb = lds0 + (unsigned)(stage * STAGE);
-        PF_READ(F0, 0);
-        PF_READ(F1, 1);
-        PF_WAIT(F0, false);
-        PF_PRODUCTS(F0);
-        PF_READ(F0, 2);
-        PF_WAIT(F1, false);
-        PF_PRODUCTS(F1);
-        PF_READ(F1, 3);
-        PF_WAIT(F0, false);
-        PF_PRODUCTS(F0);
-        PF_WAIT(F1, true);
-        PF_PRODUCTS(F1);
-    }
-#undef PF_PRODUCTS
-#undef PF_WAIT
-#undef PF_READ
-    pf_epilogue<EPI, JT>(a, acc, n0, m0, wn, wm, lane);
+    const int m0 = (int)mt * 64 * JT;
+    pf_tile_product<JT>(
+        a.wbf + (int64_t)nt * (a.K >> 6) * 16384, a.act, a.K, s_all,
+        [&](int r) { return (int64_t)min(m0 + r, a.M - 1); },  // rows past the end repeat the last one; their results are not stored
+        [&](f32x16(&acc)[2][JT], int wn, int wm, int lane) { pf_epilogue<EPI, JT>(a, acc, n0, m0, wn, wm, lane); });
 }
 
 // row groups nt0 .. in tiles of 64 JT positions
@@ -704,17 +546,17 @@ struct PfKvTile {
 
 template <int HS>
 __global__ __launch_bounds__(256) void pf_kv_tiles_kernel(const float *kc, const float *vc, unsigned char *tiles,
-                                                          int seq_len, int n_tiles_max) {
+                                                          int seq_len, int n_tiles_max, int tile0, int kq, int vd) {
     typedef PfKvTile<HS> T;
     __shared__ __align__(16) unsigned char s_img[T::BYTES];
     unsigned char *s_k = s_img, *s_v = s_img + T::K_BYTES;
-    const int t = threadIdx.x, kt = blockIdx.x, kvh = blockIdx.y, key0 = 32 * kt;
+    const int t = threadIdx.x, kt = blockIdx.x, kvh = blockIdx.y, key0 = 32 * (tile0 + kt);
     for (int c = t; c < T::BYTES / 16; c += 256) ((uint4 *)s_img)[c] = make_uint4(0, 0, 0, 0);
     __syncthreads();
     for (int idx = t; idx < 32 * (HS / 4); idx += 256) {  // K tile -> bf16 rows
         const int key = idx & 31, i4 = idx >> 5;
         float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
-        if (key0 + key < seq_len) v = *(const float4 *)(kc + (((int64_t)kvh * (HS / 4) + i4) * seq_len + key0 + key) * 4);
+        if (key0 + key < seq_len && i4 < kq) v = *(const float4 *)(kc + (((int64_t)kvh * kq + i4) * seq_len + key0 + key) * 4);
         uint2 w;
         w.x = pack_bf16(v.x, v.y);
         w.y = pack_bf16(v.z, v.w);
@@ -723,7 +565,17 @@ __global__ __launch_bounds__(256) void pf_kv_tiles_kernel(const float *kc, const
     for (int idx = t; idx < 32 * (HS / 4); idx += 256) {  // V tile -> bf16, transposed, keys permuted
         const int d4 = idx % (HS / 4), key = idx / (HS / 4);
         float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
-        if (key0 + key < seq_len) v = *(const float4 *)(vc + ((int64_t)kvh * seq_len + key0 + key) * HS + 4 * d4);
+        if (key0 + key < seq_len && 4 * d4 < vd) {
+            const float *src = vc + ((int64_t)kvh * seq_len + key0 + key) * vd + 4 * d4;
+            if (vd % 4 == 0) {
+                v = *(const float4 *)src;
+            } else {
+                v.x = src[0];
+                v.y = 4 * d4 + 1 < vd ? src[1] : 0.f;
+                v.z = 4 * d4 + 2 < vd ? src[2] : 0.f;
+                v.w = 4 * d4 + 3 < vd ? src[3] : 0.f;
+            }
+        }
         // key = 16 s + 8 a + 4 g + b  ->  slot 16 s + 8 g + 4 a + b
         const int rem = key & 15;
         const int slot = (key & 16) + 8 * ((rem >> 2) & 1) + 4 * (rem >> 3) + (rem & 3);
@@ -784,10 +636,13 @@ __device__ __forceinline__ float pf_other_half(float x) {
     return (threadIdx.x & 32) ? __uint_as_float(r[0]) : __uint_as_float(r[1]);
 }
 
-template <int HS>
+// WIN: position i sees the keys i - window + 1 .. i only; the tiles start with tile `tile0` of the sequence (32 keys each); the
+// scale of the scores, the value size (<= HS), a gate per head (sigmoid of gate[m * ldg + h]) and the output's row stride, whose
+// columns beyond the heads are zeroed, are the caller's.
+template <int HS, bool WIN>
 __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void pf_attn_kernel(const uint16_t *Qb, uint16_t *Att, const unsigned char *tiles,
                                                       int n_tiles_max, int M, int qpos0, int n_heads, int n_kv, int dim,
-                                                      unsigned n_qb, unsigned n_items, unsigned per) {
+                                                      unsigned n_qb, unsigned n_items, unsigned per, PfWindow win) {
     typedef PfKvTile<HS> T;
     constexpr int KSTEPS = HS / 16, DT = HS / 32, KH = KSTEPS / 2;
     // two stages: the copy of tile kt + 1 is in flight during the products of tile kt, one barrier per tile
@@ -820,8 +675,9 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void p
         for (int r = 0; r < 16; r++) o[d][r] = 0.0f;
     float mrun = -INFINITY, lrun = 0.0f;
     const int wave_qmax = min(M - 1, q0 + 32 * wave + 31), wg_qmax = min(M - 1, q0 + 127);
-    const int nkt = (qpos0 + wg_qmax) / 32 + 1;
-    const float c_log2 = 1.44269504088896341f / sqrtf((float)HS);
+    const int kt0 = WIN ? max(0, qpos0 + q0 - win.window + 1) / 32 - win.tile0 : 0;
+    const int nkt = (qpos0 + wg_qmax) / 32 + 1 - (WIN ? win.tile0 : 0);
+    const float c_log2 = 1.44269504088896341f * (WIN ? win.scale : 1.0f / sqrtf((float)HS));
     const unsigned char *src = tiles + (int64_t)kvh * n_tiles_max * T::BYTES + lane * 16;
     const unsigned lds0 = (unsigned)(size_t)s_t;
     const unsigned k_addr = lds0 + (unsigned)(ql * T::KROW + 16 * g), v_addr = lds0 + (unsigned)(T::K_BYTES + ql * T::VROW + 16 * g);
@@ -835,13 +691,14 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void p
                 __builtin_amdgcn_global_load_lds((const PF_AS1 void *)(gp + (b + wave) * 1024),
                                                  (PF_AS3 void *)(lp + (b + wave) * 1024), 16, 0, 0);
     };
-    issue(0, 0);
-    for (int kt = 0; kt < nkt; kt++) {
-        const int key0 = 32 * kt, stage = kt & 1;
+    issue(kt0 & 1, kt0);
+    for (int kt = kt0; kt < nkt; kt++) {
+        const int key0 = 32 * (kt + (WIN ? win.tile0 : 0)), stage = kt & 1;
         asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // this wavefront's part of the tile has landed
         __syncthreads();                                  // ... and everyone's; the other stage is free
         if (kt + 1 < nkt) issue(stage ^ 1, kt + 1);
         if (key0 > qpos0 + wave_qmax) continue;  // every key of the tile lies in this wavefront's future
+        if (WIN && key0 + 31 <= qpos0 + q0 + 32 * wave - win.window) continue;  // ... or before every window
         const unsigned so = (unsigned)(stage * T::BYTES);
         f32x16 s;
 #pragma unroll
@@ -866,13 +723,14 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void p
         // (att ./= sqrt(hs); softmax!, src/inference.jl:268-270); only a tile on the diagonal needs the mask
         float tmax = -INFINITY;
         // (wavefront-uniform: the tile reaches past the first query of the wavefront, or some query is past M)
-        const bool diagonal = key0 + 31 > qpos0 + q0 + 32 * wave || q0 + 32 * wave + 31 >= M;
+        const bool diagonal = key0 + 31 > qpos0 + q0 + 32 * wave || q0 + 32 * wave + 31 >= M ||
+                              (WIN && key0 <= qpos0 + q0 + 32 * wave + 31 - win.window);
         if (diagonal) {
 #pragma unroll
             for (int r = 0; r < 16; r++) {
                 const int key = key0 + 8 * (r >> 2) + 4 * g + (r & 3);
                 float v = s[r] * c_log2;
-                if (!qvalid || key > qpos0 + myq) v = -INFINITY;
+                if (!qvalid || key > qpos0 + myq || (WIN && key <= qpos0 + myq - win.window)) v = -INFINITY;
                 s[r] = v;
                 tmax = fmaxf(tmax, v);
             }
@@ -923,6 +781,29 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void p
         }
     }
     if (!qvalid) return;
+    if constexpr (WIN) {
+        float f = 1.0f / lrun;
+        if (win.gate) f /= 1.0f + expf(-win.gate[(int64_t)myq * win.ldg + h]);
+        __bf16 *row = (__bf16 *)Att + (int64_t)myq * win.ldo + (int64_t)h * win.vdim;
+#pragma unroll
+        for (int d = 0; d < DT; d++)
+#pragma unroll
+            for (int rq = 0; rq < 4; rq++) {
+                const int e = 32 * d + 8 * rq + 4 * g;
+                if (win.vdim % 4 == 0) {
+                    if (e < win.vdim)
+                        *(uint2 *)(row + e) = make_uint2(pack_bf16(o[d][4 * rq] * f, o[d][4 * rq + 1] * f),
+                                                         pack_bf16(o[d][4 * rq + 2] * f, o[d][4 * rq + 3] * f));
+                } else {
+#pragma unroll
+                    for (int b = 0; b < 4; b++)
+                        if (e + b < win.vdim) row[e + b] = (__bf16)(o[d][4 * rq + b] * f);
+                }
+            }
+        if (h == n_heads - 1 && g == 0)
+            for (int64_t i = (int64_t)n_heads * win.vdim; i < win.ldo; i++) ((__bf16 *)Att)[(int64_t)myq * win.ldo + i] = (__bf16)0.0f;
+        return;
+    }
     const float inv = 1.0f / lrun;
 #pragma unroll
     for (int d = 0; d < DT; d++)
@@ -1145,10 +1026,13 @@ int64_t k_pf_kv_tile_bytes(int hs) {
 
 // tiles: n_kv x n_tiles_max tiles of k_pf_kv_tile_bytes(hs); the first n_tiles of every KV head are rewritten
 hipError_t k_pf_kv_tiles(hipStream_t s, const float *kc, const float *vc, unsigned char *tiles, int n_tiles,
-                         int n_tiles_max, int hs, int n_kv, int seq_len) {
+                         int n_tiles_max, int hs, int n_kv, int seq_len, int tile0, int kdim, int vdim) {
+    if (kdim == 0) kdim = vdim = hs;
+    if (kdim % 4 != 0 || kdim > hs || vdim > hs || tile0 < 0) return hipErrorInvalidValue;
+    const int kq = kdim / 4;
     if (n_tiles < 1 || n_tiles > n_tiles_max) return hipErrorInvalidValue;
     const dim3 grid((unsigned)n_tiles, (unsigned)n_kv);
-#define GO(HS) hipLaunchKernelGGL((pf_kv_tiles_kernel<HS>), grid, dim3(256), 0, s, kc, vc, tiles, seq_len, n_tiles_max)
+#define GO(HS) hipLaunchKernelGGL((pf_kv_tiles_kernel<HS>), grid, dim3(256), 0, s, kc, vc, tiles, seq_len, n_tiles_max, tile0, kq, vdim)
     switch (hs) {
     case 32: GO(32); break;
     case 64: GO(64); break;
@@ -1162,12 +1046,23 @@ hipError_t k_pf_kv_tiles(hipStream_t s, const float *kc, const float *vc, unsign
 
 // tiles must hold the keys 0 .. qpos0 + M - 1 (k_pf_kv_tiles)
 hipError_t k_pf_attention(hipStream_t s, const uint16_t *Qb, uint16_t *Att, const unsigned char *tiles, int n_tiles_max,
-                          int M, int qpos0, int hs, int n_heads, int n_kv, int dim) {
-    if ((qpos0 + M + 31) / 32 > n_tiles_max) return hipErrorInvalidValue;
+                          int M, int qpos0, int hs, int n_heads, int n_kv, int dim, const PfWindow *win) {
+    const PfWindow w = win ? *win : PfWindow{};
+    if ((qpos0 + M + 31) / 32 - w.tile0 > n_tiles_max) return hipErrorInvalidValue;
+    if (win && (w.window < 1 || w.vdim > hs || w.ldo < (int64_t)n_heads * w.vdim || w.ldo % 4 != 0 ||
+                32 * w.tile0 > std::max(0, qpos0 - w.window + 1)))
+        return hipErrorInvalidValue;
     const unsigned n_qb = (unsigned)((M + 127) / 128), n_items = n_qb * (unsigned)n_heads, per = (n_items + 7) / 8;
     const dim3 grid(8 * per);
-#define GO(HS) \
-    hipLaunchKernelGGL((pf_attn_kernel<HS>), grid, dim3(256), 0, s, Qb, Att, tiles, n_tiles_max, M, qpos0, n_heads, n_kv, dim, n_qb, n_items, per)
+#define GO(HS)                                                                                                                          \
+    do {                                                                                                                                \
+        if (win)                                                                                                                        \
+            hipLaunchKernelGGL((pf_attn_kernel<HS, true>), grid, dim3(256), 0, s, Qb, Att, tiles, n_tiles_max, M, qpos0, n_heads, n_kv, \
+                               dim, n_qb, n_items, per, w);                                                                             \
+        else                                                                                                                            \
+            hipLaunchKernelGGL((pf_attn_kernel<HS, false>), grid, dim3(256), 0, s, Qb, Att, tiles, n_tiles_max, M, qpos0, n_heads,      \
+                               n_kv, dim, n_qb, n_items, per, w);                                                                       \
+    } while (0)
     switch (hs) {
     case 32: GO(32); break;
     case 64: GO(64); break;

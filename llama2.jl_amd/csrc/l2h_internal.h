@@ -258,20 +258,29 @@ hipError_t k_pf_gemm(hipStream_t s, const DevTensor *w, int nseg, int interleave
 // plain: rows of K bf16 values one after the other (what pf_lt_gemm multiplies from) instead of the product kernels' tiles
 hipError_t k_pf_expand(hipStream_t s, const DevTensor *w, int nseg, int interleave, int64_t K, uint16_t *dst,
                        int64_t dst_row0, int pad, int plain);
-// hipBLASLt for the plain products of the prompt pass (pf_lt.cpp): D[M][0..N) (fp32, row stride ldd) = X[M][K] W[N][K]^T
+// hipBLASLt for the plain products of the prompt pass (pf_lt.cpp): D[M][0..N) (fp32, row stride ldd) = alpha X[M][K] W[N][K]^T
 // (+ D if accumulate), bf16 operands, fp32 sums.  pf_lt_open returns nullptr, and says why, where the library cannot be used.
 // pf_lt_gemm with D == nullptr only prepares the shape (hipErrorNotSupported: the library has no algorithm for it).
 struct PfLt;
 PfLt *pf_lt_open(std::string *why);
 void pf_lt_close(PfLt *lt);
 hipError_t pf_lt_gemm(PfLt *lt, hipStream_t s, const uint16_t *W, const uint16_t *X, float *D, int M, int64_t N, int64_t K,
-                      int64_t ldd, bool accumulate, std::string *err);
+                      int64_t ldd, bool accumulate, std::string *err, float alpha = 1.0f);
 bool k_pf_attention_supported(int hs);
 int64_t k_pf_kv_tile_bytes(int hs);
+// tiles tile0 .. tile0 + n_tiles - 1 of the sequence (32 keys each), at the start of the buffer; kdim / vdim: elements of a key
+// (a multiple of 4) and of a value where they are fewer than hs, the rest being zero
 hipError_t k_pf_kv_tiles(hipStream_t s, const float *kc, const float *vc, unsigned char *tiles, int n_tiles,
-                         int n_tiles_max, int hs, int n_kv, int seq_len);
+                         int n_tiles_max, int hs, int n_kv, int seq_len, int tile0 = 0, int kdim = 0, int vdim = 0);
+// a sliding window for k_pf_attention (see pf_attn_kernel)
+struct PfWindow {
+    int window = 0, tile0 = 0, vdim = 0;
+    float scale = 0.0f;
+    const float *gate = nullptr;  // head gates' logits, or nullptr
+    int64_t ldg = 0, ldo = 0;
+};
 hipError_t k_pf_attention(hipStream_t s, const uint16_t *Qb, uint16_t *Att, const unsigned char *tiles, int n_tiles_max,
-                          int M, int qpos0, int hs, int n_heads, int n_kv, int dim);
+                          int M, int qpos0, int hs, int n_heads, int n_kv, int dim, const PfWindow *win = nullptr);
 
 static inline int64_t l2h_gguf_block_bytes(int type) {
     switch (type) {

@@ -30,7 +30,6 @@ struct Layered {
     uint16_t *side_emb = nullptr;
     float *final_norm = nullptr;
     uint64_t have = 0;
-    bool state_uncleared = false;
     int pos = 0;  // positions the state has taken in
     // one token
     float *x_alt = nullptr, *in = nullptr, *mix = nullptr, *ssq = nullptr, *gate = nullptr, *hid = nullptr, *z = nullptr,
@@ -45,6 +44,8 @@ struct Layered {
     int want_cap = 0;
     // residual stream after every layer of the last prompt pass (l2h_layered_keep)
     bool keep = false;
+    bool images_tried = false;
+    unsigned char *kvt = nullptr;  // one attention layer's keys and values as the attention kernel's tiles
     float *kept = nullptr;
     int kept_cap = 0, kept_n = 0;
 
@@ -70,6 +71,17 @@ static DeltaShape delta_shape(const Layered *l, const LayerDev &L) {
 }
 static int mixer_rows(const Layered *l, const LayerDev &L) {
     return L.d.mixer == L2H_MIX_ATTENTION ? window_shape(l, L).n_in() : delta_shape(l, L).n_in();
+}
+
+// head size of the matrix-core attention kernel that holds this layer's heads (0: none does), and the tiles of 32 keys that a
+// chunk of `cap` positions can see
+static int attention_tile_size(const l2h_layer &d) {
+    for (int hs : {32, 64, 96, 128})
+        if (std::max((d.dim + 3) / 4 * 4, d.vdim) <= hs) return hs;
+    return 0;
+}
+static int attention_tiles(const Layered *l, const LayerDev &L, int cap) {
+    return (int)std::min<int64_t>(((int64_t)l->c.seq_len + 31) / 32, ((int64_t)L.d.window + cap) / 32 + 2);
 }
 
 static int mat_alloc(l2h_model *m, LMat *t, int64_t rows, int K) {
@@ -617,10 +629,53 @@ hipError_t layered_enqueue_token(l2h_model *m) {
 // ------------------------------------------------------------------------------------------
 // prompt pass
 // ------------------------------------------------------------------------------------------
+// The matrices whose products have arithmetic behind them or are grouped (dense up, experts) get a second copy as tile images
+// for the matrix-core kernel of the prompt pass, made once, where it fits beside 2 GiB of free memory.
+#define L_IMAGE_MIN_ROWS 192  // a row group of an image is 256 rows: smaller matrices stay with k_gemm
+#define L_BIG_MIN_M 128       // positions from which the library and the images are used
+static int prompt_images(l2h_model *m) {
+    Layered *l = m->lay;
+    if (l->images_tried || l->c.precision || !m->pf_copy_mode) return L2H_OK;
+    l->images_tried = true;
+    struct Job {
+        LMat *w;
+        int64_t rows, n;
+    };
+    std::vector<Job> jobs;
+    int64_t elems = 0;
+    auto add = [&](LMat *w, int64_t rows, int64_t n) {
+        if (rows < L_IMAGE_MIN_ROWS) return;
+        jobs.push_back(Job{w, rows, n});
+        elems += n * k_tile_image_elems(rows, w->ld);
+    };
+    for (LayerDev &L : l->layer) {
+        if (L.d.ff == L2H_FF_DENSE) add(&L.up, L.d.ff_dim, 1);
+        if (L.d.ff == L2H_FF_EXPERTS) {
+            add(&L.up, L.d.ff_dim, L.d.n_experts);
+            add(&L.down, l->W(), L.d.n_experts);
+        }
+    }
+    size_t free_b = 0, total_b = 0;
+    HIPCHK(m->ctx, hipMemGetInfo(&free_b, &total_b));
+    if (free_b < (size_t)elems * 2 + ((size_t)2 << 30)) return L2H_OK;
+    for (const Job &j : jobs) {
+        uint16_t *p = nullptr;
+        const int rc = dalloc(m, &p, j.n * k_tile_image_elems(j.rows, j.w->ld), false);
+        if (rc) return rc;
+        HIPCHK(m->ctx, k_tile_image(m->ctx->stream, j.w->w, j.w->ld, j.rows, j.n, p));
+        j.w->image = p;
+        j.w->image_stride = k_tile_image_elems(j.rows, j.w->ld);
+    }
+    HIPCHK(m->ctx, hipStreamSynchronize(m->ctx->stream));
+    return L2H_OK;
+}
+
 int layered_prefill_buffers(l2h_model *m, int cap, int n_want) {
     Layered *l = m->lay;
     const l2h_layered_config &c = l->c;
     int rc;
+    cap = (cap + 255) / 256 * 256;  // (a library product computes whole groups of 128 positions)
+    if (cap > L_BIG_MIN_M && (rc = prompt_images(m))) return rc;
 #define DA(p, n)                            \
     if ((rc = dalloc(m, &(p), (n), false))) \
         return rc;
@@ -632,7 +687,7 @@ int layered_prefill_buffers(l2h_model *m, int cap, int n_want) {
     }
     if (n_want > l->want_cap) {
         DA(l->want, n_want);
-        DA(l->wl, (int64_t)n_want * c.vocab_size);
+        DA(l->wl, (int64_t)((n_want + 255) / 256 * 256) * c.vocab_size);
         l->want_cap = n_want;
     }
     if (l->keep && l->kept_cap < cap) {
@@ -641,6 +696,7 @@ int layered_prefill_buffers(l2h_model *m, int cap, int n_want) {
     }
     if (l->cap >= cap) return L2H_OK;
     int64_t n_in = 1, ch = 1, g = 1, h = 1, hd = 1, hv = 1, lhv = 64, lra = 64, lrg = 64, hid = 64, ne = 1, slots = 1, up_slots = 1, tiles = 1;
+    int64_t kvt = 0;
     bool moe = false;
     for (LayerDev &L : l->layer) {
         const l2h_layer &d = L.d;
@@ -649,6 +705,11 @@ int layered_prefill_buffers(l2h_model *m, int cap, int n_want) {
         lhv = std::max<int64_t>(lhv, L.o.ld);
         if (d.mixer == L2H_MIX_ATTENTION) {
             ch = std::max<int64_t>(ch, d.n_heads * d.dim);
+            const int hs = attention_tile_size(d);
+            if (hs && !c.precision) {
+                ch = std::max<int64_t>(ch, d.n_heads * hs);
+                kvt = std::max<int64_t>(kvt, (int64_t)d.n_kv_heads * attention_tiles(l, L, cap) * k_pf_kv_tile_bytes(hs));
+            }
         } else {
             ch = std::max<int64_t>(ch, delta_shape(l, L).channels());
             g = std::max<int64_t>(g, d.n_kv_heads);
@@ -666,9 +727,10 @@ int layered_prefill_buffers(l2h_model *m, int cap, int n_want) {
             tiles = std::max<int64_t>(tiles, ((int64_t)cap * d.top + L_GEMM_TILE - 1) / L_GEMM_TILE + d.n_experts);
         }
     }
+    if (kvt) DA(l->kvt, kvt);
     DA(l->tok, cap);
     DA(l->X, (int64_t)cap * c.width);
-    DA(l->raw, cap * n_in);
+    DA(l->raw, cap * std::max<int64_t>(n_in, c.side_dim));
     DA(l->qkv, cap * ch);
     DA(l->kq, cap * g);
     DA(l->beta, cap * h);
@@ -700,6 +762,10 @@ int layered_prefill_buffers(l2h_model *m, int cap, int n_want) {
     l->cap = cap;
     return L2H_OK;
 }
+bool layered_wants_library(l2h_model *m, int n) {
+    const Layered *l = m->lay;
+    return l->c.precision == 0 && n >= L_BIG_MIN_M && (double)n * l->ldw() * l->layer[0].in.rows >= (double)(1 << 28);
+}
 int32_t *layered_token_buffer(l2h_model *m) { return m->lay->tok; }
 int layered_capacity(l2h_model *m) { return m->lay->cap; }
 
@@ -714,16 +780,35 @@ static GemmArgs gemm_of(const LMat &w, const void *x, int M) {
     return a;
 }
 
-// a plain product (GE_STORE or GE_RESID)
+// a plain product (GE_STORE or GE_RESID); large ones go through the library, rounded up to whole groups of 128 positions so
+// that few different shapes occur: the rows beyond M are computed from whatever the buffers hold, and never read
+static bool library_takes(const l2h_model *m, const GemmArgs &a) {
+    return m->lay->c.precision == 0 && m->pf_lt && m->pf_library_mode && a.M >= L_BIG_MIN_M &&
+           (double)a.M * (double)a.n_rows * (double)a.ld >= (double)(1 << 28);
+}
 static hipError_t product(l2h_model *m, GemmArgs a, int epi, float *out, int64_t ldo, float mult) {
+    if (library_takes(m, a)) {
+        const int M = (a.M + 127) / 128 * 128;
+        const hipError_t e = pf_lt_gemm(m->pf_lt, m->ctx->stream, a.w, (const uint16_t *)a.x, out, M, a.n_rows, a.ld, ldo, epi == GE_RESID,
+                                        &m->pf_lt_err, mult);
+        if (e != hipErrorNotSupported) return e;
+        pf_lt_close(m->pf_lt);  // no algorithm for a shape: this library's own kernels from here on
+        m->pf_lt = nullptr;
+        (void)hipGetLastError();
+    }
     a.outf = out;
     a.ldo = ldo;
     a.mult = mult;
     return k_gemm(m->ctx->stream, a, m->lay->c.precision, epi);
 }
-static hipError_t to_acts(l2h_model *m, GemmArgs a, int epi, void *out, int64_t lda) {
+static bool image_takes(const LMat &w, int M) { return w.image && M >= L_BIG_MIN_M; }
+static hipError_t to_acts(l2h_model *m, GemmArgs a, int epi, void *out, int64_t lda, const LMat *w = nullptr) {
     a.outa = out;
     a.lda = lda;
+    if (w && image_takes(*w, a.M)) {
+        a.w = w->image;
+        return k_tiles(m->ctx->stream, a, epi);
+    }
     return k_gemm(m->ctx->stream, a, m->lay->c.precision, epi);
 }
 
@@ -754,7 +839,23 @@ static hipError_t prompt_attention(l2h_model *m, LayerDev &L, int M, int pos0) {
     hipStream_t s = m->ctx->stream;
     const WindowShape w = window_shape(l, L);
     const int64_t ldr = w.n_in();
+    const int hs = attention_tile_size(L.d);
     hipError_t e;
+    if (hs && l->c.precision == 0) {
+        uint16_t *qb = (uint16_t *)l->qkv;
+        PfWindow win;
+        win.window = w.window;
+        win.tile0 = std::max(0, pos0 - w.window + 1) / 32;
+        win.vdim = w.V;
+        win.scale = w.scale;
+        win.gate = w.gated ? l->raw + w.off_g() : nullptr;
+        win.ldg = ldr;
+        win.ldo = L.o.ld;
+        const int n_tiles = (pos0 + M + 31) / 32 - win.tile0, cap = attention_tiles(l, L, l->cap);
+        CK(k_window_prepare(s, w, L.freq, l->raw, ldr, L.kc, L.vc, M, pos0, nullptr, qb, hs));
+        CK(k_pf_kv_tiles(s, L.kc, L.vc, l->kvt, n_tiles, cap, hs, w.G, w.seq_len, win.tile0, w.Dp(), w.V));
+        return k_pf_attention(s, qb, (uint16_t *)l->ao, l->kvt, cap, M, pos0, hs, w.H, w.G, w.H * hs, &win);
+    }
     CK(k_window_prepare(s, w, L.freq, l->raw, ldr, L.kc, L.vc, M, pos0, l->qkv, nullptr, 0));
     CK(k_window_rows(s, w, l->qkv, l->raw, ldr, L.kc, L.vc, M, pos0, l->ao, L.o.ld, l->c.precision));
     return hipSuccess;
@@ -783,12 +884,24 @@ static hipError_t prompt_experts(l2h_model *m, LayerDev &L, int M) {
     up.act = d.ff_act;
     up.outa = l->hb;
     up.lda = L.down.ld;
-    CK(k_gemm(s, up, prec, GE_UP));
+    if (image_takes(L.up, M)) {
+        up.w = L.up.image;
+        up.expert_stride = L.up.image_stride;
+        CK(k_tiles(s, up, GE_UP));
+    } else {
+        CK(k_gemm(s, up, prec, GE_UP));
+    }
     down.n_rows = l->W();
     down.expert_stride = (int64_t)l->W() * L.down.ld;
     down.outf = l->yb;
     down.ldo = l->W();
-    CK(k_gemm(s, down, prec, GE_STORE));
+    if (image_takes(L.down, M)) {
+        down.w = L.down.image;
+        down.expert_stride = L.down.image_stride;
+        CK(k_tiles(s, down, GE_STORE));
+    } else {
+        CK(k_gemm(s, down, prec, GE_STORE));
+    }
     return k_gather_add(s, l->X, l->yb, l->slot_of, M, d.top, l->W(), l->c.residual_mult);
 }
 
@@ -818,7 +931,7 @@ hipError_t layered_prefill_chunk(l2h_model *m, int M, int pos0) {
             if (d.ff == L2H_FF_DENSE) {
                 GemmArgs up = gemm_of(L.up, l->xn, M);
                 up.act = d.ff_act;
-                CK(to_acts(m, up, GE_ACT, l->hb, L.down.ld));
+                CK(to_acts(m, up, GE_ACT, l->hb, L.down.ld, &L.up));
                 CK(product(m, gemm_of(L.down, l->hb, M), GE_RESID, l->X, W, mult));
             } else {
                 CK(prompt_experts(m, L, M));
@@ -831,7 +944,12 @@ hipError_t layered_prefill_chunk(l2h_model *m, int M, int pos0) {
             g.emb = l->side_emb + (int64_t)i * c.side_dim;
             g.emb_ld = (int64_t)c.n_layers * c.side_dim;
             g.tokens = l->tok;
-            CK(to_acts(m, g, GE_EMBED, l->sb, L.side_proj.ld));
+            if (library_takes(m, g)) {
+                CK(product(m, g, GE_STORE, l->raw, c.side_dim, 1.0f));
+                CK(k_embed_rows(s, l->raw, M, c.side_dim, g.act, g.emb, g.emb_ld, g.tokens, l->sb, L.side_proj.ld, prec));
+            } else {
+                CK(to_acts(m, g, GE_EMBED, l->sb, L.side_proj.ld));
+            }
             CK(product(m, gemm_of(L.side_proj, l->sb, M), GE_STORE, l->Y, W, 1.0f));
             py = l->Y;
             pyw = L.side_norm;

@@ -9,6 +9,9 @@ struct LMat {
     uint16_t *w = nullptr;
     int64_t rows = 0;
     int K = 0, ld = 0;
+    // tile image for the prompt pass (k_tiles.hip), or nullptr; elements of one matrix where several are stacked
+    uint16_t *image = nullptr;
+    int64_t image_stride = 0;
 };
 static inline int pad64(int64_t n) { return (int)((n + 63) / 64 * 64); }
 
@@ -92,6 +95,14 @@ struct GemmArgs {
 };
 #define L_GEMM_TILE 128
 hipError_t k_gemm(hipStream_t s, const GemmArgs &a, int prec, int epi);
+
+// the same from a tile image (k_tiles.hip): GE_ACT, and GE_UP / GE_STORE in the grouped form; bf16 activations
+hipError_t k_tiles(hipStream_t s, const GemmArgs &a, int epi);
+int64_t k_tile_image_elems(int64_t rows, int ld);
+hipError_t k_tile_image(hipStream_t s, const uint16_t *w, int ld, int64_t rows, int64_t n_mats, uint16_t *dst);
+// outa[m][n] = act(v[m][n]) * embedding element, for products that the library has stored as fp32
+hipError_t k_embed_rows(hipStream_t s, const float *v, int M, int N, int act, const uint16_t *emb, int64_t emb_ld,
+                        const int32_t *tokens, void *outa, int64_t lda, int prec);
 
 // rows of x (fp32, stride K): [x += mult * rmsnorm(y) * yw;] outa = rmsnorm(x) * w, or x itself with w == nullptr; with
 // `gather`, row r of the result is row gather[r] of x

@@ -1,0 +1,45 @@
+// Epilogues of the many-token products of layered models.
+#pragma once
+
+#include "layered_dev.h"
+
+// results (m, L .. L + 3) of a product
+template <int PREC, int EPI>
+__device__ __forceinline__ void gemm_store4(const GemmArgs &a, int64_t m, int64_t L, float v0, float v1, float v2, float v3) {
+    float v[4] = {v0, v1, v2, v3};
+    if (EPI == GE_STORE || EPI == GE_RESID || EPI == GE_DECAY || EPI == GE_SIGMOID) {
+        if (L >= a.n_rows) return;
+        float *o = a.outf + m * a.ldo + L;
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+            if (L + e >= a.n_rows) break;
+            if (EPI == GE_RESID)
+                o[e] = fmaf(a.mult, v[e], o[e]);
+            else if (EPI == GE_DECAY)
+                o[e] = -a.rate[(L + e) / a.hd] * l_softplus(v[e] + a.bias[L + e]);
+            else if (EPI == GE_SIGMOID)
+                o[e] = l_sigmoid(v[e]);
+            else
+                o[e] = v[e];
+        }
+    } else {
+        if (L >= a.lda) return;  // (lda a multiple of 64: whole groups of four)
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+            if (L + e >= a.n_rows) {
+                v[e] = 0.0f;
+                continue;
+            }
+            if (EPI == GE_UP)
+                v[e] = l_act(a.act, a.row_scale[m] * v[e]);
+            else if (EPI == GE_EMBED)
+                v[e] = l_act(a.act, v[e]) * l_bf16(a.emb[(int64_t)a.tokens[m] * a.emb_ld + L + e]);
+            else
+                v[e] = l_act(a.act, v[e]);
+        }
+        if (PREC)
+            *(float4 *)((float *)a.outa + m * a.lda + L) = make_float4(v[0], v[1], v[2], v[3]);
+        else
+            *(uint2 *)((uint16_t *)a.outa + m * a.lda + L) = make_uint2(l_pack_bf16(v[0], v[1]), l_pack_bf16(v[2], v[3]));
+    }
+}

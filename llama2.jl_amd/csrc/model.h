@@ -121,6 +121,7 @@ hipError_t layered_enqueue_token(l2h_model *m);  // embedding to logits
 hipError_t layered_output(l2h_model *m);         // m->x -> m->logits
 int layered_prefill_buffers(l2h_model *m, int cap, int n_want);
 int layered_capacity(l2h_model *m);
+bool layered_wants_library(l2h_model *m, int n);  // would a prompt of n positions run products through hipBLASLt?
 int32_t *layered_token_buffer(l2h_model *m);
 hipError_t layered_prefill_chunk(l2h_model *m, int M, int pos0);
 int layered_prefill_logits(l2h_model *m, const int32_t *rows, int n, float *logits);

@@ -201,7 +201,7 @@ static bool pf_lt_plan(PfLt *lt, hipStream_t s, LtPlan &p, const uint16_t *W, co
 // D == nullptr: only finds (and keeps) the algorithm for the shape, so that a library that has none is noticed before
 // anything has been computed with it
 hipError_t pf_lt_gemm(PfLt *lt, hipStream_t s, const uint16_t *W, const uint16_t *X, float *D, int M, int64_t N, int64_t K,
-                      int64_t ldd, bool accumulate, std::string *err) {
+                      int64_t ldd, bool accumulate, std::string *err, float alpha) {
     if (!lt || M < 1 || N < 1 || K < 1 || ldd < N) return hipErrorInvalidValue;
     const auto key = std::make_tuple(M, N, K, ldd, accumulate);
     auto it = lt->plans.find(key);
@@ -218,7 +218,7 @@ hipError_t pf_lt_gemm(PfLt *lt, hipStream_t s, const uint16_t *W, const uint16_t
     }
     if (!D) return hipSuccess;
     const LtPlan &p = it->second;
-    const float alpha = 1.0f, beta = accumulate ? 1.0f : 0.0f;
+    const float beta = accumulate ? 1.0f : 0.0f;
     const hipblasStatus_t st = lt->api.Matmul(lt->handle, p.desc, &alpha, W, p.lw, X, p.lx, &beta, D, p.ld, D, p.ld, &p.algo,
                                               lt->workspace, lt->workspace_bytes, s);
     if (st != HIPBLAS_STATUS_SUCCESS) {

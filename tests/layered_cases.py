@@ -66,6 +66,9 @@ CASES = {
     "mixed_wide": config([attention(heads=8, kv_heads=2, dim=64, vdim=64, size=37, rot=64, mlp=dense(700)),
                           delta(heads=8, kv_heads=4, dim=64, vdim=64, conv=4, ranks=(32, 32), mlp=moe(16, 4, 96))], width=520, vocab=300,
                          side=64),
+    # wide and long enough for the library's products and the tile images
+    "large": config([delta(heads=10, kv_heads=5, dim=64, vdim=64, conv=4, ranks=(40, 72), mlp=moe(6, 2, 200)),
+                     attention(heads=10, kv_heads=5, dim=96, vdim=80, size=70, rot=96, mlp=dense(600))], width=576, vocab=520, side=48),
 }
 
 

@@ -23,7 +23,7 @@ TOL = {"float32": 2e-5, "bfloat16": 3e-2}
 
 
 def _length(case):
-    return 300 if case == "attention_long_window" else 90 if "window" in case or case.startswith("mixed") else 45
+    return 300 if case in ("attention_long_window", "large") else 90 if "window" in case or case.startswith("mixed") else 45
 
 
 def _decode(dev, toks, pos0=0):
@@ -63,6 +63,23 @@ def test_prompt_and_decode_match(pkg, expected, case, precision):
     print("\n[%s, %s] prompt %.3g (layers %s), decode %.3g" % (case, precision, e_prompt, ["%.2g" % e for e in e_layer], e_decode))
     assert e_prompt <= TOL[precision] and max(e_layer) <= TOL[precision]
     assert e_decode <= TOL["float32"]  # decode steps are fp32 in both
+    dev.close()
+
+
+@pytest.mark.parametrize("library,copy", [(True, True), (False, True), (True, False), (False, False)])
+def test_forms_of_the_large_products(pkg, expected, library, copy):
+    """through hipBLASLt or not, experts and up projections from tile images or not: whole prompts and portions that are
+    no multiple of anything"""
+    c, t, tok, want, _ = expected("large")
+    dev = lc.language_model(pkg, c, t, precision="bfloat16").device()
+    dev.set_prefill_library(library)
+    dev.set_prefill_copy(copy)
+    n = len(tok)
+    assert lc.error(dev.prefill_logits(tok, np.arange(n)), want) <= TOL["bfloat16"]
+    first = dev.prefill_logits(tok[:137], np.arange(137))
+    rest = dev.prefill_logits(tok[137:], np.arange(n - 137), 137)
+    assert lc.error(np.concatenate([first, rest]), want) <= TOL["bfloat16"]
+    assert lc.error(dev.prefill_logits(tok[:190], [188, 189]), want[188:190]) <= TOL["bfloat16"]
     dev.close()
 
 

@@ -1,7 +1,7 @@
 """The prompt-pass kernels read LDS with loads issued from inline asm, some of them one step ahead of the
 wait that retires them.  The compiler believes an asm statement's outputs valid as soon as the statement
 ends, so until that wait nothing may touch the registers such a read targets.  This test compiles
-k_prefill.hip to assembly and walks the generated code: LDS reads complete in order, `s_waitcnt
+the sources to assembly and walks the generated code: LDS reads complete in order, `s_waitcnt
 lgkmcnt(N)` leaves at most the N newest under way, and no instruction in between may name a register
 that a read still under way writes."""
 import os
@@ -47,10 +47,11 @@ def _scan(path):
 
 
 @pytest.mark.skipif(shutil.which("hipcc") is None and not os.path.exists("/opt/rocm/bin/hipcc"), reason="no hipcc")
-def test_no_register_of_a_pending_lds_read_is_touched(tmp_path):
+@pytest.mark.parametrize("source", ["k_prefill", "k_tiles"])
+def test_no_register_of_a_pending_lds_read_is_touched(tmp_path, source):
     hipcc = shutil.which("hipcc") or "/opt/rocm/bin/hipcc"
-    out = tmp_path / "k_prefill.s"
-    cmd = [hipcc, "-S", "--cuda-device-only", os.path.join(CSRC, "k_prefill.hip"), "-o", str(out), "--offload-arch=gfx950",
+    out = tmp_path / (source + ".s")
+    cmd = [hipcc, "-S", "--cuda-device-only", os.path.join(CSRC, source + ".hip"), "-o", str(out), "--offload-arch=gfx950",
            "-O3", "-std=c++17", "-ffp-contract=off", "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops",
            "-I", os.path.join(ROOT, "include"), "-I", CSRC]
     subprocess.run(cmd, check=True, capture_output=True, timeout=600)

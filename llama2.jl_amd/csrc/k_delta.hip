@@ -429,6 +429,244 @@ hipError_t k_delta_scan(hipStream_t s, const DeltaShape &d, const float *qkv, co
     return hipGetLastError();
 }
 
+// ---------------------------------------------------------------------------------------------------------------
+// the recurrence in chunks of 16 tokens, on the fp32 matrix cores.  With G_i the decays' logarithms summed over the tokens
+// 0 .. i of a chunk and S0 the state before it, unrolling the recurrence gives
+//   A_ij = sum_d k_i k_j exp(G_i - G_j)  (j < i),   B_ij = sum_d q_i k_j exp(G_i - G_j)  (j <= i)
+//   U = T (V - (k exp(G)) S0),  T = (I + diag(beta) A)^-1 diag(beta)
+//   O = (q exp(G)) S0 + B U,    S = diag(exp(G_15)) S0 + (k exp(G_15 - G))^T U
+// All exponents are <= 0.  A, B, T and the scaled rows depend on no state: delta_chunk_kernel makes them for all chunks at once;
+// delta_walk_kernel then walks the chunks, 16 value columns a workgroup, the key channels split over its four wavefronts.
+//
+// Operands are stored in the order the lanes hold them.  v_mfma_f32_16x16x4_f32: lane l has A[l % 16][l / 16], B[l / 16][l % 16]
+// and, of the result, rows 4 (l / 16) + r in register r, column l % 16.  With the four steps over a tile of 16 contracted
+// indexes taken as k = 4 (l / 16) + r, a result is the next product's B operand as it stands, and an A operand's four steps are
+// one 16-byte word of lane l: (row l % 16; columns 4 (l / 16) .. + 3).
+// ---------------------------------------------------------------------------------------------------------------
+#define CH_T 16
+typedef float d_f32x4 __attribute__((ext_vector_type(4)));
+
+// the record of one (chunk, head): NT tiles of 16 key channels (a multiple of 4); kt, qt, kh: [NT][64][4]; T, B: [64][4];
+// exp(G_15): [16 NT]
+__host__ __device__ static inline int delta_chunk_tiles(int D) { return (D + 63) / 64 * 4; }
+__host__ __device__ static inline int64_t delta_chunk_floats(int NT) { return (int64_t)NT * 784 + 512; }
+
+__global__ __launch_bounds__(256) void delta_chunk_kernel(DeltaShape d, const float *qkv, const float *beta, const float *lg, int M,
+                                                          float *rec) {
+    extern __shared__ __align__(16) float s_mem[];
+    const int NT = delta_chunk_tiles(d.D), DP = 16 * NT, t = threadIdx.x, lane = t & 63, wave = t >> 6;
+    float *s_q = s_mem, *s_k = s_q + CH_T * DP, *s_g = s_k + CH_T * DP;  // [16][DP]; s_g: decays, then their logarithms' sums
+    __shared__ float s_A[CH_T][CH_T + 1], s_B[CH_T][CH_T + 1], s_T[CH_T][CH_T + 1], s_b[CH_T];
+    const int ch = blockIdx.x, h = blockIdx.y, kvh = h / (d.H / d.G), m0 = ch * CH_T, n = min(CH_T, M - m0);
+    const int D = d.D, C = d.channels(), GD = d.G * D;
+    for (int i = t; i < CH_T * DP; i += 256) {
+        const int tt = i / DP, e = i - tt * DP;
+        float q = 0.0f, k = 0.0f, g = 1.0f;
+        if (tt < n && e < D) {
+            const float *row = qkv + (int64_t)(m0 + tt) * C + kvh * D + e;
+            q = row[0];
+            k = row[GD];
+            g = expf(lg[((int64_t)(m0 + tt) * d.H + h) * D + e]);
+        }
+        s_q[i] = q;
+        s_k[i] = k;
+        s_g[i] = g;
+    }
+    if (t < CH_T) s_b[t] = t < n ? beta[(int64_t)(m0 + t) * d.H + h] : 0.0f;
+    __syncthreads();
+    // A and B: a group of 16 lanes has row j of the pairs (j, i > j), each lane every 16th channel; r = k_j times the decays of
+    // the tokens after j
+    {
+        const int j = 4 * wave + (lane >> 4), sl = lane & 15;
+        float a[CH_T], b[CH_T];
+#pragma unroll
+        for (int i = 0; i < CH_T; i++) a[i] = b[i] = 0.0f;
+        for (int e = sl; e < D; e += 16) {
+            float r = s_k[j * DP + e];
+#pragma unroll
+            for (int i = 0; i < CH_T; i++) {
+                if (i > j) r *= s_g[i * DP + e];
+                const float u = i >= j ? r : 0.0f;
+                a[i] = fmaf(s_k[i * DP + e], u, a[i]);
+                b[i] = fmaf(s_q[i * DP + e], u, b[i]);
+            }
+        }
+#pragma unroll
+        for (int i = 0; i < CH_T; i++) {
+            a[i] = row16_sum(a[i]);
+            b[i] = row16_sum(b[i]);
+            if (sl == i) {
+                s_A[i][j] = i > j ? a[i] : 0.0f;
+                s_B[i][j] = b[i];
+            }
+        }
+    }
+    __syncthreads();
+    // T by forward substitution, a lane per column
+    if (t < CH_T) {
+        float x[CH_T];
+#pragma unroll
+        for (int i = 0; i < CH_T; i++) {
+            float v = i == t ? 1.0f : 0.0f;
+#pragma unroll
+            for (int j = 0; j < i; j++) v = fmaf(-s_A[i][j], x[j], v);
+            x[i] = s_b[i] * v;
+            s_T[i][t] = x[i];
+        }
+    }
+    // sums of the logarithms, in place of the decays
+    for (int e = t; e < DP; e += 256) {
+        float g = 0.0f;
+        for (int i = 0; i < CH_T; i++) {
+            if (i < n && e < D) g += lg[((int64_t)(m0 + i) * d.H + h) * D + e];
+            s_g[i * DP + e] = g;
+        }
+    }
+    __syncthreads();
+    float *out = rec + ((int64_t)ch * d.H + h) * delta_chunk_floats(NT);
+    for (int idx = t; idx < NT * 64; idx += 256) {
+        const int tile = idx >> 6, l = idx & 63, row = l & 15, q4 = 4 * (l >> 4);
+        float4 kt, qt, kh;
+        {
+            const int o = row * DP + 16 * tile + q4;
+            const float4 k = *(const float4 *)(s_k + o), q = *(const float4 *)(s_q + o), G = *(const float4 *)(s_g + o);
+            const float4 x = make_float4(expf(G.x), expf(G.y), expf(G.z), expf(G.w));
+            kt = make_float4(k.x * x.x, k.y * x.y, k.z * x.z, k.w * x.w);
+            qt = make_float4(q.x * x.x, q.y * x.y, q.z * x.z, q.w * x.w);
+        }
+        {  // row: the channel, columns: tokens
+            const int e = 16 * tile + row;
+            const float Gc = s_g[15 * DP + e];
+            kh = make_float4(s_k[q4 * DP + e] * expf(Gc - s_g[q4 * DP + e]), s_k[(q4 + 1) * DP + e] * expf(Gc - s_g[(q4 + 1) * DP + e]),
+                             s_k[(q4 + 2) * DP + e] * expf(Gc - s_g[(q4 + 2) * DP + e]),
+                             s_k[(q4 + 3) * DP + e] * expf(Gc - s_g[(q4 + 3) * DP + e]));
+        }
+        *(float4 *)(out + 4 * idx) = kt;
+        *(float4 *)(out + 256 * NT + 4 * idx) = qt;
+        *(float4 *)(out + 512 * NT + 4 * idx) = kh;
+    }
+    if (t < 128) {
+        const float(*m)[CH_T + 1] = wave ? s_B : s_T;
+        const int row = lane & 15, q4 = 4 * (lane >> 4);
+        *(float4 *)(out + 768 * NT + 256 * wave + 4 * lane) = make_float4(m[row][q4], m[row][q4 + 1], m[row][q4 + 2], m[row][q4 + 3]);
+    }
+    for (int e = t; e < DP; e += 256) out[768 * NT + 512 + e] = e < D ? expf(s_g[15 * DP + e]) : 0.0f;
+}
+
+// one chunk's operands of a wavefront with NW tiles of key channels
+template <int NW>
+struct DeltaOps {
+    d_f32x4 kt[NW], qt[NW], kh[NW], gc[NW], T;
+    float B, v[4];
+};
+
+template <int NW>
+__global__ __launch_bounds__(256) void delta_walk_kernel(DeltaShape d, const float *rec, const float *qkv, float *state, int M, int pos0,
+                                                         float *o) {
+    __shared__ __align__(16) d_f32x4 s_w[2][4][64], s_o[2][4][64];
+    constexpr int NT = 4 * NW;
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, col = lane & 15, q4 = 4 * (lane >> 4);
+    const int h = blockIdx.y, c = blockIdx.x * 16 + col, D = d.D, V = d.V, C = d.channels();
+    const bool live = c < V;
+    float *S = state + (int64_t)h * D * V;
+    d_f32x4 s[NW];
+#pragma unroll
+    for (int i = 0; i < NW; i++)
+#pragma unroll
+        for (int r = 0; r < 4; r++) {
+            const int e = 16 * (wave * NW + i) + q4 + r;
+            s[i][r] = (live && e < D && pos0 > 0) ? S[(int64_t)e * V + c] : 0.0f;
+        }
+    const int n_ch = (M + CH_T - 1) / CH_T;
+    const float *vcol = qkv + 2 * d.G * D + h * V + (live ? c : 0);
+    auto fetch = [&](DeltaOps<NW> &x, int ch) {
+        const float *p = rec + ((int64_t)ch * d.H + h) * delta_chunk_floats(NT);
+#pragma unroll
+        for (int i = 0; i < NW; i++) {
+            const int tile = wave * NW + i;
+            x.kt[i] = *(const d_f32x4 *)(p + 256 * tile + 4 * lane);
+            x.qt[i] = *(const d_f32x4 *)(p + 256 * (NT + tile) + 4 * lane);
+            x.kh[i] = *(const d_f32x4 *)(p + 256 * (2 * NT + tile) + 4 * lane);
+            x.gc[i] = *(const d_f32x4 *)(p + 768 * NT + 512 + 16 * tile + q4);
+        }
+        x.T = *(const d_f32x4 *)(p + 768 * NT + 4 * lane);
+        x.B = p[768 * NT + 256 + 4 * lane + wave];
+#pragma unroll
+        for (int r = 0; r < 4; r++) {
+            const int m = ch * CH_T + q4 + r;
+            x.v[r] = (live && m < M) ? vcol[(int64_t)m * C] : 0.0f;
+        }
+    };
+    // the output row 4 (lane / 16) + wave of a chunk, from the four wavefronts' parts
+    auto put = [&](int ch) {
+        const int m = ch * CH_T + q4 + wave, b = ch & 1;
+        const float v = s_o[b][0][lane][wave] + s_o[b][1][lane][wave] + s_o[b][2][lane][wave] + s_o[b][3][lane][wave];
+        if (live && m < M) o[((int64_t)m * d.H + h) * V + c] = v;
+    };
+    DeltaOps<NW> cur, nxt;
+    fetch(cur, 0);
+    for (int ch = 0; ch < n_ch; ch++) {
+        const int b = ch & 1;
+        fetch(nxt, min(ch + 1, n_ch - 1));
+        d_f32x4 w = {0.f, 0.f, 0.f, 0.f}, y = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int i = 0; i < NW; i++)
+#pragma unroll
+            for (int r = 0; r < 4; r++) w = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.kt[i][r], s[i][r], w, 0, 0, 0);
+        s_w[b][wave][lane] = w;
+#pragma unroll
+        for (int i = 0; i < NW; i++)
+#pragma unroll
+            for (int r = 0; r < 4; r++) y = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.qt[i][r], s[i][r], y, 0, 0, 0);
+        __syncthreads();  // (also: the parts of the previous chunk's output are all there)
+        if (ch) put(ch - 1);
+        w = s_w[b][0][lane] + s_w[b][1][lane] + s_w[b][2][lane] + s_w[b][3][lane];
+        d_f32x4 u = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int r = 0; r < 4; r++) u = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.T[r], cur.v[r] - w[r], u, 0, 0, 0);
+        // B U: this wavefront's quarter of the contracted tokens
+        const float uw = wave == 0 ? u[0] : wave == 1 ? u[1] : wave == 2 ? u[2] : u[3];
+        y = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.B, uw, y, 0, 0, 0);
+#pragma unroll
+        for (int i = 0; i < NW; i++) {
+            s[i] *= cur.gc[i];
+#pragma unroll
+            for (int r = 0; r < 4; r++) s[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.kh[i][r], u[r], s[i], 0, 0, 0);
+        }
+        s_o[b][wave][lane] = y;
+        cur = nxt;
+    }
+    __syncthreads();
+    put(n_ch - 1);
+#pragma unroll
+    for (int i = 0; i < NW; i++)
+#pragma unroll
+        for (int r = 0; r < 4; r++) {
+            const int e = 16 * (wave * NW + i) + q4 + r;
+            if (live && e < D) S[(int64_t)e * V + c] = s[i][r];
+        }
+}
+
+int64_t delta_walk_floats(const DeltaShape &d, int M) {
+    return (int64_t)((M + CH_T - 1) / CH_T) * d.H * delta_chunk_floats(delta_chunk_tiles(d.D));
+}
+hipError_t k_delta_walk(hipStream_t s, const DeltaShape &d, const float *qkv, const float *beta, const float *lg, float *state, int M,
+                        int pos0, float *rec, float *o) {
+    if (d.D > 256 || M < 1) return hipErrorInvalidValue;
+    const int NT = delta_chunk_tiles(d.D);
+    const dim3 g1((unsigned)((M + CH_T - 1) / CH_T), (unsigned)d.H), g2((unsigned)((d.V + 15) / 16), (unsigned)d.H);
+    hipLaunchKernelGGL(delta_chunk_kernel, g1, dim3(256), (size_t)3 * CH_T * 16 * NT * sizeof(float), s, d, qkv, beta, lg, M, rec);
+#define GO(N) hipLaunchKernelGGL((delta_walk_kernel<N>), g2, dim3(256), 0, s, d, rec, qkv, state, M, pos0, o)
+    switch (NT / 4) {
+    case 1: GO(1); break;
+    case 2: GO(2); break;
+    case 3: GO(3); break;
+    default: GO(4); break;
+    }
+#undef GO
+    return hipGetLastError();
+}
+
 // one wavefront per (token, head)
 template <int PREC>
 __global__ __launch_bounds__(256) void head_norm_rows_kernel(const float *o, const float *gate, const float *normw, int M, int H, int V,

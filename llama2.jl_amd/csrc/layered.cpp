@@ -39,7 +39,7 @@ struct Layered {
     int32_t *tok = nullptr, *choice = nullptr, *slot_row = nullptr, *slot_of = nullptr, *n_tiles = nullptr, *want = nullptr;
     GemmTile *tiles = nullptr;
     float *X = nullptr, *raw = nullptr, *qkv = nullptr, *kq = nullptr, *beta = nullptr, *lg = nullptr, *gt = nullptr, *ob = nullptr,
-          *zb = nullptr, *score = nullptr, *slot_scale = nullptr, *yb = nullptr, *Y = nullptr, *wl = nullptr;
+          *zb = nullptr, *score = nullptr, *slot_scale = nullptr, *yb = nullptr, *Y = nullptr, *wl = nullptr, *rec = nullptr;
     void *xn = nullptr, *fa = nullptr, *fg = nullptr, *ao = nullptr, *hb = nullptr, *sb = nullptr;
     int want_cap = 0;
     // residual stream after every layer of the last prompt pass (l2h_layered_keep)
@@ -696,7 +696,7 @@ int layered_prefill_buffers(l2h_model *m, int cap, int n_want) {
     }
     if (l->cap >= cap) return L2H_OK;
     int64_t n_in = 1, ch = 1, g = 1, h = 1, hd = 1, hv = 1, lhv = 64, lra = 64, lrg = 64, hid = 64, ne = 1, slots = 1, up_slots = 1, tiles = 1;
-    int64_t kvt = 0;
+    int64_t kvt = 0, rec = 0;
     bool moe = false;
     for (LayerDev &L : l->layer) {
         const l2h_layer &d = L.d;
@@ -716,6 +716,7 @@ int layered_prefill_buffers(l2h_model *m, int cap, int n_want) {
             h = std::max<int64_t>(h, d.n_heads);
             hd = std::max<int64_t>(hd, d.n_heads * d.dim);
             lra = std::max<int64_t>(lra, L.a2.ld);
+            rec = std::max(rec, delta_walk_floats(delta_shape(l, L), cap));
             lrg = std::max<int64_t>(lrg, L.g2.ld);
         }
         if (d.ff == L2H_FF_DENSE) hid = std::max<int64_t>(hid, L.down.ld);
@@ -728,6 +729,7 @@ int layered_prefill_buffers(l2h_model *m, int cap, int n_want) {
         }
     }
     if (kvt) DA(l->kvt, kvt);
+    if (rec) DA(l->rec, rec);
     DA(l->tok, cap);
     DA(l->X, (int64_t)cap * c.width);
     DA(l->raw, cap * std::max<int64_t>(n_in, c.side_dim));
@@ -829,7 +831,10 @@ static hipError_t prompt_delta(l2h_model *m, LayerDev &L, int M, int pos0) {
     a.hd = d.D;
     CK(k_gemm(s, a, prec, GE_DECAY));
     CK(product(m, gemm_of(L.g2, l->fg, M), GE_SIGMOID, l->gt, hv, 1.0f));
-    CK(k_delta_scan(s, d, l->qkv, l->kq, l->beta, l->lg, L.state, M, pos0, l->ob));
+    if (M >= L_DELTA_WALK_MIN)
+        CK(k_delta_walk(s, d, l->qkv, l->beta, l->lg, L.state, M, pos0, l->rec, l->ob));
+    else
+        CK(k_delta_scan(s, d, l->qkv, l->kq, l->beta, l->lg, L.state, M, pos0, l->ob));
     CK(k_head_norm_rows(s, l->ob, l->gt, L.mixnorm, M, d.H, d.V, d.eps, l->ao, L.o.ld, prec));
     return hipSuccess;
 }

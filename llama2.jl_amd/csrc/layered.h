@@ -148,6 +148,11 @@ hipError_t k_delta_prepare(hipStream_t s, const DeltaShape &d, const float *conv
 // the recurrence over M tokens, logarithms of the decays in lg[M][H D]; o[M][H V]; then the ring takes the last tokens
 hipError_t k_delta_scan(hipStream_t s, const DeltaShape &d, const float *qkv, const float *kq, const float *beta, const float *lg,
                         float *state, int M, int pos0, float *o);
+// the same in chunks of 16 tokens on the matrix cores; rec: delta_walk_floats(d, M) floats of scratch
+int64_t delta_walk_floats(const DeltaShape &d, int M);
+hipError_t k_delta_walk(hipStream_t s, const DeltaShape &d, const float *qkv, const float *beta, const float *lg, float *state, int M,
+                        int pos0, float *rec, float *o);
+#define L_DELTA_WALK_MIN 24  // tokens from which the chunked form is used
 hipError_t k_delta_ring(hipStream_t s, const DeltaShape &d, const float *raw, int64_t ldr, float *ring, int M, int pos0);
 // outa[m][h V + j] = o * rms over the head * normw[j] * gate
 hipError_t k_head_norm_rows(hipStream_t s, const float *o, const float *gate, const float *normw, int M, int H, int V, float eps,

@@ -210,13 +210,48 @@ hipError_t k_delta_step(hipStream_t s, const DeltaShape &d, const DeltaWeights &
 // ---------------------------------------------------------------------------------------------------------------
 #define PREP_T 8
 
+// CONV_AHEAD - 1 + PREP_T inputs of a channel (tokens m0 - CONV_AHEAD + 1 .. m0 + PREP_T - 1) are fetched together, then the
+// convolution and silu of its PREP_T tokens; taps beyond CONV_AHEAD are added one by one
 __device__ __forceinline__ float delta_raw_at(const float *raw, int64_t ldr, const float *ring, int C, int taps, int ch, int m, int pos0) {
     if (m >= 0) return raw[(int64_t)m * ldr + ch];
     const int p = pos0 + m;
     return p >= 0 ? ring[(int64_t)(p % taps) * C + ch] : 0.0f;
 }
+__device__ __forceinline__ void delta_conv_rows(const float *conv, const float *raw, int64_t ldr, const float *ring, int C, int taps, int ch,
+                                                int m0, int M, int pos0, float (&y)[PREP_T]) {
+    float x[CONV_AHEAD - 1 + PREP_T], w[CONV_AHEAD];
+    const float *col = raw + ch;
+    if (m0 >= CONV_AHEAD - 1) {
+#pragma unroll
+        for (int i = 0; i < CONV_AHEAD - 1 + PREP_T; i++) x[i] = col[(int64_t)min(m0 - CONV_AHEAD + 1 + i, M - 1) * ldr];
+    } else {
+#pragma unroll
+        for (int i = 0; i < CONV_AHEAD - 1 + PREP_T; i++) {
+            const int m = m0 - CONV_AHEAD + 1 + i;
+            // (an input further back than the taps reach has left the ring: its weight is 0)
+            x[i] = (m >= 0 || -m < taps) ? delta_raw_at(raw, ldr, ring, C, taps, ch, min(m, M - 1), pos0) : 0.0f;
+        }
+    }
+#pragma unroll
+    for (int j = 0; j < CONV_AHEAD; j++) w[j] = j < taps ? conv[(int64_t)(taps - 1 - j) * C + ch] : 0.0f;
+#pragma unroll
+    for (int i = 0; i < PREP_T; i++) {
+        float v = 0.0f;
+#pragma unroll
+        for (int j = 0; j < CONV_AHEAD; j++) v = fmaf(w[j], x[i + CONV_AHEAD - 1 - j], v);
+        y[i] = v;
+    }
+    for (int j = CONV_AHEAD; j < taps; j++) {
+        const float wj = conv[(int64_t)(taps - 1 - j) * C + ch];
+        for (int i = 0; i < PREP_T; i++)
+            if (m0 + i < M) y[i] = fmaf(wj, delta_raw_at(raw, ldr, ring, C, taps, ch, m0 + i - j, pos0), y[i]);
+    }
+#pragma unroll
+    for (int i = 0; i < PREP_T; i++) y[i] = l_silu(y[i]);
+}
 
-template <int PREC>
+// NE: key channels per lane (D <= 64 NE)
+template <int PREC, int NE>
 __global__ __launch_bounds__(256) void delta_prepare_kernel(DeltaShape d, const float *conv, const float *raw, int64_t ldr,
                                                             const float *ring, int M, int pos0, float *qkv, float *kq, float *beta,
                                                             void *fa, int64_t lfa, void *fg, int64_t lfg) {
@@ -237,47 +272,47 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(DeltaShape d, const 
     if (unit >= d.G) {  // a value head
         const int ch0 = 2 * GD + (unit - d.G) * d.V;
         for (int e = lane; e < d.V; e += 64) {
-            for (int m = m0; m < m1; m++) {
-                float v = 0.0f;
-                for (int j = 0; j < taps; j++)
-                    v = fmaf(conv[(int64_t)(taps - 1 - j) * C + ch0 + e], delta_raw_at(raw, ldr, ring, C, taps, ch0 + e, m - j, pos0), v);
-                qkv[(int64_t)m * C + ch0 + e] = l_silu(v);
-            }
+            float y[PREP_T];
+            delta_conv_rows(conv, raw, ldr, ring, C, taps, ch0 + e, m0, M, pos0, y);
+#pragma unroll
+            for (int i = 0; i < PREP_T; i++)
+                if (m0 + i < M) qkv[(int64_t)(m0 + i) * C + ch0 + e] = y[i];
         }
         return;
     }
-    // a key head's q and k: D <= 256 elements, four per lane
-    const float qs = 1.0f / sqrtf((float)d.D);
-    for (int m = m0; m < m1; m++) {
-        float q[4], k[4], qq = 0.0f, kk = 0.0f, qk = 0.0f;
+    // a key head's q and k
+    float q[NE][PREP_T], k[NE][PREP_T];
 #pragma unroll
-        for (int i = 0; i < 4; i++) {
-            const int e = lane + 64 * i;
-            q[i] = k[i] = 0.0f;
-            if (e >= d.D) continue;
-            const int cq = unit * d.D + e, ck = GD + cq;
-            for (int j = 0; j < taps; j++) {
-                q[i] = fmaf(conv[(int64_t)(taps - 1 - j) * C + cq], delta_raw_at(raw, ldr, ring, C, taps, cq, m - j, pos0), q[i]);
-                k[i] = fmaf(conv[(int64_t)(taps - 1 - j) * C + ck], delta_raw_at(raw, ldr, ring, C, taps, ck, m - j, pos0), k[i]);
-            }
-            q[i] = l_silu(q[i]);
-            k[i] = l_silu(k[i]);
-            qq = fmaf(q[i], q[i], qq);
-            kk = fmaf(k[i], k[i], kk);
+    for (int i = 0; i < NE; i++) {
+        const int e = lane + 64 * i, ch = unit * d.D + min(e, d.D - 1);
+        delta_conv_rows(conv, raw, ldr, ring, C, taps, ch, m0, M, pos0, q[i]);
+        delta_conv_rows(conv, raw, ldr, ring, C, taps, GD + ch, m0, M, pos0, k[i]);
+        if (e >= d.D)
+#pragma unroll
+            for (int j = 0; j < PREP_T; j++) q[i][j] = k[i][j] = 0.0f;
+    }
+    const float qs = 1.0f / sqrtf((float)d.D);
+#pragma unroll
+    for (int j = 0; j < PREP_T; j++) {
+        float qq = 0.0f, kk = 0.0f, qk = 0.0f;
+#pragma unroll
+        for (int i = 0; i < NE; i++) {
+            qq = fmaf(q[i][j], q[i][j], qq);
+            kk = fmaf(k[i][j], k[i][j], kk);
+            qk = fmaf(q[i][j], k[i][j], qk);
         }
         const float rq = qs / sqrtf(l_wave_sum(qq) + 1e-6f), rk = 1.0f / sqrtf(l_wave_sum(kk) + 1e-6f);
+        qk = l_wave_sum(qk);
+        const int m = m0 + j;
+        if (m >= M) break;
 #pragma unroll
-        for (int i = 0; i < 4; i++) {
+        for (int i = 0; i < NE; i++) {
             const int e = lane + 64 * i;
             if (e >= d.D) continue;
-            q[i] *= rq;
-            k[i] *= rk;
-            qk = fmaf(q[i], k[i], qk);
-            qkv[(int64_t)m * C + unit * d.D + e] = q[i];
-            qkv[(int64_t)m * C + GD + unit * d.D + e] = k[i];
+            qkv[(int64_t)m * C + unit * d.D + e] = q[i][j] * rq;
+            qkv[(int64_t)m * C + GD + unit * d.D + e] = k[i][j] * rk;
         }
-        qk = l_wave_sum(qk);
-        if (lane == 0) kq[(int64_t)m * d.G + unit] = qk;
+        if (lane == 0) kq[(int64_t)m * d.G + unit] = qk * rq * rk;
     }
 }
 
@@ -286,10 +321,22 @@ hipError_t k_delta_prepare(hipStream_t s, const DeltaShape &d, const float *conv
                            int prec) {
     if (d.D > 256 || M < 1) return hipErrorInvalidValue;
     const dim3 grid((unsigned)((d.G + d.H + 1 + 3) / 4), (unsigned)((M + PREP_T - 1) / PREP_T));
-    if (prec)
-        hipLaunchKernelGGL((delta_prepare_kernel<1>), grid, dim3(256), 0, s, d, conv, raw, ldr, ring, M, pos0, qkv, kq, beta, fa, lfa, fg, lfg);
-    else
-        hipLaunchKernelGGL((delta_prepare_kernel<0>), grid, dim3(256), 0, s, d, conv, raw, ldr, ring, M, pos0, qkv, kq, beta, fa, lfa, fg, lfg);
+#define GO(N)                                                                                                                            \
+    do {                                                                                                                                 \
+        if (prec)                                                                                                                        \
+            hipLaunchKernelGGL((delta_prepare_kernel<1, N>), grid, dim3(256), 0, s, d, conv, raw, ldr, ring, M, pos0, qkv, kq, beta, fa, \
+                               lfa, fg, lfg);                                                                                            \
+        else                                                                                                                             \
+            hipLaunchKernelGGL((delta_prepare_kernel<0, N>), grid, dim3(256), 0, s, d, conv, raw, ldr, ring, M, pos0, qkv, kq, beta, fa, \
+                               lfa, fg, lfg);                                                                                            \
+    } while (0)
+    switch ((d.D + 63) / 64) {
+    case 1: GO(1); break;
+    case 2: GO(2); break;
+    case 3: GO(3); break;
+    default: GO(4); break;
+    }
+#undef GO
     return hipGetLastError();
 }
 
@@ -451,26 +498,40 @@ typedef float d_f32x4 __attribute__((ext_vector_type(4)));
 __host__ __device__ static inline int delta_chunk_tiles(int D) { return (D + 63) / 64 * 4; }
 __host__ __device__ static inline int64_t delta_chunk_floats(int NT) { return (int64_t)NT * 784 + 512; }
 
+template <int NW>
 __global__ __launch_bounds__(256) void delta_chunk_kernel(DeltaShape d, const float *qkv, const float *beta, const float *lg, int M,
                                                           float *rec) {
-    extern __shared__ __align__(16) float s_mem[];
-    const int NT = delta_chunk_tiles(d.D), DP = 16 * NT, t = threadIdx.x, lane = t & 63, wave = t >> 6;
-    float *s_q = s_mem, *s_k = s_q + CH_T * DP, *s_g = s_k + CH_T * DP;  // [16][DP]; s_g: decays, then their logarithms' sums
+    constexpr int NT = 4 * NW, DP = 16 * NT;
+    const int t = threadIdx.x, lane = t & 63, wave = t >> 6;
+    // s_g: the decays, then their logarithms' sums
+    __shared__ __align__(16) float s_q[CH_T * DP], s_k[CH_T * DP], s_g[CH_T * DP];
     __shared__ float s_A[CH_T][CH_T + 1], s_B[CH_T][CH_T + 1], s_T[CH_T][CH_T + 1], s_b[CH_T];
     const int ch = blockIdx.x, h = blockIdx.y, kvh = h / (d.H / d.G), m0 = ch * CH_T, n = min(CH_T, M - m0);
     const int D = d.D, C = d.channels(), GD = d.G * D;
-    for (int i = t; i < CH_T * DP; i += 256) {
-        const int tt = i / DP, e = i - tt * DP;
-        float q = 0.0f, k = 0.0f, g = 1.0f;
-        if (tt < n && e < D) {
-            const float *row = qkv + (int64_t)(m0 + tt) * C + kvh * D + e;
-            q = row[0];
-            k = row[GD];
-            g = expf(lg[((int64_t)(m0 + tt) * d.H + h) * D + e]);
+    // a thread has one column of 16 / (256 / columns) rows at a time: column e, rows r0, r0 + RS, ...
+    constexpr int CB = DP < 256 ? DP : 256, RS = 256 / CB, NR = CH_T / RS;  // (DP: 64, 128, 192 or 256)
+    const int e0 = t % CB, r0 = t / CB;
+    float l[NR];
+    if (r0 < RS) {
+        float q[NR], k[NR];
+#pragma unroll
+        for (int i = 0; i < NR; i++) {
+            const int tt = r0 + RS * i;
+            q[i] = k[i] = l[i] = 0.0f;
+            if (tt < n && e0 < D) {
+                const float *row = qkv + (int64_t)(m0 + tt) * C + kvh * D + e0;
+                q[i] = row[0];
+                k[i] = row[GD];
+                l[i] = lg[((int64_t)(m0 + tt) * d.H + h) * D + e0];
+            }
         }
-        s_q[i] = q;
-        s_k[i] = k;
-        s_g[i] = g;
+#pragma unroll
+        for (int i = 0; i < NR; i++) {
+            const int at = (r0 + RS * i) * DP + e0;
+            s_q[at] = q[i];
+            s_k[at] = k[i];
+            s_g[at] = expf(l[i]);
+        }
     }
     if (t < CH_T) s_b[t] = t < n ? beta[(int64_t)(m0 + t) * d.H + h] : 0.0f;
     __syncthreads();
@@ -514,11 +575,16 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(DeltaShape d, const fl
             s_T[i][t] = x[i];
         }
     }
-    // sums of the logarithms, in place of the decays
+    // sums of the logarithms, in place of the decays (whose readers are done)
+    if (r0 < RS)
+#pragma unroll
+        for (int i = 0; i < NR; i++) s_g[(r0 + RS * i) * DP + e0] = l[i];
+    __syncthreads();
     for (int e = t; e < DP; e += 256) {
         float g = 0.0f;
+#pragma unroll
         for (int i = 0; i < CH_T; i++) {
-            if (i < n && e < D) g += lg[((int64_t)(m0 + i) * d.H + h) * D + e];
+            g += s_g[i * DP + e];
             s_g[i * DP + e] = g;
         }
     }
@@ -562,11 +628,14 @@ struct DeltaOps {
 
 template <int NW>
 __global__ __launch_bounds__(256) void delta_walk_kernel(DeltaShape d, const float *rec, const float *qkv, float *state, int M, int pos0,
-                                                         float *o) {
+                                                         float *o, unsigned n_cb, unsigned n_items, unsigned per) {
     __shared__ __align__(16) d_f32x4 s_w[2][4][64], s_o[2][4][64];
     constexpr int NT = 4 * NW;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, col = lane & 15, q4 = 4 * (lane >> 4);
-    const int h = blockIdx.y, c = blockIdx.x * 16 + col, D = d.D, V = d.V, C = d.channels();
+    // the workgroups of a head read the same records: they are dealt to one of the 8 XCDs (workgroups go to them in turn)
+    const unsigned item = (blockIdx.x & 7u) * per + (blockIdx.x >> 3);
+    if (item >= n_items) return;
+    const int h = (int)(item / n_cb), c = (int)(item % n_cb) * 16 + col, D = d.D, V = d.V, C = d.channels();
     const bool live = c < V;
     float *S = state + (int64_t)h * D * V;
     d_f32x4 s[NW];
@@ -603,38 +672,51 @@ __global__ __launch_bounds__(256) void delta_walk_kernel(DeltaShape d, const flo
         const float v = s_o[b][0][lane][wave] + s_o[b][1][lane][wave] + s_o[b][2][lane][wave] + s_o[b][3][lane][wave];
         if (live && m < M) o[((int64_t)m * d.H + h) * V + c] = v;
     };
-    DeltaOps<NW> cur, nxt;
-    fetch(cur, 0);
-    for (int ch = 0; ch < n_ch; ch++) {
+    auto walk = [&](DeltaOps<NW> &x, int ch) {
         const int b = ch & 1;
-        fetch(nxt, min(ch + 1, n_ch - 1));
         d_f32x4 w = {0.f, 0.f, 0.f, 0.f}, y = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int i = 0; i < NW; i++)
 #pragma unroll
-            for (int r = 0; r < 4; r++) w = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.kt[i][r], s[i][r], w, 0, 0, 0);
+            for (int r = 0; r < 4; r++) w = __builtin_amdgcn_mfma_f32_16x16x4f32(x.kt[i][r], s[i][r], w, 0, 0, 0);
         s_w[b][wave][lane] = w;
 #pragma unroll
         for (int i = 0; i < NW; i++)
 #pragma unroll
-            for (int r = 0; r < 4; r++) y = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.qt[i][r], s[i][r], y, 0, 0, 0);
-        __syncthreads();  // (also: the parts of the previous chunk's output are all there)
+            for (int r = 0; r < 4; r++) y = __builtin_amdgcn_mfma_f32_16x16x4f32(x.qt[i][r], s[i][r], y, 0, 0, 0);
+        // LDS writes done, then the barrier (which also says that the parts of the previous chunk's output are all there);
+        // the operands under way from memory are not waited for
+        asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
         if (ch) put(ch - 1);
         w = s_w[b][0][lane] + s_w[b][1][lane] + s_w[b][2][lane] + s_w[b][3][lane];
         d_f32x4 u = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int r = 0; r < 4; r++) u = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.T[r], cur.v[r] - w[r], u, 0, 0, 0);
+        for (int r = 0; r < 4; r++) u = __builtin_amdgcn_mfma_f32_16x16x4f32(x.T[r], x.v[r] - w[r], u, 0, 0, 0);
         // B U: this wavefront's quarter of the contracted tokens
         const float uw = wave == 0 ? u[0] : wave == 1 ? u[1] : wave == 2 ? u[2] : u[3];
-        y = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.B, uw, y, 0, 0, 0);
+        y = __builtin_amdgcn_mfma_f32_16x16x4f32(x.B, uw, y, 0, 0, 0);
 #pragma unroll
         for (int i = 0; i < NW; i++) {
-            s[i] *= cur.gc[i];
+            s[i] *= x.gc[i];
 #pragma unroll
-            for (int r = 0; r < 4; r++) s[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.kh[i][r], u[r], s[i], 0, 0, 0);
+            for (int r = 0; r < 4; r++) s[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.kh[i][r], u[r], s[i], 0, 0, 0);
         }
         s_o[b][wave][lane] = y;
-        cur = nxt;
+    };
+    // the operands of three chunks are held or under way
+    DeltaOps<NW> x0, x1, x2;
+    fetch(x0, 0);
+    fetch(x1, min(1, n_ch - 1));
+    fetch(x2, min(2, n_ch - 1));
+    for (int ch = 0; ch < n_ch; ch += 3) {  // (n_ch is the same for every wavefront: so is every barrier)
+        walk(x0, ch);
+        fetch(x0, min(ch + 3, n_ch - 1));
+        if (ch + 1 >= n_ch) break;
+        walk(x1, ch + 1);
+        fetch(x1, min(ch + 4, n_ch - 1));
+        if (ch + 2 >= n_ch) break;
+        walk(x2, ch + 2);
+        fetch(x2, min(ch + 5, n_ch - 1));
     }
     __syncthreads();
     put(n_ch - 1);
@@ -653,11 +735,14 @@ int64_t delta_walk_floats(const DeltaShape &d, int M) {
 hipError_t k_delta_walk(hipStream_t s, const DeltaShape &d, const float *qkv, const float *beta, const float *lg, float *state, int M,
                         int pos0, float *rec, float *o) {
     if (d.D > 256 || M < 1) return hipErrorInvalidValue;
-    const int NT = delta_chunk_tiles(d.D);
-    const dim3 g1((unsigned)((M + CH_T - 1) / CH_T), (unsigned)d.H), g2((unsigned)((d.V + 15) / 16), (unsigned)d.H);
-    hipLaunchKernelGGL(delta_chunk_kernel, g1, dim3(256), (size_t)3 * CH_T * 16 * NT * sizeof(float), s, d, qkv, beta, lg, M, rec);
-#define GO(N) hipLaunchKernelGGL((delta_walk_kernel<N>), g2, dim3(256), 0, s, d, rec, qkv, state, M, pos0, o)
-    switch (NT / 4) {
+    const dim3 g1((unsigned)((M + CH_T - 1) / CH_T), (unsigned)d.H);
+    const unsigned n_cb = (unsigned)((d.V + 15) / 16), n_items = n_cb * (unsigned)d.H, per = (n_items + 7) / 8;
+#define GO(N)                                                                                                                      \
+    do {                                                                                                                           \
+        hipLaunchKernelGGL((delta_chunk_kernel<N>), g1, dim3(256), 0, s, d, qkv, beta, lg, M, rec);                                \
+        hipLaunchKernelGGL((delta_walk_kernel<N>), dim3(8 * per), dim3(256), 0, s, d, rec, qkv, state, M, pos0, o, n_cb, n_items, per); \
+    } while (0)
+    switch (delta_chunk_tiles(d.D) / 4) {
     case 1: GO(1); break;
     case 2: GO(2); break;
     case 3: GO(3); break;

@@ -208,7 +208,8 @@ hipError_t k_gemm(hipStream_t s, const GemmArgs &a, int prec, int epi) {
 // ---------------------------------------------------------------------------------------------------------------
 // rows: pending update, norm, conversion to activations
 // ---------------------------------------------------------------------------------------------------------------
-template <int PREC>
+// NQ: quads of elements a thread holds (K a multiple of 4, at most 1024 NQ); 0: any K, element by element
+template <int PREC, int NQ>
 __global__ __launch_bounds__(256) void norm_rows_kernel(float *X, int K, const float *w, float eps, const float *Y, const float *yw,
                                                         float mult, const int32_t *gather, void *outa, int64_t lda) {
     __shared__ float s_red[4];
@@ -216,6 +217,56 @@ __global__ __launch_bounds__(256) void norm_rows_kernel(float *X, int K, const f
     float *x = X + src * K;
     const float *y = Y ? Y + src * K : nullptr;
     const int t = threadIdx.x;
+    if constexpr (NQ > 0) {
+        float4 v[NQ];
+#pragma unroll
+        for (int u = 0; u < NQ; u++) {
+            const int i = 4 * (t + 256 * u);
+            v[u] = i < K ? *(const float4 *)(x + i) : make_float4(0.f, 0.f, 0.f, 0.f);
+        }
+        if (y) {
+            float4 z[NQ];
+            float ss = 0.0f;
+#pragma unroll
+            for (int u = 0; u < NQ; u++) {
+                const int i = 4 * (t + 256 * u);
+                z[u] = i < K ? *(const float4 *)(y + i) : make_float4(0.f, 0.f, 0.f, 0.f);
+                ss = fmaf(z[u].x, z[u].x, fmaf(z[u].y, z[u].y, fmaf(z[u].z, z[u].z, fmaf(z[u].w, z[u].w, ss))));
+            }
+            const float f = mult / sqrtf(l_block_sum(ss, s_red) / (float)K + eps);
+#pragma unroll
+            for (int u = 0; u < NQ; u++) {
+                const int i = 4 * (t + 256 * u);
+                if (i >= K) continue;
+                const float4 g = *(const float4 *)(yw + i);
+                v[u].x = fmaf(f * z[u].x, g.x, v[u].x);
+                v[u].y = fmaf(f * z[u].y, g.y, v[u].y);
+                v[u].z = fmaf(f * z[u].z, g.z, v[u].z);
+                v[u].w = fmaf(f * z[u].w, g.w, v[u].w);
+                *(float4 *)(x + i) = v[u];
+            }
+        }
+        float r = 1.0f;
+        if (w) {
+            float ss = 0.0f;
+#pragma unroll
+            for (int u = 0; u < NQ; u++) ss = fmaf(v[u].x, v[u].x, fmaf(v[u].y, v[u].y, fmaf(v[u].z, v[u].z, fmaf(v[u].w, v[u].w, ss))));
+            r = 1.0f / sqrtf(l_block_sum(ss, s_red) / (float)K + eps);
+        }
+        if (!outa) return;
+#pragma unroll
+        for (int u = 0; u < NQ; u++) {
+            const int i = 4 * (t + 256 * u);
+            if (i >= lda) continue;
+            const float4 g = w && i < K ? *(const float4 *)(w + i) : make_float4(1.f, 1.f, 1.f, 1.f);
+            const float4 q = make_float4(v[u].x * r * g.x, v[u].y * r * g.y, v[u].z * r * g.z, v[u].w * r * g.w);
+            if (PREC)
+                *(float4 *)((float *)outa + m * lda + i) = q;
+            else
+                *(uint2 *)((uint16_t *)outa + m * lda + i) = make_uint2(l_pack_bf16(q.x, q.y), l_pack_bf16(q.z, q.w));
+        }
+        return;
+    }
     float ry = 0.0f;
     if (y) {
         float ss = 0.0f;
@@ -245,10 +296,26 @@ __global__ __launch_bounds__(256) void norm_rows_kernel(float *X, int K, const f
 hipError_t k_norm_rows(hipStream_t s, float *x, int K, int M, const float *w, float eps, const float *y, const float *yw,
                        float mult, const int32_t *gather, void *outa, int64_t lda, int prec) {
     if (M < 1 || (y && gather)) return hipErrorInvalidValue;
-    if (prec)
-        hipLaunchKernelGGL((norm_rows_kernel<1>), dim3((unsigned)M), dim3(256), 0, s, x, K, w, eps, y, yw, mult, gather, outa, lda);
+#define GO(N)                                                                                                                             \
+    do {                                                                                                                                  \
+        if (prec)                                                                                                                         \
+            hipLaunchKernelGGL((norm_rows_kernel<1, N>), dim3((unsigned)M), dim3(256), 0, s, x, K, w, eps, y, yw, mult, gather, outa, lda); \
+        else                                                                                                                              \
+            hipLaunchKernelGGL((norm_rows_kernel<0, N>), dim3((unsigned)M), dim3(256), 0, s, x, K, w, eps, y, yw, mult, gather, outa, lda); \
+    } while (0)
+    // (lda, a multiple of 64, may exceed K by up to 63 columns: they are covered, too)
+    const int64_t cols = std::max<int64_t>(K, outa ? lda : 0);
+    if (K % 4 != 0 || cols > 8192)
+        GO(0);
+    else if (cols <= 1024)
+        GO(1);
+    else if (cols <= 2048)
+        GO(2);
+    else if (cols <= 4096)
+        GO(4);
     else
-        hipLaunchKernelGGL((norm_rows_kernel<0>), dim3((unsigned)M), dim3(256), 0, s, x, K, w, eps, y, yw, mult, gather, outa, lda);
+        GO(8);
+#undef GO
     return hipGetLastError();
 }
 
@@ -318,14 +385,30 @@ hipError_t k_group(hipStream_t s, const int32_t *choice, const float *score, int
 
 __global__ __launch_bounds__(256) void gather_add_kernel(float *x, const float *y, const int32_t *slot_of, int top, int K, float mult) {
     const int64_t m = blockIdx.y;
-    const int i = blockIdx.x * 256 + threadIdx.x;
+    const int i = 4 * (blockIdx.x * 256 + threadIdx.x);
     if (i >= K) return;
-    float v = 0.0f;
-    for (int k = 0; k < top; k++) v += y[(int64_t)slot_of[m * top + k] * K + i];
-    x[m * K + i] = fmaf(mult, v, x[m * K + i]);
+    if (K % 4 == 0) {
+        const float4 a = *(const float4 *)(x + m * K + i);
+        float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll 4
+        for (int k = 0; k < top; k++) {
+            const float4 q = *(const float4 *)(y + (int64_t)slot_of[m * top + k] * K + i);
+            v.x += q.x;
+            v.y += q.y;
+            v.z += q.z;
+            v.w += q.w;
+        }
+        *(float4 *)(x + m * K + i) = make_float4(fmaf(mult, v.x, a.x), fmaf(mult, v.y, a.y), fmaf(mult, v.z, a.z), fmaf(mult, v.w, a.w));
+        return;
+    }
+    for (int e = i; e < min(i + 4, K); e++) {
+        float v = 0.0f;
+        for (int k = 0; k < top; k++) v += y[(int64_t)slot_of[m * top + k] * K + e];
+        x[m * K + e] = fmaf(mult, v, x[m * K + e]);
+    }
 }
 hipError_t k_gather_add(hipStream_t s, float *x, const float *y, const int32_t *slot_of, int M, int top, int K, float mult) {
-    hipLaunchKernelGGL(gather_add_kernel, dim3((unsigned)((K + 255) / 256), (unsigned)M), dim3(256), 0, s, x, y, slot_of, top, K, mult);
+    hipLaunchKernelGGL(gather_add_kernel, dim3((unsigned)((K + 1023) / 1024), (unsigned)M), dim3(256), 0, s, x, y, slot_of, top, K, mult);
     return hipGetLastError();
 }
 

@@ -31,11 +31,11 @@ __device__ __forceinline__ void gemm_store4(const GemmArgs &a, int64_t m, int64_
                 continue;
             }
             if (EPI == GE_UP)
-                v[e] = l_act(a.act, a.row_scale[m] * v[e]);
+                v[e] = l_act_rounded<PREC>(a.act, a.row_scale[m] * v[e]);
             else if (EPI == GE_EMBED)
-                v[e] = l_act(a.act, v[e]) * l_bf16(a.emb[(int64_t)a.tokens[m] * a.emb_ld + L + e]);
+                v[e] = l_act_rounded<PREC>(a.act, v[e]) * l_bf16(a.emb[(int64_t)a.tokens[m] * a.emb_ld + L + e]);
             else
-                v[e] = l_act(a.act, v[e]);
+                v[e] = l_act_rounded<PREC>(a.act, v[e]);
         }
         if (PREC)
             *(float4 *)((float *)a.outa + m * a.lda + L) = make_float4(v[0], v[1], v[2], v[3]);

@@ -208,6 +208,7 @@ hipError_t k_delta_step(hipStream_t s, const DeltaShape &d, const DeltaWeights &
 // many tokens: convolutions and unit vectors.  A wavefront takes one unit (a key head's q and k, or a value head, or the
 // rest of the row) over PREP_T consecutive tokens.
 // ---------------------------------------------------------------------------------------------------------------
+#define CH_T 16  // tokens of a chunk of the recurrence
 #define PREP_T 8
 
 // CONV_AHEAD - 1 + PREP_T inputs of a channel (tokens m0 - CONV_AHEAD + 1 .. m0 + PREP_T - 1) are fetched together, then the
@@ -275,8 +276,8 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(DeltaShape d, const 
             float y[PREP_T];
             delta_conv_rows(conv, raw, ldr, ring, C, taps, ch0 + e, m0, M, pos0, y);
 #pragma unroll
-            for (int i = 0; i < PREP_T; i++)
-                if (m0 + i < M) qkv[(int64_t)(m0 + i) * C + ch0 + e] = y[i];
+            for (int i = 0; i < PREP_T; i++)  // (rows of v are zero from M to the end of the last chunk)
+                qkv[(int64_t)(m0 + i) * C + ch0 + e] = m0 + i < M ? y[i] : 0.0f;
         }
         return;
     }
@@ -320,7 +321,7 @@ hipError_t k_delta_prepare(hipStream_t s, const DeltaShape &d, const float *conv
                            int M, int pos0, float *qkv, float *kq, float *beta, void *fa, int64_t lfa, void *fg, int64_t lfg,
                            int prec) {
     if (d.D > 256 || M < 1) return hipErrorInvalidValue;
-    const dim3 grid((unsigned)((d.G + d.H + 1 + 3) / 4), (unsigned)((M + PREP_T - 1) / PREP_T));
+    const dim3 grid((unsigned)((d.G + d.H + 1 + 3) / 4), (unsigned)((M + CH_T - 1) / CH_T * (CH_T / PREP_T)));
 #define GO(N)                                                                                                                            \
     do {                                                                                                                                 \
         if (prec)                                                                                                                        \
@@ -490,7 +491,6 @@ hipError_t k_delta_scan(hipStream_t s, const DeltaShape &d, const float *qkv, co
 // indexes taken as k = 4 (l / 16) + r, a result is the next product's B operand as it stands, and an A operand's four steps are
 // one 16-byte word of lane l: (row l % 16; columns 4 (l / 16) .. + 3).
 // ---------------------------------------------------------------------------------------------------------------
-#define CH_T 16
 typedef float d_f32x4 __attribute__((ext_vector_type(4)));
 
 // the record of one (chunk, head): NT tiles of 16 key channels (a multiple of 4); kt, qt, kh: [NT][64][4]; T, B: [64][4];
@@ -626,16 +626,18 @@ struct DeltaOps {
     float B, v[4];
 };
 
+// (records, rows of v and rows of o exist for whole chunks: a sequence's last chunk is filled up with zero rows)
 template <int NW>
 __global__ __launch_bounds__(256) void delta_walk_kernel(DeltaShape d, const float *rec, const float *qkv, float *state, int M, int pos0,
                                                          float *o, unsigned n_cb, unsigned n_items, unsigned per) {
-    __shared__ __align__(16) d_f32x4 s_w[2][4][64], s_o[2][4][64];
+    __shared__ __align__(16) d_f32x4 s_w[2][4][64];
+    __shared__ float s_o[2][4][4][64];
     constexpr int NT = 4 * NW;
-    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, col = lane & 15, q4 = 4 * (lane >> 4);
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), col = lane & 15, q4 = 4 * (lane >> 4);
     // the workgroups of a head read the same records: they are dealt to one of the 8 XCDs (workgroups go to them in turn)
     const unsigned item = (blockIdx.x & 7u) * per + (blockIdx.x >> 3);
     if (item >= n_items) return;
-    const int h = (int)(item / n_cb), c = (int)(item % n_cb) * 16 + col, D = d.D, V = d.V, C = d.channels();
+    const int h = (int)(item / n_cb), c = (int)(item % n_cb) * 16 + col, D = d.D, V = d.V, C = d.channels(), HV = d.H * V;
     const bool live = c < V;
     float *S = state + (int64_t)h * D * V;
     d_f32x4 s[NW];
@@ -647,30 +649,37 @@ __global__ __launch_bounds__(256) void delta_walk_kernel(DeltaShape d, const flo
             s[i][r] = (live && e < D && pos0 > 0) ? S[(int64_t)e * V + c] : 0.0f;
         }
     const int n_ch = (M + CH_T - 1) / CH_T;
-    const float *vcol = qkv + 2 * d.G * D + h * V + (live ? c : 0);
+    // wavefront-uniform bases and this lane's fixed offsets from them
+    const float *rec_h = rec + (int64_t)h * delta_chunk_floats(NT) + 256 * (wave * NW);
+    const int64_t rec_step = (int64_t)d.H * delta_chunk_floats(NT);
+    const float *v_h = qkv + 2 * d.G * D + h * V;
+    float *o_h = o + (int64_t)wave * HV + h * V;
+    const unsigned l4 = 4u * lane, ov = (unsigned)(q4 * HV + c);
+    unsigned vv[4];
+#pragma unroll
+    for (int r = 0; r < 4; r++) vv[r] = (unsigned)((q4 + r) * C + (live ? c : 0));
     auto fetch = [&](DeltaOps<NW> &x, int ch) {
-        const float *p = rec + ((int64_t)ch * d.H + h) * delta_chunk_floats(NT);
+        const float *p = rec_h + ch * rec_step;
 #pragma unroll
         for (int i = 0; i < NW; i++) {
-            const int tile = wave * NW + i;
-            x.kt[i] = *(const d_f32x4 *)(p + 256 * tile + 4 * lane);
-            x.qt[i] = *(const d_f32x4 *)(p + 256 * (NT + tile) + 4 * lane);
-            x.kh[i] = *(const d_f32x4 *)(p + 256 * (2 * NT + tile) + 4 * lane);
-            x.gc[i] = *(const d_f32x4 *)(p + 768 * NT + 512 + 16 * tile + q4);
+            x.kt[i] = *(const d_f32x4 *)(p + 256 * i + l4);
+            x.qt[i] = *(const d_f32x4 *)(p + 256 * (NT + i) + l4);
+            x.kh[i] = *(const d_f32x4 *)(p + 256 * (2 * NT + i) + l4);
         }
-        x.T = *(const d_f32x4 *)(p + 768 * NT + 4 * lane);
-        x.B = p[768 * NT + 256 + 4 * lane + wave];
+        p -= 256 * (wave * NW);
 #pragma unroll
-        for (int r = 0; r < 4; r++) {
-            const int m = ch * CH_T + q4 + r;
-            x.v[r] = (live && m < M) ? vcol[(int64_t)m * C] : 0.0f;
-        }
+        for (int i = 0; i < NW; i++) x.gc[i] = *(const d_f32x4 *)(p + 768 * NT + 512 + 16 * (wave * NW + i) + q4);
+        x.T = *(const d_f32x4 *)(p + 768 * NT + l4);
+        x.B = (p + wave)[768 * NT + 256 + l4];
+        const float *v = v_h + (int64_t)ch * CH_T * C;
+#pragma unroll
+        for (int r = 0; r < 4; r++) x.v[r] = v[vv[r]];
     };
     // the output row 4 (lane / 16) + wave of a chunk, from the four wavefronts' parts
     auto put = [&](int ch) {
-        const int m = ch * CH_T + q4 + wave, b = ch & 1;
-        const float v = s_o[b][0][lane][wave] + s_o[b][1][lane][wave] + s_o[b][2][lane][wave] + s_o[b][3][lane][wave];
-        if (live && m < M) o[((int64_t)m * d.H + h) * V + c] = v;
+        const int b = ch & 1;
+        const float y = s_o[b][wave][0][lane] + s_o[b][wave][1][lane] + s_o[b][wave][2][lane] + s_o[b][wave][3][lane];
+        if (live) (o_h + (int64_t)ch * CH_T * HV)[ov] = y;
     };
     auto walk = [&](DeltaOps<NW> &x, int ch) {
         const int b = ch & 1;
@@ -687,21 +696,22 @@ __global__ __launch_bounds__(256) void delta_walk_kernel(DeltaShape d, const flo
         // LDS writes done, then the barrier (which also says that the parts of the previous chunk's output are all there);
         // the operands under way from memory are not waited for
         asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
-        if (ch) put(ch - 1);
         w = s_w[b][0][lane] + s_w[b][1][lane] + s_w[b][2][lane] + s_w[b][3][lane];
         d_f32x4 u = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int r = 0; r < 4; r++) u = __builtin_amdgcn_mfma_f32_16x16x4f32(x.T[r], x.v[r] - w[r], u, 0, 0, 0);
-        // B U: this wavefront's quarter of the contracted tokens
-        const float uw = wave == 0 ? u[0] : wave == 1 ? u[1] : wave == 2 ? u[2] : u[3];
-        y = __builtin_amdgcn_mfma_f32_16x16x4f32(x.B, uw, y, 0, 0, 0);
 #pragma unroll
         for (int i = 0; i < NW; i++) {
             s[i] *= x.gc[i];
 #pragma unroll
             for (int r = 0; r < 4; r++) s[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.kh[i][r], u[r], s[i], 0, 0, 0);
         }
-        s_o[b][wave][lane] = y;
+        // B U: this wavefront's quarter of the contracted tokens
+        const float uw = wave == 0 ? u[0] : wave == 1 ? u[1] : wave == 2 ? u[2] : u[3];
+        y = __builtin_amdgcn_mfma_f32_16x16x4f32(x.B, uw, y, 0, 0, 0);
+        if (ch) put(ch - 1);
+#pragma unroll
+        for (int r = 0; r < 4; r++) s_o[b][r][wave][lane] = y[r];
     };
     // the operands of three chunks are held or under way
     DeltaOps<NW> x0, x1, x2;

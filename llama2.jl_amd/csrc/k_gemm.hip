@@ -351,7 +351,7 @@ hipError_t k_route(hipStream_t s, const float *z, int M, int E, int top, int32_t
 // one workgroup: counts, offsets, slots and the list of tiles.  The order of an expert's slots is whatever the LDS counters
 // give; every slot is computed on its own, so no result depends on it.
 __global__ __launch_bounds__(1024) void group_kernel(const int32_t *choice, const float *score, int M, int E, int top, int32_t *slot_row,
-                                                     float *slot_scale, int32_t *slot_of, GemmTile *tiles, int32_t *n_tiles) {
+                                                     float *slot_scale, int32_t *slot_of, GemmTile *tiles, int32_t *n_tiles, int tile_rows) {
     extern __shared__ __align__(16) int s_int[];
     int *cnt = s_int, *off = s_int + E;
     const int n = M * top;
@@ -363,7 +363,7 @@ __global__ __launch_bounds__(1024) void group_kernel(const int32_t *choice, cons
         int o = 0, nt = 0;
         for (int e = 0; e < E; e++) {
             off[e] = o;
-            for (int r = 0; r < cnt[e]; r += L_GEMM_TILE) tiles[nt++] = GemmTile{e, o + r, min(L_GEMM_TILE, cnt[e] - r)};
+            for (int r = 0; r < cnt[e]; r += tile_rows) tiles[nt++] = GemmTile{e, o + r, min(tile_rows, cnt[e] - r)};
             o += cnt[e];
         }
         n_tiles[0] = nt;
@@ -377,9 +377,9 @@ __global__ __launch_bounds__(1024) void group_kernel(const int32_t *choice, cons
     }
 }
 hipError_t k_group(hipStream_t s, const int32_t *choice, const float *score, int M, int E, int top, int32_t *slot_row,
-                   float *slot_scale, int32_t *slot_of, GemmTile *tiles, int32_t *n_tiles) {
+                   float *slot_scale, int32_t *slot_of, GemmTile *tiles, int32_t *n_tiles, int tile_rows) {
     hipLaunchKernelGGL(group_kernel, dim3(1), dim3(1024), 2 * E * sizeof(int), s, choice, score, M, E, top, slot_row, slot_scale, slot_of,
-                       tiles, n_tiles);
+                       tiles, n_tiles, tile_rows);
     return hipGetLastError();
 }
 

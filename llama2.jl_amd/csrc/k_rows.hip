@@ -70,7 +70,7 @@ __global__ __launch_bounds__(ROWS_THREADS) void rows_kernel(RowsArgs a, int rows
     auto row_ptrs = [&](int64_t r, int v, const uint16_t *&w0, const uint16_t *&w1) {
         const int64_t r1 = r + 1 < row_end ? r + 1 : r;
         if (PRO == RP_UP) {
-            const int64_t e0 = r / a.rows_each, e1 = r1 / a.rows_each;
+            const unsigned n = (unsigned)a.rows_each, e0 = (unsigned)r / n, e1 = (unsigned)r1 / n;
             w0 = a.w + ((int64_t)s_sel[e0] * a.rows_each + (r - e0 * a.rows_each)) * ld;
             w1 = a.w + ((int64_t)s_sel[e1] * a.rows_each + (r1 - e1 * a.rows_each)) * ld;
         } else if (PRO == RP_DOWN) {
@@ -300,7 +300,7 @@ __global__ __launch_bounds__(ROWS_THREADS) void rows_kernel(RowsArgs a, int rows
                 float o = val;
                 if (EPI == RE_RESID) o = a.resid[r] + a.mult * val;
                 if (EPI == RE_ACT) o = l_act(a.act, val);
-                if (EPI == RE_UP) o = l_act(a.act, s_score[r / a.rows_each] * val);
+                if (EPI == RE_UP) o = l_act(a.act, s_score[(unsigned)r / (unsigned)a.rows_each] * val);
                 if (EPI == RE_EMBED) o = l_act(a.act, val) * l_bf16(a.emb[(int64_t)l_step_token(a.ctl, a.prompt) * a.emb_ld + r]);
                 a.out[r] = o;
             }

@@ -24,6 +24,31 @@ hipError_t k_tile_image(hipStream_t s, const uint16_t *w, int ld, int64_t rows, 
     return hipGetLastError();
 }
 
+// 256 rows of the matrix (row group nt of w) x the positions m0 .. of a block of mcount, which starts at row mb
+template <int EPI, int JT>
+__device__ __forceinline__ void tiles_item(const GemmArgs &a, const uint16_t *w, unsigned nt, int64_t mb, int m0, int mcount, uint4 *s_all) {
+    const int64_t n0 = (int64_t)nt * 256;
+    pf_tile_product<JT>(
+        w + (int64_t)nt * (a.ld >> 6) * 16384, (const uint16_t *)a.x, a.ld, s_all,
+        [&](int r) {
+            const int64_t row = mb + min(m0 + r, mcount - 1);  // (rows past the end repeat the last one; not stored)
+            return a.gather ? (int64_t)a.gather[row] : row;
+        },
+        [&](f32x16(&acc)[2][JT], int wn, int wm, int lane) {
+#pragma unroll
+            for (int j = 0; j < JT; j++) {
+                const int m = m0 + 32 * JT * wm + 32 * j + (lane & 31);
+                if (m >= mcount) continue;
+#pragma unroll
+                for (int i = 0; i < 2; i++)
+#pragma unroll
+                    for (int rq = 0; rq < 4; rq++)
+                        gemm_store4<0, EPI>(a, mb + m, n0 + 64 * wn + 32 * i + 8 * rq + 4 * (lane >> 5), acc[i][j][4 * rq],
+                                            acc[i][j][4 * rq + 1], acc[i][j][4 * rq + 2], acc[i][j][4 * rq + 3]);
+            }
+        });
+}
+
 // Items (row group of 256, block of 64 JT positions) are dealt to the 8 XCDs as contiguous runs: positions fastest in a single
 // product, so that workgroups on one weight tile share an L2; row groups fastest in a grouped one, where a block of positions
 // is used with one expert's matrix only.
@@ -47,26 +72,11 @@ __global__ __launch_bounds__(512) void tiles_kernel(GemmArgs a, unsigned n_nt, u
         nt = item / n_mt;
         m0 = (int)(item % n_mt) * 64 * JT;
     }
-    const int64_t n0 = (int64_t)nt * 256;
-    pf_tile_product<JT>(
-        w + (int64_t)nt * (a.ld >> 6) * 16384, (const uint16_t *)a.x, a.ld, s_all,
-        [&](int r) {
-            const int64_t row = mb + min(m0 + r, mcount - 1);  // (rows past the end repeat the last one; not stored)
-            return a.gather ? (int64_t)a.gather[row] : row;
-        },
-        [&](f32x16(&acc)[2][JT], int wn, int wm, int lane) {
-#pragma unroll
-            for (int j = 0; j < JT; j++) {
-                const int m = m0 + 32 * JT * wm + 32 * j + (lane & 31);
-                if (m >= mcount) continue;
-#pragma unroll
-                for (int i = 0; i < 2; i++)
-#pragma unroll
-                    for (int rq = 0; rq < 4; rq++)
-                        gemm_store4<0, EPI>(a, mb + m, n0 + 64 * wn + 32 * i + 8 * rq + 4 * (lane >> 5), acc[i][j][4 * rq],
-                                            acc[i][j][4 * rq + 1], acc[i][j][4 * rq + 2], acc[i][j][4 * rq + 3]);
-            }
-        });
+    // (a block of a grouped product that has at most 128 rows takes half the positions)
+    if (GROUPED && JT == 4 && mcount <= 128)
+        tiles_item<EPI, 2>(a, w, nt, mb, m0, mcount, s_all);
+    else
+        tiles_item<EPI, JT>(a, w, nt, mb, m0, mcount, s_all);
 }
 
 #define TILES_MAX_DEVICES 64
@@ -94,8 +104,8 @@ hipError_t k_tiles(hipStream_t s, const GemmArgs &a, int epi) {
     if (!a.w || !a.x || a.n_rows < 1 || a.M < 1 || a.ld % 64 != 0 || a.ldx != a.ld || a.lda % 64 != 0) return hipErrorInvalidValue;
     const unsigned n_nt = (unsigned)((a.n_rows + 255) / 256);
     if (a.tiles) {
-        if (epi == GE_UP && a.outa && a.lda >= a.n_rows && a.lda <= 256 * (int64_t)n_nt) return tiles_launch<GE_UP, 2, true>(s, a, n_nt, 0);
-        if (epi == GE_STORE && a.outf && a.ldo >= a.n_rows) return tiles_launch<GE_STORE, 2, true>(s, a, n_nt, 0);
+        if (epi == GE_UP && a.outa && a.lda >= a.n_rows && a.lda <= 256 * (int64_t)n_nt) return tiles_launch<GE_UP, 4, true>(s, a, n_nt, 0);
+        if (epi == GE_STORE && a.outf && a.ldo >= a.n_rows) return tiles_launch<GE_STORE, 4, true>(s, a, n_nt, 0);
         return hipErrorInvalidValue;
     }
     if (epi != GE_ACT || !a.outa || a.lda < a.n_rows || a.lda > 256 * (int64_t)n_nt) return hipErrorInvalidValue;

@@ -651,6 +651,7 @@ static int prompt_images(l2h_model *m) {
     for (LayerDev &L : l->layer) {
         if (L.d.ff == L2H_FF_DENSE) add(&L.up, L.d.ff_dim, 1);
         if (L.d.ff == L2H_FF_EXPERTS) {
+            if (std::min(L.d.ff_dim, l->W()) < L_IMAGE_MIN_ROWS) continue;  // (both or neither)
             add(&L.up, L.d.ff_dim, L.d.n_experts);
             add(&L.down, l->W(), L.d.n_experts);
         }
@@ -874,8 +875,10 @@ static hipError_t prompt_experts(l2h_model *m, LayerDev &L, int M) {
     hipError_t e;
     CK(product(m, gemm_of(L.router, l->xn, M), GE_STORE, l->zb, d.n_experts, 1.0f));
     CK(k_route(s, l->zb, M, d.n_experts, d.top, l->choice, l->score));
-    CK(k_group(s, l->choice, l->score, M, d.n_experts, d.top, l->slot_row, l->slot_scale, l->slot_of, l->tiles, l->n_tiles));
-    const int slots = M * d.top, max_tiles = (slots + L_GEMM_TILE - 1) / L_GEMM_TILE + d.n_experts;
+    const bool image = image_takes(L.up, M) && image_takes(L.down, M);
+    const int rows = image ? L_IMAGE_TILE : L_GEMM_TILE;
+    CK(k_group(s, l->choice, l->score, M, d.n_experts, d.top, l->slot_row, l->slot_scale, l->slot_of, l->tiles, l->n_tiles, rows));
+    const int slots = M * d.top, max_tiles = (slots + rows - 1) / rows + d.n_experts;
     GemmArgs up = gemm_of(L.up, l->xn, slots), down = gemm_of(L.down, l->hb, slots);
     for (GemmArgs *a : {&up, &down}) {
         a->tiles = l->tiles;
@@ -889,7 +892,7 @@ static hipError_t prompt_experts(l2h_model *m, LayerDev &L, int M) {
     up.act = d.ff_act;
     up.outa = l->hb;
     up.lda = L.down.ld;
-    if (image_takes(L.up, M)) {
+    if (image) {
         up.w = L.up.image;
         up.expert_stride = L.up.image_stride;
         CK(k_tiles(s, up, GE_UP));
@@ -900,7 +903,7 @@ static hipError_t prompt_experts(l2h_model *m, LayerDev &L, int M) {
     down.expert_stride = (int64_t)l->W() * L.down.ld;
     down.outf = l->yb;
     down.ldo = l->W();
-    if (image_takes(L.down, M)) {
+    if (image) {
         down.w = L.down.image;
         down.expert_stride = L.down.image_stride;
         CK(k_tiles(s, down, GE_STORE));

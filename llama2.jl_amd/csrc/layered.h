@@ -64,7 +64,7 @@ enum {
     GE_DECAY = 5,   // outf = -rate[n / hd] * softplus(v + bias[n]): the logarithm of a decay
     GE_SIGMOID = 6  // outf = sigmoid(v)
 };
-struct GemmTile {  // one 128-row block of a grouped product
+struct GemmTile {  // a block of rows of a grouped product
     int32_t expert, row0, n;
 };
 struct GemmArgs {
@@ -93,7 +93,8 @@ struct GemmArgs {
     int64_t expert_stride = 0;
     const int32_t *gather = nullptr;  // row of x for each row of the product
 };
-#define L_GEMM_TILE 128
+#define L_GEMM_TILE 128   // rows of a block for k_gemm ...
+#define L_IMAGE_TILE 256  // ... and for k_tiles
 hipError_t k_gemm(hipStream_t s, const GemmArgs &a, int prec, int epi);
 
 // the same from a tile image (k_tiles.hip): GE_ACT, and GE_UP / GE_STORE in the grouped form; bf16 activations
@@ -114,7 +115,7 @@ hipError_t k_norm_rows(hipStream_t s, float *x, int K, int M, const float *w, fl
 // consecutive), slot_of[M][top], tiles
 hipError_t k_route(hipStream_t s, const float *z, int M, int E, int top, int32_t *choice, float *score);
 hipError_t k_group(hipStream_t s, const int32_t *choice, const float *score, int M, int E, int top, int32_t *slot_row,
-                   float *slot_scale, int32_t *slot_of, GemmTile *tiles, int32_t *n_tiles);
+                   float *slot_scale, int32_t *slot_of, GemmTile *tiles, int32_t *n_tiles, int tile_rows);
 // x[m] += mult * sum_k y[slot_of[m][k]]
 hipError_t k_gather_add(hipStream_t s, float *x, const float *y, const int32_t *slot_of, int M, int top, int K, float mult);
 
@@ -141,7 +142,7 @@ struct DeltaWeights {
 hipError_t k_delta_step(hipStream_t s, const DeltaShape &d, const DeltaWeights &w, const float *in, float *ring, float *state,
                         const DecodeCtl *ctl, float *o, float *ssq, float *gate);
 // convolution, silu, unit vectors, beta: raw[M][ldr] -> qkv[M][channels], kq[M][G] (= k . q), beta[M][H], and the two low-rank
-// factors as activations
+// factors as activations; qkv and the scan's o have room for a multiple of 16 rows
 hipError_t k_delta_prepare(hipStream_t s, const DeltaShape &d, const float *conv, const float *raw, int64_t ldr, const float *ring,
                            int M, int pos0, float *qkv, float *kq, float *beta, void *fa, int64_t lfa, void *fg, int64_t lfg,
                            int prec);

@@ -10,13 +10,15 @@ __device__ __forceinline__ void gemm_store4(const GemmArgs &a, int64_t m, int64_
     if (EPI == GE_STORE || EPI == GE_RESID || EPI == GE_DECAY || EPI == GE_SIGMOID) {
         if (L >= a.n_rows) return;
         float *o = a.outf + m * a.ldo + L;
+        // (matrices have fewer than 2^31 rows: 32-bit division)
+        const unsigned h0 = EPI == GE_DECAY ? (unsigned)L / (unsigned)a.hd : 0u;
 #pragma unroll
         for (int e = 0; e < 4; e++) {
             if (L + e >= a.n_rows) break;
             if (EPI == GE_RESID)
                 o[e] = fmaf(a.mult, v[e], o[e]);
             else if (EPI == GE_DECAY)
-                o[e] = -a.rate[(L + e) / a.hd] * l_softplus(v[e] + a.bias[L + e]);
+                o[e] = -a.rate[a.hd % 4 == 0 ? h0 : (unsigned)(L + e) / (unsigned)a.hd] * l_softplus(v[e] + a.bias[L + e]);
             else if (EPI == GE_SIGMOID)
                 o[e] = l_sigmoid(v[e]);
             else

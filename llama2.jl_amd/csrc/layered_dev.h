@@ -18,7 +18,19 @@ __device__ __forceinline__ float l_bf16(uint16_t w) { return __uint_as_float((ui
 
 __device__ __forceinline__ float l_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
 __device__ __forceinline__ float l_silu(float z) { return z / (1.0f + expf(-z)); }
-__device__ __forceinline__ float l_softplus(float z) { return z > 20.0f ? z : log1pf(expf(z)); }
+// log(1 + exp(z)) = max(z, 0) + log(1 + e), e = exp(-|z|); log(1 + e) = 2 artanh(s), s = e / (2 + e) <= 1/3, by its power series
+// (the first term left out is 2 s^17 / 17 < 1e-9 of the sum): small relative error also where the result is small
+__device__ __forceinline__ float l_softplus(float z) {
+    const float e = expf(-fabsf(z)), s = e / (2.0f + e), q = s * s;
+    float p = fmaf(q, 1.0f / 15.0f, 1.0f / 13.0f);
+    p = fmaf(p, q, 1.0f / 11.0f);
+    p = fmaf(p, q, 1.0f / 9.0f);
+    p = fmaf(p, q, 1.0f / 7.0f);
+    p = fmaf(p, q, 1.0f / 5.0f);
+    p = fmaf(p, q, 1.0f / 3.0f);
+    p = fmaf(p, q, 1.0f);
+    return fmaf(2.0f * s, p, fmaxf(z, 0.0f));
+}
 __device__ __forceinline__ float l_act(int act, float z) {
     if (act == LACT_RELU2) {
         const float r = fmaxf(z, 0.0f);

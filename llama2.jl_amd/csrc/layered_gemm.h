@@ -12,17 +12,22 @@ __device__ __forceinline__ void gemm_store4(const GemmArgs &a, int64_t m, int64_
         float *o = a.outf + m * a.ldo + L;
         // (matrices have fewer than 2^31 rows: 32-bit division)
         const unsigned h0 = EPI == GE_DECAY ? (unsigned)L / (unsigned)a.hd : 0u;
+        auto value = [&](int e, float old) {
+            if (EPI == GE_RESID) return fmaf(a.mult, v[e], old);
+            if (EPI == GE_DECAY) return -a.rate[a.hd % 4 == 0 ? h0 : (unsigned)(L + e) / (unsigned)a.hd] * l_softplus(v[e] + a.bias[L + e]);
+            if (EPI == GE_SIGMOID) return l_sigmoid(v[e]);
+            return v[e];
+        };
+        if (a.ldo % 4 == 0 && L + 3 < a.n_rows) {
+            float4 q = make_float4(0.f, 0.f, 0.f, 0.f);
+            if (EPI == GE_RESID) q = *(const float4 *)o;
+            *(float4 *)o = make_float4(value(0, q.x), value(1, q.y), value(2, q.z), value(3, q.w));
+            return;
+        }
 #pragma unroll
         for (int e = 0; e < 4; e++) {
             if (L + e >= a.n_rows) break;
-            if (EPI == GE_RESID)
-                o[e] = fmaf(a.mult, v[e], o[e]);
-            else if (EPI == GE_DECAY)
-                o[e] = -a.rate[a.hd % 4 == 0 ? h0 : (unsigned)(L + e) / (unsigned)a.hd] * l_softplus(v[e] + a.bias[L + e]);
-            else if (EPI == GE_SIGMOID)
-                o[e] = l_sigmoid(v[e]);
-            else
-                o[e] = v[e];
+            o[e] = value(e, EPI == GE_RESID ? o[e] : 0.0f);
         }
     } else {
         if (L >= a.lda) return;  // (lda a multiple of 64: whole groups of four)

@@ -13,7 +13,8 @@ def config(name):
     """layers of the size of a real model's: three delta-rule layers to one of attention, dense and expert feed-forwards in
     turn, and the Llama shape that goes with it"""
     from . import layered as L
-    W, H, G, ff, experts, top, eff = {"vudelix-2k": (2048, 16, 4, 8192, 32, 4, 1024),
+    W, H, G, ff, experts, top, eff = {"vudelix-tiny": (512, 4, 2, 1024, 8, 2, 256),  # for a quick functional run
+                                      "vudelix-2k": (2048, 16, 4, 8192, 32, 4, 1024),
                                       "vudelix-4k": (4096, 32, 8, 14336, 64, 4, 2048)}[name]
     layers = []
     for i in range(8):

@@ -787,7 +787,7 @@ static GemmArgs gemm_of(const LMat &w, const void *x, int M) {
 // that few different shapes occur: the rows beyond M are computed from whatever the buffers hold, and never read
 static bool library_takes(const l2h_model *m, const GemmArgs &a) {
     return m->lay->c.precision == 0 && m->pf_lt && m->pf_library_mode && a.M >= L_BIG_MIN_M &&
-           (double)a.M * (double)a.n_rows * (double)a.ld >= (double)(1 << 28);
+           (double)a.M * (double)a.n_rows * (double)a.ld >= (double)(1 << 26);
 }
 static hipError_t product(l2h_model *m, GemmArgs a, int epi, float *out, int64_t ldo, float mult) {
     if (library_takes(m, a)) {

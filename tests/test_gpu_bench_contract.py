@@ -40,3 +40,12 @@ def test_bench_line_on_the_small_workload():
 def test_bench_refuses_more_than_one_gpu():
     rc, out, err = _run("--gpus", "2")
     assert rc != 0 and "gpu" in (out + err).lower()
+
+
+def test_layered_workload():
+    rc, out, err = _run("--workload", "vudelix-tiny", "--steps", "16", "--warmup", "4", "--repeats", "2")
+    assert rc == 0, err[-2000:]
+    d = json.loads([l for l in out.splitlines() if l.startswith("{")][0])
+    assert d["steps"] == 16 and d["unit"] == "tok/s" and d["value"] > 0 and d["config"]["workload"] == "vudelix-tiny"
+    assert d["prefill"]["tok_s"] > 0 and d["decode"]["bytes"] > 0
+    assert {"kernel per phase", "automatic"} <= set(d["beside"])

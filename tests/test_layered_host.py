@@ -132,3 +132,18 @@ def test_ctypes_structures_match_the_header(pkg, tmp_path):
         want.append(ctypes.sizeof(cls))
         want += [getattr(cls, name).offset for name, _ in cls._fields_]
     assert got == want
+
+
+def test_shapes_and_work_of_the_bench_models(pkg):
+    from llama2_jl_amd import bench_layered, layered
+    for c in lc.CASES.values():
+        t = ref.tensor_shapes(c)
+        assert layered.vudelix_shapes(layered.vudelix_config(c, lambda n: t[n])) == t
+    cfg, _ = bench_layered.config("vudelix-tiny")
+    by, fl = bench_layered.work(cfg, 64)
+    shapes = layered.vudelix_shapes(cfg)
+    experts = [n for n in shapes if ".mlp.e" in n]
+    mats = sum(np.prod(s) for n, s in shapes.items() if len(s) == 2 and n not in experts + ["embed", "side.embed"] and "conv" not in n)
+    mats += sum(np.prod(shapes[n]) for n in experts) * 2 // 8  # two experts of eight are read
+    state = 6 * 2 * 4 * 4 * 128 * 128 + 2 * 4 * 64 * 2 * 256  # read and written; keys and values of 64 positions
+    assert by == 2 * mats + state and fl > 2 * 64 * (mats - 512 * 32000)

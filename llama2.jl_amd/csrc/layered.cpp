@@ -783,14 +783,14 @@ static GemmArgs gemm_of(const LMat &w, const void *x, int M) {
     return a;
 }
 
-// a plain product (GE_STORE or GE_RESID); large ones go through the library, rounded up to whole groups of 128 positions so
+// a product whose result stays fp32; large plain ones (GE_STORE, GE_RESID) go through the library, rounded up to whole groups of 128 positions so
 // that few different shapes occur: the rows beyond M are computed from whatever the buffers hold, and never read
 static bool library_takes(const l2h_model *m, const GemmArgs &a) {
     return m->lay->c.precision == 0 && m->pf_lt && m->pf_library_mode && a.M >= L_BIG_MIN_M &&
            (double)a.M * (double)a.n_rows * (double)a.ld >= (double)(1 << 26);
 }
 static hipError_t product(l2h_model *m, GemmArgs a, int epi, float *out, int64_t ldo, float mult) {
-    if (library_takes(m, a)) {
+    if ((epi == GE_STORE || epi == GE_RESID) && library_takes(m, a)) {
         const int M = (a.M + 127) / 128 * 128;
         const hipError_t e = pf_lt_gemm(m->pf_lt, m->ctx->stream, a.w, (const uint16_t *)a.x, out, M, a.n_rows, a.ld, ldo, epi == GE_RESID,
                                         &m->pf_lt_err, mult);

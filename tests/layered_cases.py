@@ -67,7 +67,7 @@ CASES = {
                           delta(heads=8, kv_heads=4, dim=64, vdim=64, conv=4, ranks=(32, 32), mlp=moe(16, 4, 96))], width=520, vocab=300,
                          side=64),
     # wide and long enough for the library's products and the tile images
-    "large": config([delta(heads=10, kv_heads=5, dim=64, vdim=64, conv=4, ranks=(40, 72), mlp=moe(6, 2, 200)),
+    "large": config([delta(heads=10, kv_heads=5, dim=64, vdim=64, conv=4, ranks=(400, 390), mlp=moe(6, 2, 200)),
                      attention(heads=10, kv_heads=5, dim=96, vdim=80, size=70, rot=96, mlp=dense(600))], width=576, vocab=520, side=48),
 }
 

@@ -258,8 +258,9 @@ int l2h_argmax_noalloc(l2h_ctx *ctx, const float *x_dev, int64_t n, int32_t *out
  * The calls that concern k-quant weights, the other launch paths, or rows of the Llama KV cache are
  * L2H_EINVAL.
  *
- * With residual stream x and mult = residual_mult, a layer is
+ * The residual stream x starts as embed_scale times the token's embedding row.  With mult = residual_mult, a layer is
  *   x += mult * mixer(norm1(x));  x += mult * ff(norm2(x));
+ *   or, with parallel set,  h = norm1(x);  x += mult * (mixer(h) + ff(h));
  *   with side_dim > 0:  e = the layer's slice of the token's row of the side embedding,
  *     y = side_proj(gelu_tanh(side_gate x) * e);  x += mult * rmsnorm(y) * side_norm
  * Mixers:
@@ -271,13 +272,24 @@ int l2h_argmax_noalloc(l2h_ctx *ctx, const float *x_dev, int64_t n, int32_t *out
  *                  delta rule with beta = sigmoid(beta row . input) per head and a decay per head and key channel,
  *                  exp(-exp(decay rate) softplus(factor_out factor_in input + decay bias)); per-head rmsnorm, times
  *                  sigmoid(gate factors); output projection.
- * Feed-forward: dense act(up) -> down, or the `top` of n_experts experts by sigmoid(router), the score multiplying the
- * expert's input. */
-enum { L2H_MIX_ATTENTION = 0, L2H_MIX_CHANNEL_DELTA = 1 };
+ *   LATENT         causal attention with keys and values made from a latent per position (n_kv_heads = n_heads).  Queries:
+ *                  q_up (rmsnorm(q_down input) * q_norm), head by head [dim | rot_size]; kv_down input = [kv_rank | rot_size]:
+ *                  the latent c = rmsnorm(first part) * kv_norm, and one rotated key part that all heads share.  Per head
+ *                  key = [k_up c | rotated part], value = v_up c of vdim.  The cache holds c and the rotated part.  The
+ *                  rotation takes the first rot_dims of the rot_size dimensions; out_gate: the heads' outputs times
+ *                  sigmoid(out_gate input), element by element; output projection.
+ * Rotation pairs dimensions 2i and 2i+1, or, with rot_half set, i and i + rot_dims / 2.
+ * Feed-forward: dense act(up) -> down, or the `top` of n_experts experts with the largest router row . input (+ router bias);
+ * with ff_gated, act(gate) * up -> down.  route: L2H_ROUTE_SIGMOID_IN, the expert's input is multiplied by the sigmoid of its
+ * logit; L2H_ROUTE_SOFTMAX_OUT, its output by the softmax over the chosen logits.
+ * Loop (loop_times > 0): layers loop_start .. loop_stop - 1 run loop_times times in a row, each pass with caches of its own.
+ * Before pass t, x += (t > 0 ? the starting x : 0) + row t of the loop step. */
+enum { L2H_MIX_ATTENTION = 0, L2H_MIX_CHANNEL_DELTA = 1, L2H_MIX_LATENT = 2 };
 enum { L2H_FF_NONE = 0, L2H_FF_DENSE = 1, L2H_FF_EXPERTS = 2 };
-enum { L2H_ACT_GELU_ERF = 0, L2H_ACT_RELU2 = 1, L2H_ACT_GELU_TANH = 2 };
-/* Roles shared with Llama models: TOK_EMB, RMS_FINAL, OUTPUT, RMS_ATT (norm1), RMS_FFN (norm2), WQ, WK, WV, WO, W1 (up),
- * W2 (down).  Matrices are bf16 of any size; vectors bf16 or F32 (convolutions: ne0 = taps, ne1 = channels). */
+enum { L2H_ACT_GELU_ERF = 0, L2H_ACT_RELU2 = 1, L2H_ACT_GELU_TANH = 2, L2H_ACT_RELU = 3, L2H_ACT_SILU = 4 };
+enum { L2H_ROUTE_SIGMOID_IN = 0, L2H_ROUTE_SOFTMAX_OUT = 1 };
+/* Roles shared with Llama models: TOK_EMB, RMS_FINAL, OUTPUT, RMS_ATT (norm1), RMS_FFN (norm2), WQ, WK, WV, WO, W1 (up, or
+ * with ff_gated the gate), W2 (down), W3 (with ff_gated: up).  Matrices are bf16 of any size; vectors bf16 or F32 (convolutions: ne0 = taps, ne1 = channels). */
 enum {
     L2H_HEAD_GATE = 12,  /* (width, heads)                  */
     L2H_BETA = 13,       /* (width, heads)                  */
@@ -295,28 +307,42 @@ enum {
     L2H_SIDE_GATE = 28,  /* (width, side_dim)               */
     L2H_SIDE_PROJ = 29,  /* (side_dim, width)               */
     L2H_SIDE_NORM = 30,  /* (width)                         */
-    L2H_N_LAYERED_ROLES = 31
+    L2H_Q_DOWN = 31,     /* (width, q_rank)                 */
+    L2H_Q_NORM = 32,     /* (q_rank)                        */
+    L2H_Q_UP = 33,       /* (q_rank, heads * (dim + rot_size)) */
+    L2H_KV_DOWN = 34,    /* (width, kv_rank + rot_size)     */
+    L2H_KV_NORM = 35,    /* (kv_rank)                       */
+    L2H_K_UP = 36,       /* (kv_rank, heads * dim)          */
+    L2H_V_UP = 37,       /* (kv_rank, heads * vdim)         */
+    L2H_OUT_GATE = 38,   /* (width, heads * vdim)           */
+    L2H_ROUTER_BIAS = 39, /* (n_experts)                    */
+    L2H_EXPERT_GATE = 40, /* through l2h_layered_set_expert */
+    L2H_LOOP_STEP = 41,  /* (width, loop_times)             */
+    L2H_N_LAYERED_ROLES = 42
 };
 typedef struct l2h_layer {
     int32_t mixer, n_heads, n_kv_heads, dim, vdim;
     int32_t window, rot_dims, qk_norm, head_gate;   /* attention */
     int32_t taps, decay_rank, gate_rank;            /* channel delta */
-    int32_t ff, ff_dim, ff_act, n_experts, top;
-    float scale;                                    /* attention */
+    int32_t q_rank, kv_rank, rot_size, out_gate;    /* latent attention */
+    int32_t rot_half, parallel;
+    int32_t ff, ff_dim, ff_act, ff_gated, n_experts, top, route, router_bias;
+    float scale;                                    /* attention, latent attention */
     double rot_base, rot_factor, rot_low, rot_high, rot_original;
 } l2h_layer;
 typedef struct l2h_layered_config {
     int32_t width, vocab_size, n_layers, seq_len, side_dim;
     int32_t precision; /* prompt pass: 0 bf16 activations, fp32 sums; 1 fp32 throughout.  Decode steps, caches, state and
                           everything between the products are fp32 either way. */
-    float norm_eps, residual_mult;
+    int32_t loop_start, loop_stop, loop_times;
+    float norm_eps, residual_mult, embed_scale;
 } l2h_layered_config;
 int l2h_layered_create(l2h_ctx *ctx, const l2h_layered_config *cfg, const l2h_layer *layers, l2h_model **out);
-/* one expert's matrix: role L2H_EXPERT_UP (width, ff_dim) or L2H_EXPERT_DOWN (ff_dim, width) */
+/* one expert's matrix: role L2H_EXPERT_UP or L2H_EXPERT_GATE (width, ff_dim), or L2H_EXPERT_DOWN (ff_dim, width) */
 int l2h_layered_set_expert(l2h_model *m, int role, int layer, int expert, int type, const void *host, int64_t ne0,
                            int64_t ne1);
-/* For checks: with on = 1, prompt passes keep the residual stream after every layer; l2h_layered_kept copies that of one
- * layer for the last chunk of up to 2048 positions, n = positions * width floats. */
+/* For checks: with on = 1, prompt passes keep the residual stream after every layer run (a looped layer counts each time);
+ * l2h_layered_kept copies that of one run for the last chunk of up to 2048 positions, n = positions * width floats. */
 int l2h_layered_keep(l2h_model *m, int on);
 int l2h_layered_kept(l2h_model *m, int layer, float *host, int64_t n);
 

@@ -16,7 +16,8 @@ TYPE_F32, TYPE_Q4_K, TYPE_Q5_K, TYPE_Q6_K, TYPE_BF16 = 0, 12, 13, 14, 30
 (TOK_EMB, RMS_FINAL, OUTPUT, RMS_ATT, RMS_FFN, WQ, WK, WV, WO, W1, W2, W3) = range(12)
 N_ROLES = 12
 (HEAD_GATE, BETA, DECAY_RATE, DECAY_BIAS, DECAY_IN, DECAY_OUT, GATE_IN, GATE_OUT, MIX_NORM, CONV_Q, CONV_K, CONV_V, ROUTER,
- EXPERT_UP, EXPERT_DOWN, SIDE_EMB, SIDE_GATE, SIDE_PROJ, SIDE_NORM) = range(12, 31)  # layered models
+ EXPERT_UP, EXPERT_DOWN, SIDE_EMB, SIDE_GATE, SIDE_PROJ, SIDE_NORM, Q_DOWN, Q_NORM, Q_UP, KV_DOWN, KV_NORM, K_UP, V_UP, OUT_GATE,
+ ROUTER_BIAS, EXPERT_GATE, LOOP_STEP) = range(12, 42)  # layered models
 
 
 class L2HError(RuntimeError):

@@ -21,7 +21,7 @@ LIB = os.path.join(HERE, "libl2hip.so")
 LIB_TIMELINE = os.path.join(HERE, "libl2hip_tl.so")
 
 SOURCES = ["api.cpp", "synth.cpp", "pf_lt.cpp", "k_misc.hip", "k_matvec.hip", "k_attn.hip", "k_mega.hip", "k_prefill.hip", "k_flow.hip",
-           "layered.cpp", "k_rows.hip", "k_delta.hip", "k_window.hip", "k_gemm.hip", "k_tiles.hip"]
+           "layered.cpp", "k_rows.hip", "k_delta.hip", "k_window.hip", "k_latent.hip", "k_gemm.hip", "k_tiles.hip"]
 
 COMMON = [
     "-O3", "-fPIC", "-std=c++17", "-ffp-contract=off", "-Wall", "-Wno-unused-function",

@@ -310,7 +310,7 @@ extern "C" int l2h_model_set_tensor(l2h_model *m, int role, int layer, int type,
 extern "C" int l2h_layered_set_expert(l2h_model *m, int role, int layer, int expert, int type, const void *host, int64_t ne0,
                                       int64_t ne1) {
     if (!m || !host) return set_err(m ? m->ctx : nullptr, L2H_EINVAL, "l2h_layered_set_expert: NULL argument");
-    if (!m->lay || (role != L2H_EXPERT_UP && role != L2H_EXPERT_DOWN))
+    if (!m->lay || (role != L2H_EXPERT_UP && role != L2H_EXPERT_GATE && role != L2H_EXPERT_DOWN))
         return set_err(m->ctx, L2H_EINVAL, "l2h_layered_set_expert takes an expert matrix of a layered model");
     return layered_set_tensor(m, role, layer, expert, type, host, ne0, ne1);
 }

@@ -163,10 +163,10 @@ template <int PREC, int EPI>
 static hipError_t gemm_launch(hipStream_t s, const GemmArgs &a) {
     // columns the epilogue covers: an activation-typed result is zeroed up to its row stride
     const bool acts = EPI == GE_ACT || EPI == GE_UP || EPI == GE_EMBED;
-    const int64_t cols = acts ? a.lda : a.n_rows;
+    const int64_t cols = EPI == GE_GLU ? 2 * a.acols : acts ? a.acols : a.n_rows;
     if (a.tiles) {
-        if (EPI != GE_STORE && EPI != GE_UP) return hipErrorInvalidValue;
-        constexpr int E = EPI == GE_UP ? GE_UP : GE_STORE;
+        if (EPI != GE_STORE && EPI != GE_UP && EPI != GE_GLU) return hipErrorInvalidValue;
+        constexpr int E = EPI == GE_UP || EPI == GE_GLU ? EPI : GE_STORE;
         if (cols > 64) {
             hipLaunchKernelGGL((gemm_kernel<PREC, E, 128, L_GEMM_TILE, true>), dim3((unsigned)a.max_tiles, (unsigned)((cols + 127) / 128)),
                                dim3(256), 0, s, a);
@@ -186,10 +186,17 @@ static hipError_t gemm_launch(hipStream_t s, const GemmArgs &a) {
     return hipGetLastError();
 }
 
-hipError_t k_gemm(hipStream_t s, const GemmArgs &a, int prec, int epi) {
-    if (!a.w || !a.x || a.n_rows < 1 || a.M < 1 || a.ld % 64 != 0 || a.ldx < a.ld || a.lda % 64 != 0) return hipErrorInvalidValue;
+hipError_t k_gemm(hipStream_t s, const GemmArgs &args, int prec, int epi) {
+    GemmArgs a = args;
+    if (!a.acols) a.acols = a.lda;
+    if (!a.w || !a.x || a.n_rows < 1 || a.M < 1 || a.ld % 64 != 0 || a.ldx < a.ld || a.lda % 64 != 0 || a.acols % 64 != 0 ||
+        a.acols > a.lda)
+        return hipErrorInvalidValue;
     const bool acts = epi == GE_ACT || epi == GE_UP || epi == GE_EMBED;
-    if (acts ? (!a.outa || a.lda < a.n_rows) : (!a.outf || a.ldo < a.n_rows)) return hipErrorInvalidValue;
+    if (epi == GE_GLU ? (!a.outa || a.n_rows % 2 != 0 || 2 * a.acols < a.n_rows)
+        : acts        ? (!a.outa || a.acols < a.n_rows)
+                      : (!a.outf || a.ldo < a.n_rows))
+        return hipErrorInvalidValue;
 #define GO(E) \
     case E: return prec ? gemm_launch<1, E>(s, a) : gemm_launch<0, E>(s, a)
     switch (epi) {
@@ -200,6 +207,7 @@ hipError_t k_gemm(hipStream_t s, const GemmArgs &a, int prec, int epi) {
         GO(GE_EMBED);
         GO(GE_DECAY);
         GO(GE_SIGMOID);
+        GO(GE_GLU);
     }
 #undef GO
     return hipErrorInvalidValue;
@@ -322,29 +330,23 @@ hipError_t k_norm_rows(hipStream_t s, float *x, int K, int M, const float *w, fl
 // ---------------------------------------------------------------------------------------------------------------
 // mixture of experts
 // ---------------------------------------------------------------------------------------------------------------
-// one workgroup per token: an expert's place is the number of experts with a larger logit (the lower index first among equals)
-__global__ __launch_bounds__(64) void route_kernel(const float *z, int E, int top, int32_t *choice, float *score) {
+// one workgroup per token
+__global__ __launch_bounds__(64) void route_kernel(const float *z, int64_t ldz, const float *bias, int E, int top, int kind, int32_t *choice,
+                                                   float *score) {
     extern __shared__ __align__(16) float s_mem[];
+    __shared__ int s_sel[64];
+    __shared__ float s_score[64];
     const int64_t m = blockIdx.x;
-    for (int e = threadIdx.x; e < E; e += 64) s_mem[e] = z[m * E + e];
-    for (int k = threadIdx.x; k < top; k += 64) {  // (a place that no number takes, with NaN among them, stays defined)
-        choice[m * top + k] = 0;
-        score[m * top + k] = 0.0f;
-    }
-    __syncthreads();
-    for (int e = threadIdx.x; e < E; e += 64) {
-        const float v = s_mem[e];
-        int rank = 0;
-        for (int o = 0; o < E; o++) rank += (s_mem[o] > v || (s_mem[o] == v && o < e)) ? 1 : 0;
-        if (rank < top) {
-            choice[m * top + rank] = e;
-            score[m * top + rank] = l_sigmoid(v);
-        }
+    l_route(z + m * ldz, bias, E, top, kind, s_mem, s_sel, s_score);
+    for (int k = threadIdx.x; k < top; k += 64) {
+        choice[m * top + k] = s_sel[k];
+        score[m * top + k] = s_score[k];
     }
 }
-hipError_t k_route(hipStream_t s, const float *z, int M, int E, int top, int32_t *choice, float *score) {
-    if (E < 1 || top < 1 || top > E) return hipErrorInvalidValue;
-    hipLaunchKernelGGL(route_kernel, dim3((unsigned)M), dim3(64), E * sizeof(float), s, z, E, top, choice, score);
+hipError_t k_route(hipStream_t s, const float *z, int64_t ldz, const float *bias, int M, int E, int top, int kind, int32_t *choice,
+                   float *score) {
+    if (E < 1 || top < 1 || top > E || top > 64) return hipErrorInvalidValue;
+    hipLaunchKernelGGL(route_kernel, dim3((unsigned)M), dim3(64), E * sizeof(float), s, z, ldz, bias, E, top, kind, choice, score);
     return hipGetLastError();
 }
 
@@ -409,6 +411,17 @@ __global__ __launch_bounds__(256) void gather_add_kernel(float *x, const float *
 }
 hipError_t k_gather_add(hipStream_t s, float *x, const float *y, const int32_t *slot_of, int M, int top, int K, float mult) {
     hipLaunchKernelGGL(gather_add_kernel, dim3((unsigned)((K + 1023) / 1024), (unsigned)M), dim3(256), 0, s, x, y, slot_of, top, K, mult);
+    return hipGetLastError();
+}
+
+__global__ __launch_bounds__(256) void stream_add_kernel(float *x, const float *a, const float *b, int K) {
+    const int i = blockIdx.x * 256 + threadIdx.x;
+    if (i >= K) return;
+    const int64_t at = (int64_t)blockIdx.y * K + i;
+    x[at] = (a ? x[at] + a[at] : x[at]) + b[i];
+}
+hipError_t k_stream_add(hipStream_t s, float *x, const float *a, const float *b, int M, int K) {
+    hipLaunchKernelGGL(stream_add_kernel, dim3((unsigned)((K + 255) / 256), (unsigned)M), dim3(256), 0, s, x, a, b, K);
     return hipGetLastError();
 }
 

@@ -76,7 +76,8 @@ hipError_t k_repack(hipStream_t s, const DevTensor &t, const void *raw_dev, bool
 // (src/inference.jl:354-360,385).
 // ------------------------------------------------------------------------------------------
 __global__ __launch_bounds__(256) void embed_kernel(DevTensor emb, const DecodeCtl *ctl, const int32_t *prompt,
-                                                    float *x, float *rope_cs, int hs, float theta_scale) {
+                                                    float *x, float *rope_cs, int hs, float theta_scale,
+                                                    float scale, float *x_copy) {
     const int i = blockIdx.x * blockDim.x + threadIdx.x;
     if (blockIdx.x == 0 && threadIdx.x < (hs >> 1)) {
         // cos/sin of this position's RoPE angles, shared by all layers and heads: theta_i is
@@ -88,13 +89,15 @@ __global__ __launch_bounds__(256) void embed_kernel(DevTensor emb, const DecodeC
     }
     if (i >= emb.ne0) return;
     const int tok = ctl->step < ctl->n_prompt ? prompt[ctl->step] : ctl->last_argmax;
-    x[i] = dequant_elem(emb, tok, i);
+    const float v = scale * dequant_elem(emb, tok, i);
+    x[i] = v;
+    if (x_copy) x_copy[i] = v;
 }
 
 hipError_t k_embed(hipStream_t s, const DevTensor &emb, const DecodeCtl *ctl, const int32_t *prompt, float *x,
-                   float *rope_cs, int head_size, float theta_scale) {
+                   float *rope_cs, int head_size, float theta_scale, float scale, float *x_copy) {
     hipLaunchKernelGGL(embed_kernel, dim3((unsigned)((emb.ne0 + 255) / 256)), dim3(256), 0, s, emb, ctl, prompt, x,
-                       rope_cs, head_size, theta_scale);
+                       rope_cs, head_size, theta_scale, scale, x_copy);
     return hipGetLastError();
 }
 

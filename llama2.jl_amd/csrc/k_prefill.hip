@@ -13,11 +13,13 @@
 // small per-position kernels
 // ------------------------------------------------------------------------------------------
 // X[m][:] = dequantized embedding row of tokens[m]  (src/inference.jl:236)
-__global__ __launch_bounds__(256) void pf_embed_kernel(DevTensor emb, const int32_t *tokens, float *X, int M) {
+__global__ __launch_bounds__(256) void pf_embed_kernel(DevTensor emb, const int32_t *tokens, float *X, int M, float scale, float *X_copy) {
     const int m = blockIdx.y;
     const int i = blockIdx.x * blockDim.x + threadIdx.x;
     if (m >= M || i >= emb.ne0) return;
-    X[(int64_t)m * emb.ne0 + i] = dequant_elem(emb, tokens[m], i);
+    const float v = scale * dequant_elem(emb, tokens[m], i);
+    X[(int64_t)m * emb.ne0 + i] = v;
+    if (X_copy) X_copy[(int64_t)m * emb.ne0 + i] = v;
 }
 
 // cos/sin of the RoPE angles of positions pos0..pos0+M-1: theta_i = fp32(pos) advanced by i fp32
@@ -536,11 +538,13 @@ __global__ __launch_bounds__(512) void pf_gemm_bf16_mixed_kernel(PfGemmArgs a, u
 // padding per row to spread the banks) followed by V^T (head-dim-major, keys permuted, padded rows).  The 64
 // workgroups that need a tile (4 heads of the group x 16 query blocks) then only copy it.
 // ------------------------------------------------------------------------------------------
+// HS: size of a key, and of a value up to 128
 template <int HS>
 struct PfKvTile {
+    static constexpr int VS = HS <= 128 ? HS : 128;
     static constexpr int KROW = HS * 2 + 16;  // bytes per key row
     static constexpr int VROW = 80;           // bytes per head-dim row of V^T: 32 keys + 16 bytes of padding
-    static constexpr int K_BYTES = 32 * KROW, V_BYTES = HS * VROW;
+    static constexpr int K_BYTES = 32 * KROW, V_BYTES = VS * VROW;
     static constexpr int BYTES = (K_BYTES + V_BYTES + 1023) / 1024 * 1024;  // copied 1 KB at a time
 };
 
@@ -587,6 +591,54 @@ __global__ __launch_bounds__(256) void pf_kv_tiles_kernel(const float *kc, const
     }
     __syncthreads();
     uint4 *dst = (uint4 *)(tiles + ((int64_t)kvh * n_tiles_max + kt) * T::BYTES);
+    for (int c = t; c < T::BYTES / 16; c += 256) dst[c] = ((const uint4 *)s_img)[c];
+}
+
+// The same tiles from rows of projected keys and values (k_pf_row_tiles): a workgroup makes the tile of one head and 32
+// positions, a key being its head's kd elements, then the `tail` elements that all heads share.
+template <int HS>
+__global__ __launch_bounds__(256) void pf_row_tiles_kernel(const float *kv, int64_t ldkv, const float *tails, int64_t ldt, int tail,
+                                                           unsigned char *tiles, int pos0, int n, int n_tiles_max, int kd, int vd) {
+    typedef PfKvTile<HS> T;
+    __shared__ __align__(16) unsigned char s_img[T::BYTES];
+    unsigned char *s_k = s_img, *s_v = s_img + T::K_BYTES;
+    const int t = threadIdx.x, h = blockIdx.x, H = gridDim.x, r0 = 32 * blockIdx.y;
+    for (int c = t; c < T::BYTES / 16; c += 256) ((uint4 *)s_img)[c] = make_uint4(0, 0, 0, 0);
+    __syncthreads();
+    const bool quads = kd % 4 == 0 && vd % 4 == 0 && ldkv % 4 == 0 && tail % 4 == 0 && ldt % 4 == 0;
+    for (int idx = t; idx < 32 * (HS / 4); idx += 256) {
+        const int key = idx / (HS / 4), e = 4 * (idx % (HS / 4)), r = r0 + key;
+        if (r >= n || e >= kd + tail) continue;
+        const float *k = kv + (int64_t)r * ldkv + (int64_t)h * kd, *tl = tails + (int64_t)(pos0 + r) * ldt;
+        float v[4];
+        if (quads) {
+            const float4 q = e < kd ? *(const float4 *)(k + e) : *(const float4 *)(tl + e - kd);
+            v[0] = q.x, v[1] = q.y, v[2] = q.z, v[3] = q.w;
+        } else {
+#pragma unroll
+            for (int b = 0; b < 4; b++) v[b] = e + b < kd ? k[e + b] : e + b < kd + tail ? tl[e + b - kd] : 0.0f;
+        }
+        *(uint2 *)(s_k + key * T::KROW + e * 2) = make_uint2(pack_bf16(v[0], v[1]), pack_bf16(v[2], v[3]));
+    }
+    for (int idx = t; idx < 32 * (T::VS / 4); idx += 256) {
+        const int key = idx / (T::VS / 4), e = 4 * (idx % (T::VS / 4)), r = r0 + key;
+        if (r >= n || e >= vd) continue;
+        const float *src = kv + (int64_t)r * ldkv + (int64_t)H * kd + (int64_t)h * vd + e;
+        float v[4];
+        if (quads) {
+            const float4 q = *(const float4 *)src;
+            v[0] = q.x, v[1] = q.y, v[2] = q.z, v[3] = q.w;
+        } else {
+#pragma unroll
+            for (int b = 0; b < 4; b++) v[b] = e + b < vd ? src[b] : 0.0f;
+        }
+        const int rem = key & 15, slot = (key & 16) + 8 * ((rem >> 2) & 1) + 4 * (rem >> 3) + (rem & 3);
+        __bf16 *dst = (__bf16 *)(s_v + e * T::VROW) + slot;
+#pragma unroll
+        for (int b = 0; b < 4; b++) dst[b * (T::VROW / 2)] = (__bf16)v[b];
+    }
+    __syncthreads();
+    uint4 *dst = (uint4 *)(tiles + ((int64_t)h * n_tiles_max + (pos0 + r0) / 32) * T::BYTES);
     for (int c = t; c < T::BYTES / 16; c += 256) dst[c] = ((const uint4 *)s_img)[c];
 }
 
@@ -637,14 +689,15 @@ __device__ __forceinline__ float pf_other_half(float x) {
 }
 
 // WIN: position i sees the keys i - window + 1 .. i only; the tiles start with tile `tile0` of the sequence (32 keys each); the
-// scale of the scores, the value size (<= HS), a gate per head (sigmoid of gate[m * ldg + h]) and the output's row stride, whose
-// columns beyond the heads are zeroed, are the caller's.
+// scale of the scores, the value size (<= HS and 128), a gate per head (sigmoid of gate[m * ldg + h]) or per element
+// (gate[m * ldg + h vdim + e]) and the output's row stride, whose columns beyond the heads are zeroed, are the caller's.
 template <int HS, bool WIN>
 __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void pf_attn_kernel(const uint16_t *Qb, uint16_t *Att, const unsigned char *tiles,
                                                       int n_tiles_max, int M, int qpos0, int n_heads, int n_kv, int dim,
                                                       unsigned n_qb, unsigned n_items, unsigned per, PfWindow win) {
     typedef PfKvTile<HS> T;
-    constexpr int KSTEPS = HS / 16, DT = HS / 32, KH = KSTEPS / 2;
+    constexpr int KSTEPS = HS / 16, DT = T::VS / 32, NG = HS <= 128 ? 2 : (KSTEPS + 3) / 4, KH = KSTEPS / NG;
+    static_assert(KH * NG == KSTEPS && KH <= 4, "");
     // two stages: the copy of tile kt + 1 is in flight during the products of tile kt, one barrier per tile
     __shared__ __align__(16) unsigned char s_t[2 * T::BYTES];
     const int t = threadIdx.x, lane = t & 63, wave = __builtin_amdgcn_readfirstlane(t >> 6), g = lane >> 5, ql = lane & 31;
@@ -704,13 +757,13 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void p
 #pragma unroll
         for (int r = 0; r < 16; r++) s[r] = 0.0f;
         {
-            pf_u32x4 ka[2][4];
-            pf_lds_issue<KH, 32>(ka[0], k_addr + so);
-            pf_lds_issue<KH, 32>(ka[1], k_addr + so + (unsigned)(32 * KH));
-            pf_lds_retire<KH>(ka[0]);
-            pf_lds_retire<KH>(ka[1]);
+            pf_u32x4 ka[NG][4];
 #pragma unroll
-            for (int half = 0; half < 2; half++)
+            for (int part = 0; part < NG; part++) pf_lds_issue<KH, 32>(ka[part], k_addr + so + (unsigned)(32 * KH * part));
+#pragma unroll
+            for (int part = 0; part < NG; part++) pf_lds_retire<KH>(ka[part]);
+#pragma unroll
+            for (int half = 0; half < NG; half++)
 #pragma unroll
                 for (int i = 0; i < KH; i++)
                     s = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8, ka[half][i]), qf[KH * half + i], s, 0, 0, 0);
@@ -783,7 +836,19 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void p
     if (!qvalid) return;
     if constexpr (WIN) {
         float f = 1.0f / lrun;
-        if (win.gate) f /= 1.0f + expf(-win.gate[(int64_t)myq * win.ldg + h]);
+        if (win.gate && !win.gate_each) f /= 1.0f + expf(-win.gate[(int64_t)myq * win.ldg + h]);
+        if (win.gate && win.gate_each) {
+            const float *gl = win.gate + (int64_t)myq * win.ldg + (int64_t)h * win.vdim;
+#pragma unroll
+            for (int d = 0; d < DT; d++)
+#pragma unroll
+                for (int rq = 0; rq < 4; rq++) {
+                    const int e = 32 * d + 8 * rq + 4 * g;
+#pragma unroll
+                    for (int b = 0; b < 4; b++)
+                        if (e + b < win.vdim) o[d][4 * rq + b] /= 1.0f + expf(-gl[e + b]);
+                }
+        }
         __bf16 *row = (__bf16 *)Att + (int64_t)myq * win.ldo + (int64_t)h * win.vdim;
 #pragma unroll
         for (int d = 0; d < DT; d++)
@@ -801,7 +866,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void p
                 }
             }
         if (h == n_heads - 1 && g == 0)
-            for (int64_t i = (int64_t)n_heads * win.vdim; i < win.ldo; i++) ((__bf16 *)Att)[(int64_t)myq * win.ldo + i] = (__bf16)0.0f;
+            for (int64_t i = (int64_t)n_heads * win.vdim; i < win.cols; i++) ((__bf16 *)Att)[(int64_t)myq * win.ldo + i] = (__bf16)0.0f;
         return;
     }
     const float inv = 1.0f / lrun;
@@ -820,9 +885,9 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void p
 // ------------------------------------------------------------------------------------------
 // launchers
 // ------------------------------------------------------------------------------------------
-hipError_t k_pf_embed(hipStream_t s, const DevTensor &emb, const int32_t *tokens, float *X, int M) {
+hipError_t k_pf_embed(hipStream_t s, const DevTensor &emb, const int32_t *tokens, float *X, int M, float scale, float *X_copy) {
     hipLaunchKernelGGL(pf_embed_kernel, dim3((unsigned)((emb.ne0 + 255) / 256), (unsigned)M), dim3(256), 0, s, emb,
-                       tokens, X, M);
+                       tokens, X, M, scale, X_copy);
     return hipGetLastError();
 }
 hipError_t k_pf_rope_table(hipStream_t s, float *cs, int pos0, int M, int half, float theta_scale) {
@@ -1020,6 +1085,7 @@ int64_t k_pf_kv_tile_bytes(int hs) {
     case 64: return PfKvTile<64>::BYTES;
     case 96: return PfKvTile<96>::BYTES;
     case 128: return PfKvTile<128>::BYTES;
+    case 192: return PfKvTile<192>::BYTES;
     }
     return 0;
 }
@@ -1044,12 +1110,33 @@ hipError_t k_pf_kv_tiles(hipStream_t s, const float *kc, const float *vc, unsign
     return hipGetLastError();
 }
 
-// tiles must hold the keys 0 .. qpos0 + M - 1 (k_pf_kv_tiles)
+hipError_t k_pf_row_tiles(hipStream_t s, const float *kv, int64_t ldkv, const float *tails, int64_t ldt, int tail, unsigned char *tiles,
+                          int pos0, int n, int n_tiles_max, int hs, int n_heads, int kdim, int vdim) {
+    if (n < 1 || pos0 < 0 || pos0 % 32 != 0 || (pos0 + n + 31) / 32 > n_tiles_max || kdim + tail > hs || vdim > std::min(hs, 128) ||
+        ldkv < (int64_t)n_heads * (kdim + vdim) || ldt < tail)
+        return hipErrorInvalidValue;
+    const dim3 grid((unsigned)n_heads, (unsigned)((n + 31) / 32));
+#define GO(HS) \
+    hipLaunchKernelGGL((pf_row_tiles_kernel<HS>), grid, dim3(256), 0, s, kv, ldkv, tails, ldt, tail, tiles, pos0, n, n_tiles_max, kdim, vdim)
+    switch (hs) {
+    case 32: GO(32); break;
+    case 64: GO(64); break;
+    case 96: GO(96); break;
+    case 128: GO(128); break;
+    case 192: GO(192); break;
+    default: return hipErrorInvalidValue;
+    }
+#undef GO
+    return hipGetLastError();
+}
+
+// tiles must hold the keys 0 .. qpos0 + M - 1 (k_pf_kv_tiles); a key size of 192 has the windowed form only
 hipError_t k_pf_attention(hipStream_t s, const uint16_t *Qb, uint16_t *Att, const unsigned char *tiles, int n_tiles_max,
                           int M, int qpos0, int hs, int n_heads, int n_kv, int dim, const PfWindow *win) {
-    const PfWindow w = win ? *win : PfWindow{};
+    PfWindow w = win ? *win : PfWindow{};
+    if (!w.cols) w.cols = w.ldo;
     if ((qpos0 + M + 31) / 32 - w.tile0 > n_tiles_max) return hipErrorInvalidValue;
-    if (win && (w.window < 1 || w.vdim > hs || w.ldo < (int64_t)n_heads * w.vdim || w.ldo % 4 != 0 ||
+    if (win && (w.window < 1 || w.vdim > std::min(hs, 128) || w.cols > w.ldo || w.cols < (int64_t)n_heads * w.vdim || w.ldo < (int64_t)n_heads * w.vdim || w.ldo % 4 != 0 ||
                 32 * w.tile0 > std::max(0, qpos0 - w.window + 1)))
         return hipErrorInvalidValue;
     const unsigned n_qb = (unsigned)((M + 127) / 128), n_items = n_qb * (unsigned)n_heads, per = (n_items + 7) / 8;
@@ -1068,6 +1155,11 @@ hipError_t k_pf_attention(hipStream_t s, const uint16_t *Qb, uint16_t *Att, cons
     case 64: GO(64); break;
     case 96: GO(96); break;
     case 128: GO(128); break;
+    case 192:
+        if (!win) return hipErrorInvalidValue;
+        hipLaunchKernelGGL((pf_attn_kernel<192, true>), grid, dim3(256), 0, s, Qb, Att, tiles, n_tiles_max, M, qpos0, n_heads, n_kv, dim,
+                           n_qb, n_items, per, w);
+        break;
     default: return hipErrorInvalidValue;
     }
 #undef GO

@@ -94,22 +94,7 @@ __global__ __launch_bounds__(ROWS_THREADS) void rows_kernel(RowsArgs a, int rows
     }
 
     if (PRO == RP_UP || PRO == RP_DOWN) {
-        // an expert's place among all by score: the number of larger ones (the lower index first among equals)
-        float *zs = s_mem + (int64_t)nvec * 2 * plane;
-        for (int e = t; e < a.n_experts; e += ROWS_THREADS) zs[e] = a.z[e];
-        if (t < a.top) s_sel[t] = 0, s_score[t] = 0.0f;  // (a place that no number takes, with NaN among them, stays defined)
-        __syncthreads();
-        for (int e = t; e < a.n_experts; e += ROWS_THREADS) {
-            const float z = zs[e];
-            int rank = 0;
-#pragma unroll 8
-            for (int o = 0; o < a.n_experts; o++) rank += (zs[o] > z || (zs[o] == z && o < e)) ? 1 : 0;
-            if (rank < a.top) {
-                s_sel[rank] = e;
-                s_score[rank] = l_sigmoid(z);
-            }
-        }
-        __syncthreads();
+        l_route(a.z, a.z_bias, a.n_experts, a.top, a.route, s_mem + (int64_t)nvec * 2 * plane, s_sel, s_score);
         if (r0 < row_end) {
             row_ptrs(r0, 0, w0, w1);
             fetch(cur, kstart);
@@ -294,13 +279,26 @@ __global__ __launch_bounds__(ROWS_THREADS) void rows_kernel(RowsArgs a, int rows
                     acc1 += s_part[i][1];
                 }
             }
-            if ((!KSPLIT || wave == 0) && lane < (two ? 2 : 1)) {
+            if (EPI == RE_GLU || (EPI == RE_STORE_GLU && r0 >= a.glu_from)) {  // (whole pairs)
+                if ((!KSPLIT || wave == 0) && lane == 0) {
+                    float s_in = 1.0f, s_out = 1.0f;
+                    if (PRO == RP_UP) (a.route == LROUTE_SIGMOID_IN ? s_in : s_out) = s_score[(unsigned)r0 / (unsigned)a.rows_each];
+                    const float o = s_out * l_act(a.act, s_in * acc0) * (s_in * acc1);
+                    if (EPI == RE_GLU)
+                        a.out[r0 >> 1] = o;
+                    else
+                        a.out2[(r0 - a.glu_from) >> 1] = o;
+                }
+            } else if ((!KSPLIT || wave == 0) && lane < (two ? 2 : 1)) {
                 const int64_t r = r0 + lane;
                 const float val = lane ? acc1 : acc0;
                 float o = val;
                 if (EPI == RE_RESID) o = a.resid[r] + a.mult * val;
                 if (EPI == RE_ACT) o = l_act(a.act, val);
-                if (EPI == RE_UP) o = l_act(a.act, s_score[(unsigned)r / (unsigned)a.rows_each] * val);
+                if (EPI == RE_UP) {
+                    const float f = s_score[(unsigned)r / (unsigned)a.rows_each];
+                    o = a.route == LROUTE_SIGMOID_IN ? l_act(a.act, f * val) : f * l_act(a.act, val);
+                }
                 if (EPI == RE_EMBED) o = l_act(a.act, val) * l_bf16(a.emb[(int64_t)l_step_token(a.ctl, a.prompt) * a.emb_ld + r]);
                 a.out[r] = o;
             }
@@ -355,6 +353,8 @@ hipError_t k_rows(hipStream_t s, const RowsArgs &a, int pro, int epi, int n_cu) 
     if ((pro == RP_UP || pro == RP_DOWN) &&
         (!a.z || a.n_experts < 1 || a.n_experts > ROWS_MAX_EXPERTS || a.top < 1 || a.top > ROWS_MAX_TOP || a.top > a.n_experts))
         return hipErrorInvalidValue;
+    if ((epi == RE_GLU && a.n_rows % 2 != 0) || (epi == RE_STORE_GLU && (a.n_rows % 2 != 0 || a.glu_from % 2 != 0 || !a.out2)))
+        return hipErrorInvalidValue;
 #define GO(P, E) \
     if (pro == P && epi == E) return rows_split<P, E>(s, a, n_cu)
     GO(RP_NORM, RE_STORE);
@@ -363,6 +363,9 @@ hipError_t k_rows(hipStream_t s, const RowsArgs &a, int pro, int epi, int n_cu) 
     GO(RP_PLAIN, RE_RESID);
     GO(RP_PLAIN, RE_EMBED);
     GO(RP_UP, RE_UP);
+    GO(RP_NORM, RE_GLU);
+    GO(RP_NORM, RE_STORE_GLU);
+    GO(RP_UP, RE_GLU);
     GO(RP_DOWN, RE_RESID);
     GO(RP_HEADNORM, RE_RESID);
 #undef GO

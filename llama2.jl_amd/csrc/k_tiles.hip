@@ -100,16 +100,25 @@ static hipError_t tiles_launch(hipStream_t s, const GemmArgs &a, unsigned n_nt, 
 }
 
 // a.w: the image; otherwise as k_gemm with bf16 activations (ldx == ld)
-hipError_t k_tiles(hipStream_t s, const GemmArgs &a, int epi) {
-    if (!a.w || !a.x || a.n_rows < 1 || a.M < 1 || a.ld % 64 != 0 || a.ldx != a.ld || a.lda % 64 != 0) return hipErrorInvalidValue;
+hipError_t k_tiles(hipStream_t s, const GemmArgs &args, int epi) {
+    GemmArgs a = args;
+    if (!a.acols) a.acols = a.lda;
+    if (!a.w || !a.x || a.n_rows < 1 || a.M < 1 || a.ld % 64 != 0 || a.ldx != a.ld || a.lda % 64 != 0 || a.acols % 64 != 0 ||
+        a.acols > a.lda)
+        return hipErrorInvalidValue;
     const unsigned n_nt = (unsigned)((a.n_rows + 255) / 256);
+    const bool covered = a.outa && a.acols >= a.n_rows && a.acols <= 256 * (int64_t)n_nt;
+    const bool pairs = a.outa && a.n_rows % 2 == 0 && 2 * a.acols >= a.n_rows && 2 * a.acols <= 256 * (int64_t)n_nt;
     if (a.tiles) {
-        if (epi == GE_UP && a.outa && a.lda >= a.n_rows && a.lda <= 256 * (int64_t)n_nt) return tiles_launch<GE_UP, 4, true>(s, a, n_nt, 0);
+        if (epi == GE_UP && covered) return tiles_launch<GE_UP, 4, true>(s, a, n_nt, 0);
+        if (epi == GE_GLU && pairs) return tiles_launch<GE_GLU, 4, true>(s, a, n_nt, 0);
         if (epi == GE_STORE && a.outf && a.ldo >= a.n_rows) return tiles_launch<GE_STORE, 4, true>(s, a, n_nt, 0);
         return hipErrorInvalidValue;
     }
-    if (epi != GE_ACT || !a.outa || a.lda < a.n_rows || a.lda > 256 * (int64_t)n_nt) return hipErrorInvalidValue;
+    if (!(epi == GE_ACT && covered) && !(epi == GE_GLU && pairs)) return hipErrorInvalidValue;
     const unsigned n_mt4 = (unsigned)((a.M + 255) / 256), n_mt2 = (unsigned)((a.M + 127) / 128);
+    if (epi == GE_GLU)
+        return n_nt * n_mt4 >= 256 ? tiles_launch<GE_GLU, 4, false>(s, a, n_nt, n_mt4) : tiles_launch<GE_GLU, 2, false>(s, a, n_nt, n_mt2);
     if (n_nt * n_mt4 >= 256) return tiles_launch<GE_ACT, 4, false>(s, a, n_nt, n_mt4);
     return tiles_launch<GE_ACT, 2, false>(s, a, n_nt, n_mt2);
 }

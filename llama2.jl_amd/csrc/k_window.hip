@@ -52,7 +52,7 @@ __global__ __launch_bounds__(256) void window_step_kernel(WindowShape w, const f
     if (has_new) {
         if (wave == 3) {
             for (int i = D + lane; i < Dp; i += 64) s_k[i] = 0.0f;
-            l_rotate_norm(in + w.off_k() + g * D, s_k, D, w.rot, freq, pos, w.qk_norm, w.eps, lane);
+            l_rotate_norm(in + w.off_k() + g * D, s_k, D, w.rot, w.rot_half, freq, pos, w.qk_norm, w.eps, lane);
         }
         for (int i = t; i < V; i += 256) vc[((int64_t)g * w.seq_len + pos) * V + i] = v_new[i];
     }
@@ -61,7 +61,7 @@ __global__ __launch_bounds__(256) void window_step_kernel(WindowShape w, const f
         __syncthreads();
         for (int j = wave; j < NH; j += 4) {
             for (int i = (j < nh ? D : 0) + lane; i < Dp; i += 64) s_q[j * Dp + i] = 0.0f;
-            if (j < nh) l_rotate_norm(in + (g * gq + h0 + j) * D, s_q + j * Dp, D, w.rot, freq, pos, w.qk_norm, w.eps, lane);
+            if (j < nh) l_rotate_norm(in + (g * gq + h0 + j) * D, s_q + j * Dp, D, w.rot, w.rot_half, freq, pos, w.qk_norm, w.eps, lane);
         }
         __syncthreads();
         if (has_new && h0 == 0)
@@ -220,7 +220,7 @@ __global__ __launch_bounds__(256) void window_prepare_kernel(WindowShape w, cons
     const float *r = raw + (int64_t)m * ldr;
     const bool isq = unit < w.H;
     const int g = unit - w.H;
-    l_rotate_norm(isq ? r + unit * D : r + w.off_k() + g * D, x, D, w.rot, freq, pos, w.qk_norm, w.eps, lane);
+    l_rotate_norm(isq ? r + unit * D : r + w.off_k() + g * D, x, D, w.rot, w.rot_half, freq, pos, w.qk_norm, w.eps, lane);
     __builtin_amdgcn_wave_barrier();
     if (isq) {
         if (qf)

@@ -209,7 +209,7 @@ inline int flow_form(const FlowArgs &a) { return a.mixed ? (a.qkv.ppr == 0 ? 2 :
 // Each returns hipGetLastError() of its launch.
 hipError_t k_repack(hipStream_t s, const DevTensor &t, const void *raw_dev, bool inverse, void *raw_out);
 hipError_t k_embed(hipStream_t s, const DevTensor &emb, const DecodeCtl *ctl, const int32_t *prompt, float *x,
-                   float *rope_cs, int head_size, float theta_scale);
+                   float *rope_cs, int head_size, float theta_scale, float scale = 1.0f, float *x_copy = nullptr);
 hipError_t k_dequant(hipStream_t s, const DevTensor &t, int64_t row0, int64_t nrows, float *y);
 hipError_t k_swiglu(hipStream_t s, float *hb, const float *hb2, int n);
 hipError_t k_matvec(hipStream_t s, PhaseArgs a, int pro, int epi);
@@ -247,7 +247,7 @@ hipError_t k_f32_to_f64(hipStream_t s, const float *x, double *y, int64_t n);
 
 // batched prompt pass (k_prefill.hip); activations travel as bf16 bit patterns
 enum { PF_STORE = 0, PF_RESID = 1, PF_SWIGLU = 2 };
-hipError_t k_pf_embed(hipStream_t s, const DevTensor &emb, const int32_t *tokens, float *X, int M);
+hipError_t k_pf_embed(hipStream_t s, const DevTensor &emb, const int32_t *tokens, float *X, int M, float scale = 1.0f, float *X_copy = nullptr);
 hipError_t k_pf_rope_table(hipStream_t s, float *cs, int pos0, int M, int half, float theta_scale);
 hipError_t k_pf_rmsnorm(hipStream_t s, const float *X, const float *w, uint16_t *out, int M, int64_t K);
 hipError_t k_pf_rope_scatter(hipStream_t s, const float *raw, const float *cs, uint16_t *Qb, float *kc, float *vc, int M,
@@ -272,12 +272,17 @@ int64_t k_pf_kv_tile_bytes(int hs);
 // (a multiple of 4) and of a value where they are fewer than hs, the rest being zero
 hipError_t k_pf_kv_tiles(hipStream_t s, const float *kc, const float *vc, unsigned char *tiles, int n_tiles,
                          int n_tiles_max, int hs, int n_kv, int seq_len, int tile0 = 0, int kdim = 0, int vdim = 0);
+// the same from rows of projected keys and values, whose heads share a last part of the key: kv row r [n_heads kdim | n_heads vdim]
+// (stride ldkv) is position pos0 + r, its shared part `tail` at tails + (pos0 + r) * ldt.  n rows; pos0 a multiple of 32
+hipError_t k_pf_row_tiles(hipStream_t s, const float *kv, int64_t ldkv, const float *tails, int64_t ldt, int tail, unsigned char *tiles,
+                          int pos0, int n, int n_tiles_max, int hs, int n_heads, int kdim, int vdim);
 // a sliding window for k_pf_attention (see pf_attn_kernel)
 struct PfWindow {
     int window = 0, tile0 = 0, vdim = 0;
     float scale = 0.0f;
-    const float *gate = nullptr;  // head gates' logits, or nullptr
-    int64_t ldg = 0, ldo = 0;
+    const float *gate = nullptr;  // gates' logits, one per head or (gate_each) one per element, or nullptr
+    int gate_each = 0;
+    int64_t ldg = 0, ldo = 0, cols = 0;  // columns up to cols (0: ldo) are zeroed behind the heads
 };
 hipError_t k_pf_attention(hipStream_t s, const uint16_t *Qb, uint16_t *Att, const unsigned char *tiles, int n_tiles_max,
                           int M, int qpos0, int hs, int n_heads, int n_kv, int dim, const PfWindow *win = nullptr);

@@ -1,6 +1,7 @@
 // Layered models: a decoder whose layers are described one by one (l2h_layered_create): which mixer (windowed attention, gated
-// delta rule), which feed-forward (none, dense, mixture of experts), an optional per-token input per layer.  This file holds
-// their tensors and per-sequence state and issues their launch sequences; the token loop, the recorded graph, argmax, sampling
+// delta rule, latent attention), which feed-forward (none, dense, mixture of experts), one norm or two, an optional per-token
+// input per layer; a stretch of layers may run several times over.  This file holds their tensors and per-sequence state and
+// issues their launch sequences; the token loop, the recorded graph, argmax, sampling
 // and the prompt pass's chunking are the library's own (api.cpp).
 #include <math.h>
 #include <string.h>
@@ -12,13 +13,26 @@ namespace {
 struct LayerDev {
     l2h_layer d{};
     uint64_t have = 0;  // bit per role that has been set
-    LMat in;            // every row that reads the mixer's input: q | k | v | (gates) or q | k | v | beta | factors
-    LMat o, a2, g2, up, down, router, side_gate, side_proj;
-    std::vector<uint8_t> have_up, have_down;  // experts
+    // every row that reads the mixer's input: q | k | v | (gates) or q | k | v | beta | factors or what LatentShape says; in a
+    // parallel layer also the router's rows and behind them (from row n_plain on) a gated dense feed-forward's.  up, down and
+    // router then name parts of `in` and `o`.
+    LMat in;
+    int n_plain = 0, off_z = 0;
+    // o: the mixer's output matrix; with `joined` its rows go on, at column o_cols, as the dense feed-forward's output matrix
+    LMat o;
+    bool joined = false;
+    int o_cols = 0;
+    LMat a2, g2, up, down, router, side_gate, side_proj, uq, ukv;
+    std::vector<uint8_t> have_up, have_down, have_gate;  // experts
     float *norm1 = nullptr, *norm2 = nullptr, *mixnorm = nullptr, *side_norm = nullptr, *conv = nullptr, *rate = nullptr,
-          *bias = nullptr, *freq = nullptr;
-    // per sequence
-    float *kc = nullptr, *vc = nullptr;      // attention
+          *bias = nullptr, *freq = nullptr, *qnorm = nullptr, *kvnorm = nullptr, *router_bias = nullptr;
+    bool stacked() const { return d.parallel && d.ff == L2H_FF_DENSE && d.ff_gated; }  // its feed-forward's rows are in `in`
+    int up_rows() const { return d.ff_dim * (d.ff_gated ? 2 : 1); }                     // rows of up, of one expert's up
+};
+// One run of a layer: a looped layer has one for each pass.  What a sequence carries belongs to the run.
+struct LayerRun {
+    int layer = 0, pass = -1;                 // pass: of which this is the first layer (-1: of none)
+    float *kc = nullptr, *vc = nullptr;       // attention; latent attention has its rows in kc
     float *ring = nullptr, *state = nullptr;  // delta rule
 };
 }  // namespace
@@ -26,20 +40,26 @@ struct LayerDev {
 struct Layered {
     l2h_layered_config c{};
     std::vector<LayerDev> layer;
+    std::vector<LayerRun> run;
     LMat head;
+    float *loop_step = nullptr;
     uint16_t *side_emb = nullptr;
     float *final_norm = nullptr;
     uint64_t have = 0;
     int pos = 0;  // positions the state has taken in
     // one token
     float *x_alt = nullptr, *in = nullptr, *mix = nullptr, *ssq = nullptr, *gate = nullptr, *hid = nullptr, *z = nullptr,
-          *se = nullptr, *y = nullptr, *part = nullptr;
+          *se = nullptr, *y = nullptr, *part = nullptr, *x0 = nullptr, *lq = nullptr, *qa = nullptr;
     // prompt pass, for `cap` positions
     int cap = 0;
     int32_t *tok = nullptr, *choice = nullptr, *slot_row = nullptr, *slot_of = nullptr, *n_tiles = nullptr, *want = nullptr;
     GemmTile *tiles = nullptr;
     float *X = nullptr, *raw = nullptr, *qkv = nullptr, *kq = nullptr, *beta = nullptr, *lg = nullptr, *gt = nullptr, *ob = nullptr,
-          *zb = nullptr, *score = nullptr, *slot_scale = nullptr, *yb = nullptr, *Y = nullptr, *wl = nullptr, *rec = nullptr;
+          *zb = nullptr, *score = nullptr, *slot_scale = nullptr, *yb = nullptr, *Y = nullptr, *wl = nullptr, *rec = nullptr, *X0 = nullptr, *lat_qa = nullptr,
+          *lat_part = nullptr, *kvx = nullptr;
+    uint16_t *qb = nullptr, *xc = nullptr;
+    int kvx_cap = 0;
+    void *cq = nullptr;
     void *xn = nullptr, *fa = nullptr, *fg = nullptr, *ao = nullptr, *hb = nullptr, *sb = nullptr;
     int want_cap = 0;
     // residual stream after every layer of the last prompt pass (l2h_layered_keep)
@@ -52,12 +72,22 @@ struct Layered {
     int W() const { return c.width; }
     int ldw() const { return pad64(c.width); }
     int asize() const { return c.precision ? 4 : 2; }
+    bool adds_again() const { return c.loop_times > 1 && c.loop_stop > c.loop_start; }  // a later pass adds the starting x
 };
 
 static WindowShape window_shape(const Layered *l, const LayerDev &L) {
     WindowShape w{};
     w.H = L.d.n_heads, w.G = L.d.n_kv_heads, w.D = L.d.dim, w.V = L.d.vdim;
     w.window = L.d.window, w.rot = L.d.rot_dims, w.gated = L.d.head_gate, w.qk_norm = L.d.qk_norm;
+    w.rot_half = L.d.rot_half;
+    w.scale = L.d.scale, w.eps = l->c.norm_eps;
+    w.seq_len = l->c.seq_len;
+    return w;
+}
+static LatentShape latent_shape(const Layered *l, const LayerDev &L) {
+    LatentShape w{};
+    w.H = L.d.n_heads, w.D = L.d.dim, w.R = L.d.rot_size, w.V = L.d.vdim, w.C = L.d.kv_rank, w.Q = L.d.q_rank;
+    w.rot = L.d.rot_dims, w.rot_half = L.d.rot_half, w.gated = L.d.out_gate;
     w.scale = L.d.scale, w.eps = l->c.norm_eps;
     w.seq_len = l->c.seq_len;
     return w;
@@ -70,6 +100,7 @@ static DeltaShape delta_shape(const Layered *l, const LayerDev &L) {
     return d;
 }
 static int mixer_rows(const Layered *l, const LayerDev &L) {
+    if (L.d.mixer == L2H_MIX_LATENT) return latent_shape(l, L).n_in();
     return L.d.mixer == L2H_MIX_ATTENTION ? window_shape(l, L).n_in() : delta_shape(l, L).n_in();
 }
 
@@ -83,12 +114,26 @@ static int attention_tile_size(const l2h_layer &d) {
 static int attention_tiles(const Layered *l, const LayerDev &L, int cap) {
     return (int)std::min<int64_t>(((int64_t)l->c.seq_len + 31) / 32, ((int64_t)L.d.window + cap) / 32 + 2);
 }
+// the same for the keys and values that a latent attention layer's heads make for themselves; all keys are seen
+static int latent_tile_size(const Layered *l, const l2h_layer &d) {
+    if (l->c.precision) return 0;
+    for (int hs : {32, 64, 96, 128, 192})
+        if (d.dim + d.rot_size <= hs && d.vdim <= std::min(hs, 128)) return hs;
+    return 0;
+}
+static int latent_tiles(const Layered *l) { return (l->c.seq_len + 31) / 32; }
 
 static int mat_alloc(l2h_model *m, LMat *t, int64_t rows, int K) {
     t->rows = rows;
     t->K = K;
     t->ld = pad64(K);
     return dalloc(m, &t->w, rows * t->ld, true);
+}
+static LMat mat_rows(const LMat &t, int64_t row0, int64_t rows) {
+    LMat v = t;
+    v.w = t.w ? t.w + row0 * t.ld : nullptr;
+    v.rows = rows;
+    return v;
 }
 
 // ------------------------------------------------------------------------------------------
@@ -105,28 +150,41 @@ extern "C" int l2h_layered_create(l2h_ctx *ctx, const l2h_layered_config *cfg, c
     if (c.width > 32768) return set_err(ctx, L2H_EINVAL, "width %d is larger than 32768", c.width);
     for (int i = 0; i < c.n_layers; i++) {
         const l2h_layer &d = layers[i];
-        if (d.mixer != L2H_MIX_ATTENTION && d.mixer != L2H_MIX_CHANNEL_DELTA) return set_err(ctx, L2H_EINVAL, "layer %d: unknown mixer %d", i, d.mixer);
+        if (d.mixer != L2H_MIX_ATTENTION && d.mixer != L2H_MIX_CHANNEL_DELTA && d.mixer != L2H_MIX_LATENT) return set_err(ctx, L2H_EINVAL, "layer %d: unknown mixer %d", i, d.mixer);
         if (d.n_heads < 1 || d.n_kv_heads < 1 || d.n_heads % d.n_kv_heads != 0)
             return set_err(ctx, L2H_EINVAL, "layer %d: %d heads over %d key/value heads", i, d.n_heads, d.n_kv_heads);
-        if (d.dim < 1 || d.dim > 256 || d.vdim < 1 || d.vdim > 256)
-            return set_err(ctx, L2H_EINVAL, "layer %d: head sizes %d, %d (1 to 256 are built)", i, d.dim, d.vdim);
+        const int max_head = d.mixer == L2H_MIX_LATENT ? 1024 : 256;
+        if (d.dim < 1 || d.dim > max_head || d.vdim < 1 || d.vdim > max_head)
+            return set_err(ctx, L2H_EINVAL, "layer %d: head sizes %d, %d (1 to %d are built)", i, d.dim, d.vdim, max_head);
         if ((int64_t)d.n_heads * d.vdim > 32768) return set_err(ctx, L2H_EINVAL, "layer %d: heads x value size above 32768", i);
         if (d.mixer == L2H_MIX_ATTENTION) {
             if (d.window < 1 || std::min(d.window, c.seq_len) > 900000) return set_err(ctx, L2H_EINVAL, "layer %d: window %d", i, d.window);
-            if (d.rot_dims < 0 || d.rot_dims > d.dim || d.rot_dims % 2) return set_err(ctx, L2H_EINVAL, "layer %d: %d rotated of %d dimensions", i, d.rot_dims, d.dim);
-            if (d.rot_dims && !(d.rot_base > 0.0)) return set_err(ctx, L2H_EINVAL, "layer %d: rotation base must be positive", i);
-            if (d.rot_original > 0.0 && (!(d.rot_factor > 0.0) || !(d.rot_low > 0.0) || !(d.rot_high > d.rot_low)))
-                return set_err(ctx, L2H_EINVAL, "layer %d: frequency scaling needs factor > 0 and 0 < low < high", i);
+        } else if (d.mixer == L2H_MIX_LATENT) {
+            if (d.n_kv_heads != d.n_heads) return set_err(ctx, L2H_EINVAL, "layer %d: latent attention has a key/value head for every head", i);
+            if (d.q_rank < 1 || d.q_rank > 32768 || d.kv_rank < 1 || d.kv_rank > L_LATENT_MAX_RANK || d.rot_size < 0 || d.rot_size > 256)
+                return set_err(ctx, L2H_EINVAL, "layer %d: ranks %d, %d, rotated part %d", i, d.q_rank, d.kv_rank, d.rot_size);
+            if ((int64_t)d.n_heads * (d.dim + d.rot_size) > 65536) return set_err(ctx, L2H_EINVAL, "layer %d: heads x key size above 65536", i);
         } else if (d.taps < 1 || d.taps > 64 || d.decay_rank < 1 || d.decay_rank > 4096 || d.gate_rank < 1 || d.gate_rank > 4096) {
             return set_err(ctx, L2H_EINVAL, "layer %d: taps %d, ranks %d, %d", i, d.taps, d.decay_rank, d.gate_rank);
         }
+        if (d.mixer != L2H_MIX_CHANNEL_DELTA) {
+            const int turns = d.mixer == L2H_MIX_LATENT ? d.rot_size : d.dim;
+            if (d.rot_dims < 0 || d.rot_dims > turns || d.rot_dims % 2) return set_err(ctx, L2H_EINVAL, "layer %d: %d rotated of %d dimensions", i, d.rot_dims, turns);
+            if (d.rot_dims && !(d.rot_base > 0.0)) return set_err(ctx, L2H_EINVAL, "layer %d: rotation base must be positive", i);
+            if (d.rot_original > 0.0 && (!(d.rot_factor > 0.0) || !(d.rot_low > 0.0) || !(d.rot_high > d.rot_low)))
+                return set_err(ctx, L2H_EINVAL, "layer %d: frequency scaling needs factor > 0 and 0 < low < high", i);
+        }
         if (d.ff != L2H_FF_NONE && d.ff != L2H_FF_DENSE && d.ff != L2H_FF_EXPERTS) return set_err(ctx, L2H_EINVAL, "layer %d: unknown feed-forward %d", i, d.ff);
-        if (d.ff != L2H_FF_NONE && (d.ff_dim < 1 || d.ff_act < 0 || d.ff_act > 2)) return set_err(ctx, L2H_EINVAL, "layer %d: feed-forward of %d, activation %d", i, d.ff_dim, d.ff_act);
+        if (d.ff != L2H_FF_NONE && (d.ff_dim < 1 || d.ff_act < 0 || d.ff_act > L2H_ACT_SILU)) return set_err(ctx, L2H_EINVAL, "layer %d: feed-forward of %d, activation %d", i, d.ff_dim, d.ff_act);
         if (d.ff == L2H_FF_DENSE && d.ff_dim > 36864) return set_err(ctx, L2H_EINVAL, "layer %d: feed-forward of %d is larger than 36864", i, d.ff_dim);
         if (d.ff == L2H_FF_EXPERTS && (d.n_experts < 1 || d.n_experts > 1024 || d.top < 1 || d.top > d.n_experts || d.top > 64 ||
                                        (int64_t)d.top * pad64(d.ff_dim) > 36864))
             return set_err(ctx, L2H_EINVAL, "layer %d: %d of %d experts of %d", i, d.top, d.n_experts, d.ff_dim);
+        if (d.ff == L2H_FF_EXPERTS && d.route != L2H_ROUTE_SIGMOID_IN && d.route != L2H_ROUTE_SOFTMAX_OUT)
+            return set_err(ctx, L2H_EINVAL, "layer %d: unknown kind of router %d", i, d.route);
     }
+    if (c.loop_times < 0 || (c.loop_times > 0 && (c.loop_start < 0 || c.loop_stop <= c.loop_start || c.loop_stop > c.n_layers)))
+        return set_err(ctx, L2H_EINVAL, "layers %d to %d run %d times", c.loop_start, c.loop_stop, c.loop_times);
     HIPCHK(ctx, hipSetDevice(ctx->device));
     l2h_model *m = new l2h_model();
     Layered *l = new Layered();
@@ -138,11 +196,23 @@ extern "C" int l2h_layered_create(l2h_ctx *ctx, const l2h_layered_config *cfg, c
     m->c.seq_len = c.seq_len;
     l->c = c;
     l->layer.resize((size_t)c.n_layers);
+    for (int i = 0; i < c.n_layers; i++) {
+        const bool again = c.loop_times > 0 && i == c.loop_start;
+        for (int t = 0; t < (again ? c.loop_times : 1); t++)
+            for (int j = i; j < (again ? c.loop_stop : i + 1); j++) {
+                LayerRun r;
+                r.layer = j;
+                if (again && j == i) r.pass = t;
+                l->run.push_back(r);
+            }
+        if (again) i = c.loop_stop - 1;
+    }
     int rc = L2H_OK;
 #define A(call) \
     if (rc == L2H_OK) rc = (call)
     A(mat_alloc(m, &l->head, c.vocab_size, c.width));
     A(dalloc(m, &l->final_norm, c.width, true));
+    if (c.loop_times) A(dalloc(m, &l->loop_step, (int64_t)c.loop_times * c.width, true));
     if (c.side_dim) A(dalloc(m, &l->side_emb, (int64_t)c.vocab_size * c.n_layers * c.side_dim, true));
     DevTensor &e = m->glob[L2H_TOK_EMB];
     e.type = L2H_TYPE_BF16;
@@ -156,10 +226,23 @@ extern "C" int l2h_layered_create(l2h_ctx *ctx, const l2h_layered_config *cfg, c
         L.d = layers[i];
         const l2h_layer &d = L.d;
         const int HV = d.n_heads * d.vdim;
-        A(mat_alloc(m, &L.in, mixer_rows(l, L), c.width));
-        A(mat_alloc(m, &L.o, c.width, HV));
+        L.n_plain = mixer_rows(l, L);
+        const bool routed = d.parallel && d.ff == L2H_FF_EXPERTS;
+        if (routed || L.stacked()) L.n_plain = pad4(L.n_plain);
+        L.off_z = L.n_plain;
+        if (routed) L.n_plain = pad4(L.off_z + d.n_experts);
+        A(mat_alloc(m, &L.in, L.n_plain + (L.stacked() ? L.up_rows() : 0), c.width));
+        L.o_cols = pad64(HV);
+        L.joined = d.parallel && d.ff == L2H_FF_DENSE && d.mixer == L2H_MIX_LATENT && L.o_cols + d.ff_dim <= 36864;
+        A(mat_alloc(m, &L.o, c.width, L.joined ? L.o_cols + d.ff_dim : HV));
         A(dalloc(m, &L.norm1, c.width, true));
-        if (d.mixer == L2H_MIX_ATTENTION) {
+        if (d.mixer == L2H_MIX_LATENT) {
+            A(mat_alloc(m, &L.uq, d.n_heads * (d.dim + d.rot_size), d.q_rank));
+            A(mat_alloc(m, &L.ukv, d.n_heads * (d.dim + d.vdim), d.kv_rank));
+            A(dalloc(m, &L.qnorm, d.q_rank, true));
+            A(dalloc(m, &L.kvnorm, d.kv_rank, true));
+        }
+        if (d.mixer != L2H_MIX_CHANNEL_DELTA) {
             std::vector<float> f((size_t)d.rot_dims / 2 + 1, 0.0f);
             for (int k = 0; k < d.rot_dims / 2; k++) {
                 double v = pow(d.rot_base, -2.0 * k / d.rot_dims);
@@ -188,11 +271,19 @@ extern "C" int l2h_layered_create(l2h_ctx *ctx, const l2h_layered_config *cfg, c
         }
         if (d.ff != L2H_FF_NONE) {
             const int64_t n = d.ff == L2H_FF_EXPERTS ? d.n_experts : 1;
-            A(dalloc(m, &L.norm2, c.width, true));
-            A(mat_alloc(m, &L.up, n * d.ff_dim, c.width));
-            A(mat_alloc(m, &L.down, n * c.width, d.ff_dim));
+            if (!d.parallel) A(dalloc(m, &L.norm2, c.width, true));
+            if (L.stacked())
+                L.up = mat_rows(L.in, L.n_plain, L.up_rows());
+            else
+                A(mat_alloc(m, &L.up, n * L.up_rows(), c.width));
+            if (!L.joined) A(mat_alloc(m, &L.down, n * c.width, d.ff_dim));
             if (d.ff == L2H_FF_EXPERTS) {
-                A(mat_alloc(m, &L.router, n, c.width));
+                if (routed)
+                    L.router = mat_rows(L.in, L.off_z, n);
+                else
+                    A(mat_alloc(m, &L.router, n, c.width));
+                if (d.router_bias) A(dalloc(m, &L.router_bias, n, true));
+                L.have_gate.assign((size_t)n, 0);
                 L.have_up.assign((size_t)n, 0);
                 L.have_down.assign((size_t)n, 0);
             }
@@ -221,10 +312,11 @@ void layered_free(l2h_model *m) {
 // tensors
 // ------------------------------------------------------------------------------------------
 static const char *layered_role_name(int r) {
-    static const char *n[] = {"token embedding", "final norm", "output", "norm 1", "norm 2", "q", "k", "v", "mixer output", "up", "down", "(w3)",
+    static const char *n[] = {"token embedding", "final norm", "output", "norm 1", "norm 2", "q", "k", "v", "mixer output", "up", "down", "w3",
                               "head gate", "beta", "decay rate", "decay bias", "decay factor in", "decay factor out", "gate factor in",
                               "gate factor out", "mixer norm", "q convolution", "k convolution", "v convolution", "router", "expert up",
-                              "expert down", "side embedding", "side gate", "side projection", "side norm"};
+                              "expert down", "side embedding", "side gate", "side projection", "side norm", "q down", "q norm", "q up",
+                              "k/v down", "k/v norm", "k up", "v up", "output gate", "router bias", "expert gate", "loop step"};
     return (r >= 0 && r < L2H_N_LAYERED_ROLES) ? n[r] : "?";
 }
 
@@ -238,7 +330,7 @@ static float bf16_value(uint16_t b) {
 // where a tensor goes: rows of a matrix, or an fp32 vector
 struct LSlot {
     LMat *mat = nullptr;
-    int64_t row0 = 0;
+    int64_t row0 = 0, row_step = 1, col0 = 0;
     float *vec = nullptr;
     uint16_t *flat = nullptr;  // bf16, unpadded
     int64_t e0 = 0, e1 = 0;
@@ -268,6 +360,10 @@ static int layered_slot(l2h_model *m, int role, int layer, int expert, LSlot *s)
         return L2H_OK;
     case L2H_OUTPUT: mat(&l->head, 0, c.vocab_size); return L2H_OK;
     case L2H_RMS_FINAL: vec(l->final_norm, c.width); return L2H_OK;
+    case L2H_LOOP_STEP:
+        if (!c.loop_times) break;
+        vec(l->loop_step, c.width, c.loop_times);
+        return L2H_OK;
     case L2H_SIDE_EMB:
         if (!c.side_dim) break;
         t.flat = l->side_emb;
@@ -278,41 +374,67 @@ static int layered_slot(l2h_model *m, int role, int layer, int expert, LSlot *s)
     LayerDev &L = l->layer[(size_t)layer];
     const l2h_layer &d = L.d;
     const int H = d.n_heads, G = d.n_kv_heads, D = d.dim, V = d.vdim;
-    const bool att = d.mixer == L2H_MIX_ATTENTION;
+    const bool att = d.mixer == L2H_MIX_ATTENTION, lat = d.mixer == L2H_MIX_LATENT;
+    const LatentShape ls = latent_shape(l, L);
+    // rows of a feed-forward's input matrix: with a gate, gate and up in turn
+    auto pair = [&](int64_t row0, int which) {
+        mat(&L.up, d.ff_gated ? 2 * row0 + which : row0, d.ff_dim);
+        t.row_step = d.ff_gated ? 2 : 1;
+    };
     const DeltaShape ds = delta_shape(l, L);
     const WindowShape ws = window_shape(l, L);
     switch (role) {
     case L2H_RMS_ATT: vec(L.norm1, c.width); return L2H_OK;
     case L2H_RMS_FFN:
-        if (d.ff == L2H_FF_NONE) break;
+        if (!L.norm2) break;
         vec(L.norm2, c.width);
         return L2H_OK;
-    case L2H_WQ: mat(&L.in, 0, att ? H * D : G * D); return L2H_OK;
-    case L2H_WK: mat(&L.in, att ? ws.off_k() : G * D, G * D); return L2H_OK;
-    case L2H_WV: mat(&L.in, att ? ws.off_v() : 2 * G * D, att ? G * V : H * V); return L2H_OK;
-    case L2H_WO: mat(&L.o, 0, c.width); return L2H_OK;
+    case L2H_WQ:
+        if (lat) break;
+        mat(&L.in, 0, att ? H * D : G * D);
+        return L2H_OK;
+    case L2H_WK:
+        if (lat) break;
+        mat(&L.in, att ? ws.off_k() : G * D, G * D);
+        return L2H_OK;
+    case L2H_WV:
+        if (lat) break;
+        mat(&L.in, att ? ws.off_v() : 2 * G * D, att ? G * V : H * V);
+        return L2H_OK;
+    case L2H_WO:
+        mat(&L.o, 0, c.width);
+        t.e0 = H * V;
+        return L2H_OK;
     case L2H_HEAD_GATE:
         if (!att || !d.head_gate) break;
         mat(&L.in, ws.off_g(), H);
         return L2H_OK;
     case L2H_W1:
-        if (d.ff != L2H_FF_DENSE) break;
-        mat(&L.up, 0, d.ff_dim);
+    case L2H_W3:
+        if (d.ff != L2H_FF_DENSE || (role == L2H_W3 && !d.ff_gated)) break;
+        pair(0, role == L2H_W3);
         return L2H_OK;
     case L2H_W2:
         if (d.ff != L2H_FF_DENSE) break;
-        mat(&L.down, 0, c.width);
+        mat(L.joined ? &L.o : &L.down, 0, c.width);
+        t.e0 = d.ff_dim;
+        if (L.joined) t.col0 = L.o_cols;
         return L2H_OK;
     case L2H_ROUTER:
         if (d.ff != L2H_FF_EXPERTS) break;
         mat(&L.router, 0, d.n_experts);
         return L2H_OK;
+    case L2H_ROUTER_BIAS:
+        if (!L.router_bias) break;
+        vec(L.router_bias, d.n_experts);
+        return L2H_OK;
     case L2H_EXPERT_UP:
+    case L2H_EXPERT_GATE:
     case L2H_EXPERT_DOWN:
-        if (d.ff != L2H_FF_EXPERTS) break;
+        if (d.ff != L2H_FF_EXPERTS || (role == L2H_EXPERT_GATE && !d.ff_gated)) break;
         if (expert < 0 || expert >= d.n_experts) return set_err(m->ctx, L2H_EINVAL, "expert %d out of range", expert);
-        if (role == L2H_EXPERT_UP)
-            mat(&L.up, (int64_t)expert * d.ff_dim, d.ff_dim);
+        if (role != L2H_EXPERT_DOWN)
+            pair((int64_t)expert * d.ff_dim, role == L2H_EXPERT_UP);
         else
             mat(&L.down, (int64_t)expert * c.width, c.width);
         return L2H_OK;
@@ -329,7 +451,20 @@ static int layered_slot(l2h_model *m, int role, int layer, int expert, LSlot *s)
         vec(L.side_norm, c.width);
         return L2H_OK;
     }
-    if (!att) switch (role) {
+    if (lat) switch (role) {
+        case L2H_Q_DOWN: mat(&L.in, 0, d.q_rank); return L2H_OK;
+        case L2H_Q_NORM: vec(L.qnorm, d.q_rank); return L2H_OK;
+        case L2H_Q_UP: mat(&L.uq, 0, H * (D + d.rot_size)); return L2H_OK;
+        case L2H_KV_DOWN: mat(&L.in, ls.off_kv(), d.kv_rank + d.rot_size); return L2H_OK;
+        case L2H_KV_NORM: vec(L.kvnorm, d.kv_rank); return L2H_OK;
+        case L2H_K_UP: mat(&L.ukv, 0, H * D); return L2H_OK;
+        case L2H_V_UP: mat(&L.ukv, H * D, H * V); return L2H_OK;
+        case L2H_OUT_GATE:
+            if (!d.out_gate) break;
+            mat(&L.in, ls.off_g(), H * V);
+            return L2H_OK;
+        }
+    if (d.mixer == L2H_MIX_CHANNEL_DELTA) switch (role) {
         case L2H_BETA: mat(&L.in, ds.off_b(), H); return L2H_OK;
         case L2H_DECAY_IN: mat(&L.in, ds.off_a(), d.decay_rank); return L2H_OK;
         case L2H_GATE_IN: mat(&L.in, ds.off_g(), d.gate_rank); return L2H_OK;
@@ -383,15 +518,16 @@ int layered_set_tensor(l2h_model *m, int role, int layer, int expert, int type, 
     } else if (s.flat) {
         HIPCHK(ctx, hipMemcpy(s.flat, host, (size_t)(ne0 * ne1) * 2, hipMemcpyHostToDevice));
     } else {
-        HIPCHK(ctx, hipMemcpy2D(s.mat->w + s.row0 * s.mat->ld, (size_t)s.mat->ld * 2, host, (size_t)ne0 * 2, (size_t)ne0 * 2, (size_t)ne1,
-                                hipMemcpyHostToDevice));
+        HIPCHK(ctx, hipMemcpy2D(s.mat->w + s.row0 * s.mat->ld + s.col0, (size_t)(s.mat->ld * s.row_step) * 2, host, (size_t)ne0 * 2,
+                                (size_t)ne0 * 2, (size_t)ne1, hipMemcpyHostToDevice));
     }
-    if (role == L2H_TOK_EMB || role == L2H_OUTPUT || role == L2H_RMS_FINAL || role == L2H_SIDE_EMB) {
+    if (role == L2H_TOK_EMB || role == L2H_OUTPUT || role == L2H_RMS_FINAL || role == L2H_SIDE_EMB || role == L2H_LOOP_STEP) {
         l->have |= (uint64_t)1 << role;
     } else {
         LayerDev &L = l->layer[(size_t)layer];
         L.have |= (uint64_t)1 << role;
         if (role == L2H_EXPERT_UP) L.have_up[(size_t)expert] = 1;
+        if (role == L2H_EXPERT_GATE) L.have_gate[(size_t)expert] = 1;
         if (role == L2H_EXPERT_DOWN) L.have_down[(size_t)expert] = 1;
     }
     return L2H_OK;
@@ -400,12 +536,33 @@ int layered_set_tensor(l2h_model *m, int role, int layer, int expert, int type, 
 // ------------------------------------------------------------------------------------------
 // state
 // ------------------------------------------------------------------------------------------
+// floats of what a run of the layer keeps for a sequence: run_state 0 .. 3
+static void run_floats(const Layered *l, const LayerDev &L, int64_t n[4]) {
+    n[0] = n[1] = n[2] = n[3] = 0;
+    if (L.d.mixer == L2H_MIX_ATTENTION) {
+        const WindowShape w = window_shape(l, L);
+        n[0] = (int64_t)w.G * w.Dp() * w.seq_len;
+        n[1] = (int64_t)w.G * w.V * w.seq_len;
+    } else if (L.d.mixer == L2H_MIX_LATENT) {
+        const LatentShape w = latent_shape(l, L);
+        n[0] = (int64_t)w.ld() * w.seq_len;
+    } else {
+        const DeltaShape s = delta_shape(l, L);
+        n[2] = (int64_t)s.taps * s.channels();
+        n[3] = (int64_t)s.H * s.D * s.V;
+    }
+}
+static float **run_state(LayerRun &r, int k) {
+    float **p[4] = {&r.kc, &r.vc, &r.ring, &r.state};
+    return p[k];
+}
+
 int layered_finalize(l2h_model *m) {
     l2h_ctx *ctx = m->ctx;
     Layered *l = m->lay;
     const l2h_layered_config &c = l->c;
     int n_in = 1, hv = 1, hid = 1, ne = 1, ssq = 1;
-    int64_t part = 1;
+    int64_t part = 1, lq = 0, qa = 0;
     auto missing = [&](uint64_t have, int role, int layer) -> int {
         if (have >> role & 1) return L2H_OK;
         return set_err(ctx, L2H_ESTATE, "missing tensor \"%s\"%s%s", layered_role_name(role), layer >= 0 ? " of layer " : "",
@@ -415,46 +572,63 @@ int layered_finalize(l2h_model *m) {
     for (int r : {L2H_TOK_EMB, L2H_OUTPUT, L2H_RMS_FINAL})
         if ((rc = missing(l->have, r, -1))) return rc;
     if (c.side_dim && (rc = missing(l->have, L2H_SIDE_EMB, -1))) return rc;
+    if (c.loop_times && (rc = missing(l->have, L2H_LOOP_STEP, -1))) return rc;
 #define DA(p, n, z)                       \
     if ((rc = dalloc(m, &(p), (n), (z)))) \
         return rc;
     for (int i = 0; i < c.n_layers; i++) {
         LayerDev &L = l->layer[(size_t)i];
         const l2h_layer &d = L.d;
-        std::vector<int> need = {L2H_RMS_ATT, L2H_WQ, L2H_WK, L2H_WV, L2H_WO};
-        if (d.mixer == L2H_MIX_ATTENTION) {
-            if (d.head_gate) need.push_back(L2H_HEAD_GATE);
+        std::vector<int> need = {L2H_RMS_ATT, L2H_WO};
+        if (d.mixer == L2H_MIX_LATENT) {
+            for (int r : {L2H_Q_DOWN, L2H_Q_NORM, L2H_Q_UP, L2H_KV_DOWN, L2H_KV_NORM, L2H_K_UP, L2H_V_UP}) need.push_back(r);
+            if (d.out_gate) need.push_back(L2H_OUT_GATE);
         } else {
+            for (int r : {L2H_WQ, L2H_WK, L2H_WV}) need.push_back(r);
+        }
+        if (d.mixer == L2H_MIX_ATTENTION && d.head_gate) need.push_back(L2H_HEAD_GATE);
+        if (d.mixer == L2H_MIX_CHANNEL_DELTA) {
             for (int r : {L2H_BETA, L2H_DECAY_RATE, L2H_DECAY_BIAS, L2H_DECAY_IN, L2H_DECAY_OUT, L2H_GATE_IN, L2H_GATE_OUT, L2H_MIX_NORM,
                           L2H_CONV_Q, L2H_CONV_K, L2H_CONV_V})
                 need.push_back(r);
         }
-        if (d.ff != L2H_FF_NONE) need.push_back(L2H_RMS_FFN);
+        if (L.norm2) need.push_back(L2H_RMS_FFN);
         if (d.ff == L2H_FF_DENSE) need.push_back(L2H_W1), need.push_back(L2H_W2);
+        if (d.ff == L2H_FF_DENSE && d.ff_gated) need.push_back(L2H_W3);
         if (d.ff == L2H_FF_EXPERTS) {
             need.push_back(L2H_ROUTER);
+            if (d.router_bias) need.push_back(L2H_ROUTER_BIAS);
             for (int e = 0; e < d.n_experts; e++)
-                if (!L.have_up[(size_t)e] || !L.have_down[(size_t)e]) return set_err(ctx, L2H_ESTATE, "missing expert %d of layer %d", e, i);
+                if (!L.have_up[(size_t)e] || !L.have_down[(size_t)e] || (d.ff_gated && !L.have_gate[(size_t)e])) return set_err(ctx, L2H_ESTATE, "missing expert %d of layer %d", e, i);
         }
         if (c.side_dim)
             for (int r : {L2H_SIDE_GATE, L2H_SIDE_PROJ, L2H_SIDE_NORM}) need.push_back(r);
         for (int r : need)
             if ((rc = missing(L.have, r, i))) return rc;
-        if (d.mixer == L2H_MIX_ATTENTION) {
-            const WindowShape w = window_shape(l, L);
-            DA(L.kc, (int64_t)w.G * w.Dp() * w.seq_len, true);
-            DA(L.vc, (int64_t)w.G * w.V * w.seq_len, true);
-            part = std::max(part, window_part_floats(w));
-        } else {
-            const DeltaShape s = delta_shape(l, L);
-            DA(L.ring, (int64_t)s.taps * s.channels(), true);
-            DA(L.state, (int64_t)s.H * s.D * s.V, true);
-            ssq = std::max(ssq, s.H * delta_splits(s.V));
+        if (d.mixer == L2H_MIX_ATTENTION) part = std::max(part, window_part_floats(window_shape(l, L)));
+        if (d.mixer == L2H_MIX_LATENT) {
+            const LatentShape w = latent_shape(l, L);
+            part = std::max(part, latent_part_floats(w, w.H));
+            lq = std::max(lq, (int64_t)w.H * w.hq());
+            qa = std::max(qa, (int64_t)w.H * w.ld());
         }
-        n_in = std::max(n_in, mixer_rows(l, L));
-        hv = std::max(hv, d.n_heads * d.vdim);
+        if (d.mixer == L2H_MIX_CHANNEL_DELTA) ssq = std::max(ssq, d.n_heads * delta_splits(d.vdim));
+        n_in = std::max(n_in, L.n_plain);
+        hv = std::max(hv, std::max(d.n_heads * d.vdim, L.joined ? L.o.ld : 0));
         if (d.ff != L2H_FF_NONE) hid = std::max(hid, d.ff_dim * (d.ff == L2H_FF_EXPERTS ? d.top : 1));
         if (d.ff == L2H_FF_EXPERTS) ne = std::max(ne, d.n_experts);
+    }
+    for (LayerRun &r : l->run) {
+        const LayerDev &L = l->layer[(size_t)r.layer];
+        int64_t n[4];
+        run_floats(l, L, n);
+        for (int k = 0; k < 4; k++)
+            if (n[k]) DA(*run_state(r, k), n[k], true);
+    }
+    if (l->adds_again()) DA(l->x0, c.width, true);
+    if (lq) {
+        DA(l->lq, lq, true);
+        DA(l->qa, qa, true);
     }
     DA(m->x, c.width, true);
     DA(l->x_alt, c.width, true);
@@ -486,17 +660,11 @@ void layered_advance(l2h_model *m, int pos) { m->lay->pos = pos; }
 int layered_reset(l2h_model *m) {
     Layered *l = m->lay;
     hipStream_t s = m->ctx->stream;
-    for (LayerDev &L : l->layer) {
-        const l2h_layer &d = L.d;
-        if (d.mixer == L2H_MIX_ATTENTION) {
-            const WindowShape w = window_shape(l, L);
-            HIPCHK(m->ctx, hipMemsetAsync(L.kc, 0, (size_t)w.G * w.Dp() * w.seq_len * 4, s));
-            HIPCHK(m->ctx, hipMemsetAsync(L.vc, 0, (size_t)w.G * w.V * w.seq_len * 4, s));
-        } else {
-            const DeltaShape t = delta_shape(l, L);
-            HIPCHK(m->ctx, hipMemsetAsync(L.ring, 0, (size_t)t.taps * t.channels() * 4, s));
-            HIPCHK(m->ctx, hipMemsetAsync(L.state, 0, (size_t)t.H * t.D * t.V * 4, s));
-        }
+    for (LayerRun &r : l->run) {
+        int64_t n[4];
+        run_floats(l, l->layer[(size_t)r.layer], n);
+        for (int k = 0; k < 4; k++)
+            if (n[k]) HIPCHK(m->ctx, hipMemsetAsync(*run_state(r, k), 0, (size_t)n[k] * 4, s));
     }
     HIPCHK(m->ctx, hipStreamSynchronize(s));
     l->pos = 0;
@@ -523,28 +691,35 @@ static RowsArgs rows_of(const LMat &w, const float *x, float *out) {
     return a;
 }
 
-// The residual stream moves to the other of its two buffers where a layer's pending per-token update is applied, by the
-// launch that reads it next; it ends in m->x.
-static float *stream_buf(const l2h_model *m, int layer) {
-    const Layered *l = m->lay;
-    return (l->c.side_dim && ((l->c.n_layers - layer) & 1)) ? l->x_alt : m->x;
-}
-
-// norm of the residual stream (with the update that the layer before left pending) and a matrix
-static RowsArgs normed(const l2h_model *m, int layer, const LMat &w, const float *normw, float *out) {
-    const Layered *l = m->lay;
-    RowsArgs a = rows_of(w, stream_buf(m, layer), out);
-    a.normw = normw;
-    a.eps = l->c.norm_eps;
-    if (l->c.side_dim && layer > 0) {
-        a.x = stream_buf(m, layer - 1);
-        a.y = l->y;
-        a.yw = l->layer[(size_t)layer - 1].side_norm;
-        a.mult = l->c.residual_mult;
-        a.x_out = stream_buf(m, layer);
+// The residual stream moves to the other of its two buffers where a layer's pending per-token update is applied by the launch
+// that reads it next; it ends in m->x.  (Before a pass of a loop the update is applied where the stream lies.)
+struct Stream {
+    l2h_model *m;
+    float *x;
+    const float *yw = nullptr;  // the update l->y is pending, with these weights
+    explicit Stream(l2h_model *model) : m(model) {
+        const Layered *l = m->lay;
+        int moves = 0;
+        for (size_t r = 0; l->c.side_dim && r < l->run.size(); r++)
+            if (r + 1 == l->run.size() || l->run[r + 1].pass < 0) moves++;
+        x = moves & 1 ? l->x_alt : m->x;
     }
-    return a;
-}
+    // norm of the stream and a matrix
+    RowsArgs normed(const LMat &w, const float *normw, float *out) {
+        const Layered *l = m->lay;
+        RowsArgs a = rows_of(w, x, out);
+        a.normw = normw;
+        a.eps = l->c.norm_eps;
+        if (yw) {
+            a.y = l->y;
+            a.yw = yw;
+            a.mult = l->c.residual_mult;
+            a.x_out = x = x == m->x ? l->x_alt : m->x;
+            yw = nullptr;
+        }
+        return a;
+    }
+};
 
 hipError_t layered_output(l2h_model *m) {
     Layered *l = m->lay;
@@ -554,75 +729,114 @@ hipError_t layered_output(l2h_model *m) {
     return k_rows(m->ctx->stream, a, RP_NORM, RE_STORE, m->ctx->prop.multiProcessorCount);
 }
 
+static hipError_t step_latent(l2h_model *m, const LayerDev &L, const LayerRun &run, int cu) {
+    Layered *l = m->lay;
+    hipStream_t s = m->ctx->stream;
+    const LatentShape w = latent_shape(l, L);
+    hipError_t e;
+    RowsArgs q = rows_of(L.uq, l->in, l->lq);
+    q.normw = L.qnorm;
+    q.eps = w.eps;
+    CK(k_rows(s, q, RP_NORM, RE_STORE, cu));
+    CK(k_latent_query(s, w, L.freq, l->lq, L.ukv.w, L.ukv.ld, l->qa, 1, 0, m->ctl, l->in, L.kvnorm, run.kc));
+    CK(k_latent_attend(s, w, l->qa, run.kc, l->part, 1, 0, m->ctl));
+    const int64_t cols = L.joined ? L.o_cols : w.H * w.V;
+    return k_latent_value(s, w, l->part, L.ukv.w, L.ukv.ld, l->in, 0, 1, l->mix, cols, cols, 1);
+}
+
 hipError_t layered_enqueue_token(l2h_model *m) {
     Layered *l = m->lay;
     hipStream_t s = m->ctx->stream;
     const int cu = m->ctx->prop.multiProcessorCount;
     const l2h_layered_config &c = l->c;
     hipError_t e;
-    CK(k_embed(s, m->glob[L2H_TOK_EMB], m->ctl, m->prompt_dev, stream_buf(m, 0), m->rope_cs, 0, 1.0f));
-    for (int i = 0; i < c.n_layers; i++) {
-        LayerDev &L = l->layer[(size_t)i];
+    Stream st(m);
+    CK(k_embed(s, m->glob[L2H_TOK_EMB], m->ctl, m->prompt_dev, st.x, m->rope_cs, 0, 1.0f, c.embed_scale, l->x0));
+    for (const LayerRun &run : l->run) {
+        LayerDev &L = l->layer[(size_t)run.layer];
         const l2h_layer &d = L.d;
-        float *x = stream_buf(m, i);
-        CK(k_rows(s, normed(m, i, L.in, L.norm1, l->in), RP_NORM, RE_STORE, cu));
+        if (run.pass >= 0) {
+            if (st.yw) CK(k_norm_rows(s, st.x, c.width, 1, nullptr, c.norm_eps, l->y, st.yw, c.residual_mult, nullptr, nullptr, 0, 1));
+            st.yw = nullptr;
+            CK(k_stream_add(s, st.x, run.pass ? l->x0 : nullptr, l->loop_step + (int64_t)run.pass * c.width, 1, c.width));
+        }
+        RowsArgs in = st.normed(L.in, L.norm1, l->in);
+        float *x = st.x;
+        const bool early = d.parallel;  // the feed-forward reads the mixer's input
+        if (L.stacked()) {
+            in.glu_from = L.n_plain;
+            in.act = d.ff_act;
+            in.out2 = L.joined ? l->mix + L.o_cols : l->hid;
+            CK(k_rows(s, in, RP_NORM, RE_STORE_GLU, cu));
+        } else {
+            CK(k_rows(s, in, RP_NORM, RE_STORE, cu));
+        }
         RowsArgs o = rows_of(L.o, l->mix, x);
         o.resid = x;
         o.mult = c.residual_mult;
+        int o_pro = RP_PLAIN;
         if (d.mixer == L2H_MIX_ATTENTION) {
-            CK(k_window_step(s, window_shape(l, L), L.freq, l->in, L.kc, L.vc, m->ctl, l->part, l->mix));
-            CK(k_rows(s, o, RP_PLAIN, RE_RESID, cu));
+            CK(k_window_step(s, window_shape(l, L), L.freq, l->in, run.kc, run.vc, m->ctl, l->part, l->mix));
+        } else if (d.mixer == L2H_MIX_LATENT) {
+            CK(step_latent(m, L, run, cu));
         } else {
             const DeltaWeights w = {L.conv, L.rate, L.bias, L.a2.w, L.g2.w, L.a2.ld, L.g2.ld};
-            CK(k_delta_step(s, delta_shape(l, L), w, l->in, L.ring, L.state, m->ctl, l->mix, l->ssq, l->gate));
+            CK(k_delta_step(s, delta_shape(l, L), w, l->in, run.ring, run.state, m->ctl, l->mix, l->ssq, l->gate));
             o.normw = L.mixnorm;
             o.eps = c.norm_eps;
             o.ssq = l->ssq;
             o.gate = l->gate;
             o.hv = d.vdim;
             o.n_split = delta_splits(d.vdim);
-            CK(k_rows(s, o, RP_HEADNORM, RE_RESID, cu));
+            o_pro = RP_HEADNORM;
         }
-        if (d.ff != L2H_FF_NONE) {
+        if (!early || d.ff == L2H_FF_NONE || (L.stacked() && L.joined)) CK(k_rows(s, o, o_pro, RE_RESID, cu));
+        if (d.ff != L2H_FF_NONE && !(L.stacked() && L.joined)) {
             RowsArgs up = rows_of(L.up, x, l->hid), down = rows_of(L.down, l->hid, x);
-            up.normw = L.norm2;
+            up.normw = early ? L.norm1 : L.norm2;
             up.eps = c.norm_eps;
             up.act = d.ff_act;
             down.resid = x;
             down.mult = c.residual_mult;
             if (d.ff == L2H_FF_DENSE) {
-                CK(k_rows(s, up, RP_NORM, RE_ACT, cu));
-                CK(k_rows(s, down, RP_PLAIN, RE_RESID, cu));
+                if (L.joined) up.out = l->mix + L.o_cols;
+                if (!L.stacked()) CK(k_rows(s, up, RP_NORM, d.ff_gated ? RE_GLU : RE_ACT, cu));
+                if (early) CK(k_rows(s, o, o_pro, RE_RESID, cu));
+                if (!L.joined) CK(k_rows(s, down, RP_PLAIN, RE_RESID, cu));
             } else {
                 RowsArgs r = rows_of(L.router, x, l->z);
-                r.normw = L.norm2;
+                r.normw = up.normw;
                 r.eps = c.norm_eps;
-                CK(k_rows(s, r, RP_NORM, RE_STORE, cu));
+                if (!early) CK(k_rows(s, r, RP_NORM, RE_STORE, cu));
                 for (RowsArgs *a : {&up, &down}) {
-                    a->z = l->z;
+                    a->z = early ? l->in + L.off_z : l->z;
+                    a->z_bias = L.router_bias;
                     a->n_experts = d.n_experts;
                     a->top = d.top;
+                    a->route = d.route;
                 }
-                up.rows_each = d.ff_dim;
-                up.n_rows = (int64_t)d.top * d.ff_dim;
+                up.rows_each = L.up_rows();
+                up.n_rows = (int64_t)d.top * L.up_rows();
                 down.rows_each = c.width;
                 down.n_rows = c.width;
-                CK(k_rows(s, up, RP_UP, RE_UP, cu));
+                CK(k_rows(s, up, RP_UP, d.ff_gated ? RE_GLU : RE_UP, cu));
+                if (early) CK(k_rows(s, o, o_pro, RE_RESID, cu));
                 CK(k_rows(s, down, RP_DOWN, RE_RESID, cu));
             }
         }
         if (c.side_dim) {
             RowsArgs g = rows_of(L.side_gate, x, l->se);
             g.act = LACT_GELU_TANH;
-            g.emb = l->side_emb + (int64_t)i * c.side_dim;
+            g.emb = l->side_emb + (int64_t)run.layer * c.side_dim;
             g.emb_ld = (int64_t)c.n_layers * c.side_dim;
             g.ctl = m->ctl;
             g.prompt = m->prompt_dev;
             CK(k_rows(s, g, RP_PLAIN, RE_EMBED, cu));
             CK(k_rows(s, rows_of(L.side_proj, l->se, l->y), RP_PLAIN, RE_STORE, cu));
+            st.yw = L.side_norm;
         }
     }
-    CK(k_rows(s, normed(m, c.n_layers, l->head, l->final_norm, m->logits), RP_NORM, RE_STORE, cu));
+    CK(k_rows(s, st.normed(l->head, l->final_norm, m->logits), RP_NORM, RE_STORE, cu));
     return hipSuccess;
 }
 
@@ -649,10 +863,10 @@ static int prompt_images(l2h_model *m) {
         elems += n * k_tile_image_elems(rows, w->ld);
     };
     for (LayerDev &L : l->layer) {
-        if (L.d.ff == L2H_FF_DENSE) add(&L.up, L.d.ff_dim, 1);
+        if (L.d.ff == L2H_FF_DENSE) add(&L.up, L.up_rows(), 1);
         if (L.d.ff == L2H_FF_EXPERTS) {
-            if (std::min(L.d.ff_dim, l->W()) < L_IMAGE_MIN_ROWS) continue;  // (both or neither)
-            add(&L.up, L.d.ff_dim, L.d.n_experts);
+            if (std::min(L.up_rows(), l->W()) < L_IMAGE_MIN_ROWS) continue;  // (both or neither)
+            add(&L.up, L.up_rows(), L.d.n_experts);
             add(&L.down, l->W(), L.d.n_experts);
         }
     }
@@ -692,16 +906,18 @@ int layered_prefill_buffers(l2h_model *m, int cap, int n_want) {
         l->want_cap = n_want;
     }
     if (l->keep && l->kept_cap < cap) {
-        DA(l->kept, (int64_t)c.n_layers * cap * c.width);
+        DA(l->kept, (int64_t)l->run.size() * cap * c.width);
         l->kept_cap = cap;
     }
     if (l->cap >= cap) return L2H_OK;
     int64_t n_in = 1, ch = 1, g = 1, h = 1, hd = 1, hv = 1, lhv = 64, lra = 64, lrg = 64, hid = 64, ne = 1, slots = 1, up_slots = 1, tiles = 1;
-    int64_t kvt = 0, rec = 0;
+    int64_t kvt = 0, rec = 0, qb = 0, xc = 0, kvx = 0, cq = 0, lat_qa = 0, lat_part = 0;
+    // tokens of a block of latent attention: few where longer prompts go another way
+    const int lat_block = std::min(cap, L_LATENT_BLOCK), kvx_cap = std::min((c.seq_len + 255) / 256 * 256, 2048);
     bool moe = false;
     for (LayerDev &L : l->layer) {
         const l2h_layer &d = L.d;
-        n_in = std::max<int64_t>(n_in, mixer_rows(l, L));
+        n_in = std::max<int64_t>(n_in, L.n_plain);
         hv = std::max<int64_t>(hv, d.n_heads * d.vdim);
         lhv = std::max<int64_t>(lhv, L.o.ld);
         if (d.mixer == L2H_MIX_ATTENTION) {
@@ -710,6 +926,20 @@ int layered_prefill_buffers(l2h_model *m, int cap, int n_want) {
             if (hs && !c.precision) {
                 ch = std::max<int64_t>(ch, d.n_heads * hs);
                 kvt = std::max<int64_t>(kvt, (int64_t)d.n_kv_heads * attention_tiles(l, L, cap) * k_pf_kv_tile_bytes(hs));
+            }
+        } else if (d.mixer == L2H_MIX_LATENT) {
+            const LatentShape w = latent_shape(l, L);
+            const int hs = latent_tile_size(l, d);
+            const int64_t block = hs ? std::min(lat_block, L_LATENT_SMALL) : lat_block;
+            ch = std::max<int64_t>(ch, w.H * w.hq());
+            cq = std::max<int64_t>(cq, L.uq.ld);
+            lat_qa = std::max(lat_qa, block * w.H * w.ld());
+            for (int64_t k = 1; k <= block; k++) lat_part = std::max(lat_part, latent_part_floats(w, k * w.H));
+            if (hs) {
+                qb = std::max<int64_t>(qb, w.H * hs);
+                xc = std::max<int64_t>(xc, L.ukv.ld);
+                kvx = std::max<int64_t>(kvx, L.ukv.rows);
+                kvt = std::max<int64_t>(kvt, (int64_t)w.H * latent_tiles(l) * k_pf_kv_tile_bytes(hs));
             }
         } else {
             ch = std::max<int64_t>(ch, delta_shape(l, L).channels());
@@ -720,7 +950,7 @@ int layered_prefill_buffers(l2h_model *m, int cap, int n_want) {
             rec = std::max(rec, delta_walk_floats(delta_shape(l, L), cap));
             lrg = std::max<int64_t>(lrg, L.g2.ld);
         }
-        if (d.ff == L2H_FF_DENSE) hid = std::max<int64_t>(hid, L.down.ld);
+        if (d.ff == L2H_FF_DENSE && !L.joined) hid = std::max<int64_t>(hid, L.down.ld);
         if (d.ff == L2H_FF_EXPERTS) {
             moe = true;
             ne = std::max<int64_t>(ne, d.n_experts);
@@ -731,6 +961,18 @@ int layered_prefill_buffers(l2h_model *m, int cap, int n_want) {
     }
     if (kvt) DA(l->kvt, kvt);
     if (rec) DA(l->rec, rec);
+    if (cq) {
+        DB(l->cq, cap * cq);
+        DA(l->lat_qa, lat_qa);
+        DA(l->lat_part, lat_part);
+    }
+    if (qb) {
+        DA(l->qb, cap * qb);
+        DA(l->xc, kvx_cap * xc);
+        DA(l->kvx, kvx_cap * kvx);
+        l->kvx_cap = kvx_cap;
+    }
+    if (l->adds_again()) DA(l->X0, (int64_t)cap * c.width);
     DA(l->tok, cap);
     DA(l->X, (int64_t)cap * c.width);
     DA(l->raw, cap * std::max<int64_t>(n_in, c.side_dim));
@@ -805,9 +1047,10 @@ static hipError_t product(l2h_model *m, GemmArgs a, int epi, float *out, int64_t
     return k_gemm(m->ctx->stream, a, m->lay->c.precision, epi);
 }
 static bool image_takes(const LMat &w, int M) { return w.image && M >= L_BIG_MIN_M; }
-static hipError_t to_acts(l2h_model *m, GemmArgs a, int epi, void *out, int64_t lda, const LMat *w = nullptr) {
+static hipError_t to_acts(l2h_model *m, GemmArgs a, int epi, void *out, int64_t lda, const LMat *w = nullptr, int64_t cols = 0) {
     a.outa = out;
     a.lda = lda;
+    a.acols = cols;
     if (w && image_takes(*w, a.M)) {
         a.w = w->image;
         return k_tiles(m->ctx->stream, a, epi);
@@ -815,15 +1058,15 @@ static hipError_t to_acts(l2h_model *m, GemmArgs a, int epi, void *out, int64_t 
     return k_gemm(m->ctx->stream, a, m->lay->c.precision, epi);
 }
 
-static hipError_t prompt_delta(l2h_model *m, LayerDev &L, int M, int pos0) {
+static hipError_t prompt_delta(l2h_model *m, LayerDev &L, const LayerRun &run, int M, int pos0) {
     Layered *l = m->lay;
     hipStream_t s = m->ctx->stream;
     const int prec = l->c.precision;
     const DeltaShape d = delta_shape(l, L);
-    const int64_t ldr = d.n_in(), hd = d.H * d.D, hv = d.H * d.V;
+    const int64_t ldr = L.n_plain, hd = d.H * d.D, hv = d.H * d.V;
     hipError_t e;
-    CK(k_delta_prepare(s, d, L.conv, l->raw, ldr, L.ring, M, pos0, l->qkv, l->kq, l->beta, l->fa, L.a2.ld, l->fg, L.g2.ld, prec));
-    CK(k_delta_ring(s, d, l->raw, ldr, L.ring, M, pos0));
+    CK(k_delta_prepare(s, d, L.conv, l->raw, ldr, run.ring, M, pos0, l->qkv, l->kq, l->beta, l->fa, L.a2.ld, l->fg, L.g2.ld, prec));
+    CK(k_delta_ring(s, d, l->raw, ldr, run.ring, M, pos0));
     GemmArgs a = gemm_of(L.a2, l->fa, M);
     a.outf = l->lg;
     a.ldo = hd;
@@ -833,18 +1076,18 @@ static hipError_t prompt_delta(l2h_model *m, LayerDev &L, int M, int pos0) {
     CK(k_gemm(s, a, prec, GE_DECAY));
     CK(product(m, gemm_of(L.g2, l->fg, M), GE_SIGMOID, l->gt, hv, 1.0f));
     if (M >= L_DELTA_WALK_MIN)
-        CK(k_delta_walk(s, d, l->qkv, l->beta, l->lg, L.state, M, pos0, l->rec, l->ob));
+        CK(k_delta_walk(s, d, l->qkv, l->beta, l->lg, run.state, M, pos0, l->rec, l->ob));
     else
-        CK(k_delta_scan(s, d, l->qkv, l->kq, l->beta, l->lg, L.state, M, pos0, l->ob));
+        CK(k_delta_scan(s, d, l->qkv, l->kq, l->beta, l->lg, run.state, M, pos0, l->ob));
     CK(k_head_norm_rows(s, l->ob, l->gt, L.mixnorm, M, d.H, d.V, d.eps, l->ao, L.o.ld, prec));
     return hipSuccess;
 }
 
-static hipError_t prompt_attention(l2h_model *m, LayerDev &L, int M, int pos0) {
+static hipError_t prompt_attention(l2h_model *m, LayerDev &L, const LayerRun &run, int M, int pos0) {
     Layered *l = m->lay;
     hipStream_t s = m->ctx->stream;
     const WindowShape w = window_shape(l, L);
-    const int64_t ldr = w.n_in();
+    const int64_t ldr = L.n_plain;
     const int hs = attention_tile_size(L.d);
     hipError_t e;
     if (hs && l->c.precision == 0) {
@@ -858,13 +1101,53 @@ static hipError_t prompt_attention(l2h_model *m, LayerDev &L, int M, int pos0) {
         win.ldg = ldr;
         win.ldo = L.o.ld;
         const int n_tiles = (pos0 + M + 31) / 32 - win.tile0, cap = attention_tiles(l, L, l->cap);
-        CK(k_window_prepare(s, w, L.freq, l->raw, ldr, L.kc, L.vc, M, pos0, nullptr, qb, hs));
-        CK(k_pf_kv_tiles(s, L.kc, L.vc, l->kvt, n_tiles, cap, hs, w.G, w.seq_len, win.tile0, w.Dp(), w.V));
+        CK(k_window_prepare(s, w, L.freq, l->raw, ldr, run.kc, run.vc, M, pos0, nullptr, qb, hs));
+        CK(k_pf_kv_tiles(s, run.kc, run.vc, l->kvt, n_tiles, cap, hs, w.G, w.seq_len, win.tile0, w.Dp(), w.V));
         return k_pf_attention(s, qb, (uint16_t *)l->ao, l->kvt, cap, M, pos0, hs, w.H, w.G, w.H * hs, &win);
     }
-    CK(k_window_prepare(s, w, L.freq, l->raw, ldr, L.kc, L.vc, M, pos0, l->qkv, nullptr, 0));
-    CK(k_window_rows(s, w, l->qkv, l->raw, ldr, L.kc, L.vc, M, pos0, l->ao, L.o.ld, l->c.precision));
+    CK(k_window_prepare(s, w, L.freq, l->raw, ldr, run.kc, run.vc, M, pos0, l->qkv, nullptr, 0));
+    CK(k_window_rows(s, w, l->qkv, l->raw, ldr, run.kc, run.vc, M, pos0, l->ao, L.o.ld, l->c.precision));
     return hipSuccess;
+}
+
+static hipError_t prompt_latent(l2h_model *m, LayerDev &L, const LayerRun &run, int M, int pos0) {
+    Layered *l = m->lay;
+    hipStream_t s = m->ctx->stream;
+    const LatentShape w = latent_shape(l, L);
+    const int64_t ldr = L.n_plain, ldq = w.H * w.hq(), ldkv = L.ukv.rows, lda = L.o.ld;
+    const int prec = l->c.precision, hs = latent_tile_size(l, L.d);
+    hipError_t e;
+    CK(k_latent_prepare(s, w, L.qnorm, L.kvnorm, L.freq, l->raw, ldr, run.kc, M, pos0, l->cq, L.uq.ld, prec));
+    CK(product(m, gemm_of(L.uq, l->cq, M), GE_STORE, l->qkv, ldq, 1.0f));
+    if (!hs || M <= L_LATENT_SMALL) {
+        const int block = std::min(std::min(l->cap, L_LATENT_BLOCK), hs ? L_LATENT_SMALL : M);
+        for (int m0 = 0; m0 < M; m0 += block) {
+            const int n = std::min(block, M - m0);
+            void *out = (char *)l->ao + (int64_t)m0 * lda * l->asize();
+            CK(k_latent_query(s, w, L.freq, l->qkv + m0 * ldq, L.ukv.w, L.ukv.ld, l->lat_qa, n, pos0 + m0, nullptr, nullptr, nullptr, nullptr));
+            CK(k_latent_attend(s, w, l->lat_qa, run.kc, l->lat_part, n, pos0 + m0, nullptr));
+            CK(k_latent_value(s, w, l->lat_part, L.ukv.w, L.ukv.ld, l->raw + m0 * ldr, ldr, n, out, lda, L.o_cols, prec));
+        }
+        return hipSuccess;
+    }
+    CK(k_latent_heads(s, w, L.freq, l->qkv, l->qb, hs, M, pos0));
+    const int tiles = latent_tiles(l);
+    for (int p = 0; p < pos0 + M; p += l->kvx_cap) {  // the heads' own keys and values, from the cached latents
+        const int n = std::min(l->kvx_cap, pos0 + M - p);
+        CK(k_latent_rows(s, w, run.kc, p, n, l->xc, L.ukv.ld));
+        CK(product(m, gemm_of(L.ukv, l->xc, n), GE_STORE, l->kvx, ldkv, 1.0f));
+        CK(k_pf_row_tiles(s, l->kvx, ldkv, run.kc + w.Cp(), w.ld(), w.R, l->kvt, p, n, tiles, hs, w.H, w.D, w.V));
+    }
+    PfWindow win;
+    win.window = l->c.seq_len;  // (every key)
+    win.vdim = w.V;
+    win.scale = w.scale;
+    win.gate = w.gated ? l->raw + w.off_g() : nullptr;
+    win.gate_each = 1;
+    win.ldg = ldr;
+    win.ldo = lda;
+    win.cols = L.o_cols;
+    return k_pf_attention(s, l->qb, (uint16_t *)l->ao, l->kvt, tiles, M, pos0, hs, w.H, w.H, w.H * hs, &win);
 }
 
 static hipError_t prompt_experts(l2h_model *m, LayerDev &L, int M) {
@@ -873,8 +1156,10 @@ static hipError_t prompt_experts(l2h_model *m, LayerDev &L, int M) {
     const l2h_layer &d = L.d;
     const int prec = l->c.precision;
     hipError_t e;
-    CK(product(m, gemm_of(L.router, l->xn, M), GE_STORE, l->zb, d.n_experts, 1.0f));
-    CK(k_route(s, l->zb, M, d.n_experts, d.top, l->choice, l->score));
+    if (!d.parallel) CK(product(m, gemm_of(L.router, l->xn, M), GE_STORE, l->zb, d.n_experts, 1.0f));
+    // (a parallel layer's logits are among the products of the mixer's input)
+    CK(k_route(s, d.parallel ? l->raw + L.off_z : l->zb, d.parallel ? L.n_plain : d.n_experts, L.router_bias, M, d.n_experts, d.top, d.route,
+               l->choice, l->score));
     const bool image = image_takes(L.up, M) && image_takes(L.down, M);
     const int rows = image ? L_IMAGE_TILE : L_GEMM_TILE;
     CK(k_group(s, l->choice, l->score, M, d.n_experts, d.top, l->slot_row, l->slot_scale, l->slot_of, l->tiles, l->n_tiles, rows));
@@ -885,19 +1170,21 @@ static hipError_t prompt_experts(l2h_model *m, LayerDev &L, int M) {
         a->n_tiles = l->n_tiles;
         a->max_tiles = max_tiles;
     }
-    up.n_rows = d.ff_dim;
-    up.expert_stride = (int64_t)d.ff_dim * L.up.ld;
+    const int epi = d.ff_gated ? GE_GLU : GE_UP;
+    up.n_rows = L.up_rows();
+    up.expert_stride = (int64_t)L.up_rows() * L.up.ld;
     up.gather = l->slot_row;
     up.row_scale = l->slot_scale;
+    up.scale_in = d.route == L2H_ROUTE_SIGMOID_IN;
     up.act = d.ff_act;
     up.outa = l->hb;
     up.lda = L.down.ld;
     if (image) {
         up.w = L.up.image;
         up.expert_stride = L.up.image_stride;
-        CK(k_tiles(s, up, GE_UP));
+        CK(k_tiles(s, up, epi));
     } else {
-        CK(k_gemm(s, up, prec, GE_UP));
+        CK(k_gemm(s, up, prec, epi));
     }
     down.n_rows = l->W();
     down.expert_stride = (int64_t)l->W() * L.down.ld;
@@ -920,26 +1207,40 @@ hipError_t layered_prefill_chunk(l2h_model *m, int M, int pos0) {
     const int W = c.width, ldw = l->ldw(), prec = c.precision;
     const float mult = c.residual_mult, eps = c.norm_eps;
     hipError_t e;
-    CK(k_pf_embed(s, m->glob[L2H_TOK_EMB], l->tok, l->X, M));
+    CK(k_pf_embed(s, m->glob[L2H_TOK_EMB], l->tok, l->X, M, c.embed_scale, l->X0));
     const float *py = nullptr, *pyw = nullptr;  // per-token update that waits for the next reader of the residual stream
-    auto keep = [&](int layer) -> hipError_t {
-        if (!l->keep || layer < 0) return hipSuccess;
-        return hipMemcpyAsync(l->kept + ((int64_t)layer * l->kept_cap) * W, l->X, (size_t)M * W * 4, hipMemcpyDeviceToDevice, s);
+    auto keep = [&](int r) -> hipError_t {
+        if (!l->keep || r < 0) return hipSuccess;
+        return hipMemcpyAsync(l->kept + ((int64_t)r * l->kept_cap) * W, l->X, (size_t)M * W * 4, hipMemcpyDeviceToDevice, s);
     };
-    for (int i = 0; i < c.n_layers; i++) {
-        LayerDev &L = l->layer[(size_t)i];
+    for (int r = 0; r < (int)l->run.size(); r++) {
+        const LayerRun &run = l->run[(size_t)r];
+        LayerDev &L = l->layer[(size_t)run.layer];
         const l2h_layer &d = L.d;
+        bool kept = false;
+        if (run.pass >= 0) {
+            if (py) CK(k_norm_rows(s, l->X, W, M, nullptr, eps, py, pyw, mult, nullptr, nullptr, 0, prec));
+            py = nullptr;
+            CK(keep(r - 1));
+            kept = true;
+            CK(k_stream_add(s, l->X, run.pass ? l->X0 : nullptr, l->loop_step + (int64_t)run.pass * W, M, W));
+        }
         CK(k_norm_rows(s, l->X, W, M, L.norm1, eps, py, pyw, mult, nullptr, l->xn, ldw, prec));
-        CK(keep(i - 1));
-        CK(product(m, gemm_of(L.in, l->xn, M), GE_STORE, l->raw, L.in.rows, 1.0f));
-        CK(d.mixer == L2H_MIX_ATTENTION ? prompt_attention(m, L, M, pos0) : prompt_delta(m, L, M, pos0));
+        py = nullptr;
+        if (!kept) CK(keep(r - 1));
+        CK(product(m, gemm_of(mat_rows(L.in, 0, L.n_plain), l->xn, M), GE_STORE, l->raw, L.n_plain, 1.0f));
+        CK(d.mixer == L2H_MIX_ATTENTION ? prompt_attention(m, L, run, M, pos0)
+           : d.mixer == L2H_MIX_LATENT  ? prompt_latent(m, L, run, M, pos0)
+                                        : prompt_delta(m, L, run, M, pos0));
+        GemmArgs up = gemm_of(L.up, l->xn, M);
+        up.act = d.ff_act;
+        const int up_epi = d.ff_gated ? GE_GLU : GE_ACT;
+        if (L.joined) CK(to_acts(m, up, up_epi, (char *)l->ao + (int64_t)L.o_cols * l->asize(), L.o.ld, &L.up, L.o.ld - L.o_cols));
         CK(product(m, gemm_of(L.o, l->ao, M), GE_RESID, l->X, W, mult));
-        if (d.ff != L2H_FF_NONE) {
-            CK(k_norm_rows(s, l->X, W, M, L.norm2, eps, nullptr, nullptr, mult, nullptr, l->xn, ldw, prec));
+        if (d.ff != L2H_FF_NONE && !L.joined) {
+            if (!d.parallel) CK(k_norm_rows(s, l->X, W, M, L.norm2, eps, nullptr, nullptr, mult, nullptr, l->xn, ldw, prec));
             if (d.ff == L2H_FF_DENSE) {
-                GemmArgs up = gemm_of(L.up, l->xn, M);
-                up.act = d.ff_act;
-                CK(to_acts(m, up, GE_ACT, l->hb, L.down.ld, &L.up));
+                CK(to_acts(m, up, up_epi, l->hb, L.down.ld, &L.up));
                 CK(product(m, gemm_of(L.down, l->hb, M), GE_RESID, l->X, W, mult));
             } else {
                 CK(prompt_experts(m, L, M));
@@ -949,7 +1250,7 @@ hipError_t layered_prefill_chunk(l2h_model *m, int M, int pos0) {
             CK(k_norm_rows(s, l->X, W, M, nullptr, eps, nullptr, nullptr, mult, nullptr, l->xn, ldw, prec));
             GemmArgs g = gemm_of(L.side_gate, l->xn, M);
             g.act = LACT_GELU_TANH;
-            g.emb = l->side_emb + (int64_t)i * c.side_dim;
+            g.emb = l->side_emb + (int64_t)run.layer * c.side_dim;
             g.emb_ld = (int64_t)c.n_layers * c.side_dim;
             g.tokens = l->tok;
             if (library_takes(m, g)) {
@@ -964,7 +1265,7 @@ hipError_t layered_prefill_chunk(l2h_model *m, int M, int pos0) {
         }
     }
     if (py) CK(k_norm_rows(s, l->X, W, M, nullptr, eps, py, pyw, mult, nullptr, nullptr, 0, prec));
-    CK(keep(c.n_layers - 1));
+    CK(keep((int)l->run.size() - 1));
     l->kept_n = M;
     // the last position becomes the decode state's residual stream
     return hipMemcpyAsync(m->x, l->X + (int64_t)(M - 1) * W, (size_t)W * 4, hipMemcpyDeviceToDevice, s);
@@ -994,7 +1295,7 @@ extern "C" int l2h_layered_keep(l2h_model *m, int on) {
 extern "C" int l2h_layered_kept(l2h_model *m, int layer, float *host, int64_t n) {
     if (!m || !m->lay || !host) return L2H_EINVAL;
     Layered *l = m->lay;
-    if (!l->kept || layer < 0 || layer >= l->c.n_layers || n != (int64_t)l->kept_n * l->c.width)
+    if (!l->kept || layer < 0 || layer >= (int)l->run.size() || n != (int64_t)l->kept_n * l->c.width)
         return set_err(m->ctx, L2H_EINVAL, "kept residual stream: layer %d, %lld floats (holds %d positions)", layer, (long long)n, l->kept_n);
     HIPCHK(m->ctx, hipStreamSynchronize(m->ctx->stream));
     HIPCHK(m->ctx, hipMemcpy(host, l->kept + (int64_t)layer * l->kept_cap * l->c.width, (size_t)n * 4, hipMemcpyDeviceToHost));

@@ -36,6 +36,8 @@ __device__ __forceinline__ float l_act(int act, float z) {
         const float r = fmaxf(z, 0.0f);
         return r * r;
     }
+    if (act == LACT_RELU) return fmaxf(z, 0.0f);
+    if (act == LACT_SILU) return l_silu(z);
     if (act == LACT_GELU_TANH) return 0.5f * z * (1.0f + tanhf(0.797884560802865356f * fmaf(0.044715f * z * z, z, z)));
     return 0.5f * z * (1.0f + erff(z * 0.707106781186547524f));
 }
@@ -87,14 +89,16 @@ __device__ __forceinline__ int l_step_token(const DecodeCtl *ctl, const int32_t 
     return ctl->step < ctl->n_prompt ? prompt[ctl->step] : ctl->last_argmax;
 }
 
-// Rotation of the pairs (2 i, 2 i + 1), i < rot / 2, of one head at `pos` and division by the head's root mean square, by
-// one wavefront.  src and dst hold D elements.
-__device__ __forceinline__ void l_rotate_norm(const float *src, float *dst, int D, int rot, const float *freq, int pos, int norm,
-                                              float eps, int lane) {
+// Rotation of the pairs (2 i, 2 i + 1), or with `half` (i, i + rot / 2), i < rot / 2, of one head at `pos` and division by the
+// head's root mean square, by one wavefront.  src and dst hold D elements.
+__device__ __forceinline__ void l_rotate_norm(const float *src, float *dst, int D, int rot, int half, const float *freq, int pos,
+                                              int norm, float eps, int lane) {
     float ss = 0.0f;
     for (int p = lane; 2 * p < D; p += 64) {
-        float a = src[2 * p], b = 2 * p + 1 < D ? src[2 * p + 1] : 0.0f;
-        if (2 * p < rot) {
+        const bool turned = 2 * p < rot, apart = half && turned;
+        const int ia = apart ? p : 2 * p, ib = apart ? p + rot / 2 : 2 * p + 1;
+        float a = src[ia], b = ib < D ? src[ib] : 0.0f;
+        if (turned) {
             const float ang = (float)pos * freq[p];
             const float c = cosf(ang), s = sinf(ang), u = a, v = b;
             a = u * c - v * s;
@@ -102,13 +106,44 @@ __device__ __forceinline__ void l_rotate_norm(const float *src, float *dst, int 
         }
         ss = fmaf(a, a, ss);
         ss = fmaf(b, b, ss);
-        dst[2 * p] = a;
-        if (2 * p + 1 < D) dst[2 * p + 1] = b;
+        dst[ia] = a;
+        if (ib < D) dst[ib] = b;
     }
     if (!norm) return;
     const float r = 1.0f / sqrtf(l_wave_sum(ss) / (float)D + eps);
     for (int p = lane; 2 * p < D; p += 64) {
-        dst[2 * p] *= r;
-        if (2 * p + 1 < D) dst[2 * p + 1] *= r;
+        const bool apart = half && 2 * p < rot;
+        const int ia = apart ? p : 2 * p, ib = apart ? p + rot / 2 : 2 * p + 1;
+        dst[ia] *= r;
+        if (ib < D) dst[ib] *= r;
+    }
+}
+
+// Choice of experts by one workgroup: an expert's place among all by its logit is the number of larger ones (the lower index
+// first among equals); sel[place], score[place] for the first `top` places.  zs: LDS for E logits; sel and score are LDS or
+// global memory of the workgroup's own.
+__device__ __forceinline__ void l_route(const float *z, const float *bias, int E, int top, int kind, float *zs, int *sel, float *score) {
+    const int t = threadIdx.x, nt = blockDim.x;
+    for (int e = t; e < E; e += nt) zs[e] = z[e] + (bias ? bias[e] : 0.0f);
+    for (int k = t; k < top; k += nt) sel[k] = 0, score[k] = 0.0f;  // (a place that no number takes, with NaN among them, stays defined)
+    __syncthreads();
+    for (int e = t; e < E; e += nt) {
+        const float v = zs[e];
+        int rank = 0;
+#pragma unroll 8
+        for (int o = 0; o < E; o++) rank += (zs[o] > v || (zs[o] == v && o < e)) ? 1 : 0;
+        if (rank < top) {
+            sel[rank] = e;
+            score[rank] = kind == LROUTE_SIGMOID_IN ? l_sigmoid(v) : v;
+        }
+    }
+    __syncthreads();
+    if (kind == LROUTE_SOFTMAX_OUT) {
+        if (t < 64) {  // (top <= 64)
+            const float v = t < top ? score[t] : -INFINITY, m = wave_max_f32(v);
+            const float p = t < top ? expf(v - m) : 0.0f, sum = l_wave_sum(p);
+            if (t < top) score[t] = p / sum;
+        }
+        __syncthreads();
     }
 }

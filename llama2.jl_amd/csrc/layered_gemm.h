@@ -29,8 +29,21 @@ __device__ __forceinline__ void gemm_store4(const GemmArgs &a, int64_t m, int64_
             if (L + e >= a.n_rows) break;
             o[e] = value(e, EPI == GE_RESID ? o[e] : 0.0f);
         }
+    } else if (EPI == GE_GLU) {
+        // (n_rows even: pairs are whole)
+        const int64_t i = L >> 1;
+        if (i >= a.acols) return;
+        float o[2] = {0.0f, 0.0f};
+        const float f = a.row_scale ? a.row_scale[m] : 1.0f, fi = a.scale_in ? f : 1.0f, fo = a.scale_in ? 1.0f : f;
+#pragma unroll
+        for (int e = 0; e < 2; e++)
+            if (L + 2 * e < a.n_rows) o[e] = fo * l_act_rounded<PREC>(a.act, fi * v[2 * e]) * (fi * v[2 * e + 1]);
+        if (PREC)
+            *(float2 *)((float *)a.outa + m * a.lda + i) = make_float2(o[0], o[1]);
+        else
+            *(uint32_t *)((uint16_t *)a.outa + m * a.lda + i) = l_pack_bf16(o[0], o[1]);
     } else {
-        if (L >= a.lda) return;  // (lda a multiple of 64: whole groups of four)
+        if (L >= a.acols) return;  // (acols a multiple of 64: whole groups of four)
 #pragma unroll
         for (int e = 0; e < 4; e++) {
             if (L + e >= a.n_rows) {
@@ -38,7 +51,7 @@ __device__ __forceinline__ void gemm_store4(const GemmArgs &a, int64_t m, int64_
                 continue;
             }
             if (EPI == GE_UP)
-                v[e] = l_act_rounded<PREC>(a.act, a.row_scale[m] * v[e]);
+                v[e] = a.scale_in ? l_act_rounded<PREC>(a.act, a.row_scale[m] * v[e]) : a.row_scale[m] * l_act_rounded<PREC>(a.act, v[e]);
             else if (EPI == GE_EMBED)
                 v[e] = l_act_rounded<PREC>(a.act, v[e]) * l_bf16(a.emb[(int64_t)a.tokens[m] * a.emb_ld + L + e]);
             else

@@ -10,18 +10,27 @@ from .safetensors import read_safetensors
 from .tokenizer import IdTokenizer
 
 
-def _vudelix(raw, tensors, seq_len, precision):
+def _array(tensors):
     def array(name):
         if name not in tensors:
             raise layered.ConfigError("model.safetensors has no tensor %r" % name)
         return tensors[name][1]
+    return array
 
+
+def _vudelix(raw, tensors, seq_len, precision):
+    array = _array(tensors)
     config = layered.vudelix_config(raw, lambda name: array(name).shape, seq_len, precision)
     return config, layered.vudelix_weights(config, array)
 
 
+def _lezepel(raw, tensors, seq_len, precision):
+    config = layered.lezepel_config(raw, seq_len, precision)
+    return config, layered.lezepel_weights(config, _array(tensors))
+
+
 # architecture -> (config.json, tensors, seq_len, precision) -> (config, weights)
-ARCHITECTURES = {"Vudelix": _vudelix}
+ARCHITECTURES = {"Vudelix": _vudelix, "Lezepel": _lezepel}
 
 
 def load_model(path, seq_len=4096, precision="bfloat16"):

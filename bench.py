@@ -64,7 +64,7 @@ WORKLOADS = {
 }
 
 # layered models beside a Llama model of equal size (llama2.jl_amd/bench_layered.py)
-LAYERED_WORKLOADS = ["vudelix-2k", "vudelix-4k", "vudelix-tiny"]
+LAYERED_WORKLOADS = ["vudelix-2k", "vudelix-4k", "vudelix-tiny", "lezepel-2k", "lezepel-4k", "lezepel-tiny"]
 
 
 def log(*a):

@@ -217,8 +217,11 @@ struct LatentShape {
 #define L_LATENT_MAX_RANK 1024
 #define L_LATENT_BLOCK 128  // tokens whose queries go through k_up^T at a time
 #define L_LATENT_SMALL 16   // up to so many tokens of a prompt go that way, more through their heads' own keys and values
+#define L_LATENT_SPLITS 128
 // workgroups that share the keys of one block of 16 (token, head) columns
-static inline int latent_splits(int64_t cols) { return (int)std::min<int64_t>(64, std::max<int64_t>(1, 512 / ((cols + 15) / 16))); }
+static inline int latent_splits(int64_t cols) {
+    return (int)std::min<int64_t>(L_LATENT_SPLITS, std::max<int64_t>(1, 512 / ((cols + 15) / 16)));
+}
 static inline int64_t latent_part_floats(const LatentShape &w, int64_t cols) { return cols * latent_splits(cols) * (w.Cp() + 4); }
 // raw[M][ldr] -> cache rows pos0 .., and the normed query latent as activations cq[M][lcq]
 hipError_t k_latent_prepare(hipStream_t s, const LatentShape &w, const float *qnorm, const float *kvnorm, const float *freq,

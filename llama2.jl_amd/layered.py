@@ -385,3 +385,7 @@ def lezepel_shapes(config):
             else:
                 out[name] = (W, s.ff_dim) if parts[-1] == "down" else (s.ff_dim, W)
     return out
+
+
+# architecture -> (shapes, weights): a model of a given configuration from its tensors by name
+DESIGNS = {"Vudelix": (vudelix_shapes, vudelix_weights), "Lezepel": (lezepel_shapes, lezepel_weights)}

@@ -149,7 +149,8 @@ def layered_model(config, seed=20240607):
             return p[at:at + n].reshape(ne1, ne0)
         return np.resize(np.roll(p, -int(rng.integers(0, p.size))), (ne1, ne0))
 
-    shapes = layered.vudelix_shapes(config)
+    shapes_of, weights_of = layered.DESIGNS[config.architecture]
+    shapes = shapes_of(config)
 
     def tensor(name):
         last, shape = name.split(".")[-1], shapes[name]
@@ -159,6 +160,10 @@ def layered_model(config, seed=20240607):
             return np.full(shape, -3.0, np.float32)
         if last == "dt_bias":
             return np.full(shape, -2.0, np.float32)
+        if len(shape) == 1:
+            return np.zeros(shape, np.float32)
+        if last == "step":
+            return bits(rng.standard_normal(shape))
         return matrix(*shape)
 
-    return LanguageModel(config, IdTokenizer(config.vocab_size), layered.vudelix_weights(config, tensor))
+    return LanguageModel(config, IdTokenizer(config.vocab_size), weights_of(config, tensor))

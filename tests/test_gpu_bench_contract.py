@@ -49,3 +49,11 @@ def test_layered_workload():
     assert d["steps"] == 16 and d["unit"] == "tok/s" and d["value"] > 0 and d["config"]["workload"] == "vudelix-tiny"
     assert d["prefill"]["tok_s"] > 0 and d["decode"]["bytes"] > 0
     assert {"kernel per phase", "automatic"} <= set(d["beside"])
+
+
+def test_latent_workload():
+    rc, out, err = _run("--workload", "lezepel-tiny", "--steps", "16", "--warmup", "4", "--repeats", "2")
+    assert rc == 0, err[-2000:]
+    d = json.loads([l for l in out.splitlines() if l.startswith("{")][0])
+    assert d["config"]["workload"] == "lezepel-tiny" and d["config"]["layer_runs"] == 8 and d["value"] > 0
+    assert {"Vudelix", "kernel per phase", "automatic"} <= set(d["beside"])

@@ -88,3 +88,16 @@ def test_model_folder_reader(pkg, tmp_path):
     r["loop"] = None
     (d / "config.json").write_text(json.dumps(r))
     assert pkg.load_model(str(d)).config.runs == [0, 1, 2, 3]
+
+
+def test_work_of_the_bench_models(pkg):
+    from llama2_jl_amd import bench_layered, layered
+    cfg, _ = bench_layered.config("lezepel-tiny")
+    by, fl = bench_layered.work(cfg, 64)
+    shapes = layered.lezepel_shapes(cfg)
+    mats = np.prod(shapes["head"])
+    for i in cfg.runs:  # a looped layer's weights are read in every pass
+        for n, s in shapes.items():
+            if n.startswith("l%d." % i) and len(s) == 2:
+                mats += np.prod(s) / (4 if ".mlp.e" in n else 1)  # two experts of eight are read
+    assert by == 2 * mats + 8 * 4 * 64 * (128 + 64) and fl > 2 * 64 * (mats - np.prod(shapes["head"]))
